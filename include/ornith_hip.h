@@ -360,6 +360,9 @@ ORNITH_API int ornith_gdn_step(ornith_ctx* ctx, const void* d_conv_state, const 
  * inv_freq_i = theta^(-i/(dims/2)), computed in double on the host and uploaded. */
 ORNITH_API int ornith_rope_table(ornith_ctx* ctx, int npos, int dims, double theta, float* d_cos,
                                  float* d_sin);
+/* the same with every frequency divided by `factor` (linear position scaling) */
+ORNITH_API int ornith_rope_table_scaled(ornith_ctx* ctx, int npos, int dims, double theta, double factor,
+                                        float* d_cos, float* d_sin);
 /* Attention::forward up to the cache write (src/model/qwen3_5.rs:439-463): per-head
  * rms_norm of q and k (weights [hd]), partial RoPE at position offset + t, append of
  * K and V at rows [offset, offset+T) of the caches bf16 [Hkv, cap, hd]
@@ -519,6 +522,23 @@ ORNITH_API int ornith_model_load(ornith_ctx* ctx, const ornith_weights* ws,
  * receives num_nextn_predict_layers. Host only. */
 ORNITH_API int ornith_text_config_load(const char* model_dir, ornith_text_config* out,
                                        int* mtp_layers);
+/* The model registry: config.json's "architecture" names the design ("Pigodra": mLSTM and
+ * differential-attention layers over a 32-bit residual stream; no such key: the Qwen3.5 keys of
+ * ornith_text_config_load). act_dtype: ORNITH_BF16, or ORNITH_F32 for activations, products and
+ * KV rows in 32-bit where the design runs so (ORNITH_ERR_UNSUPPORTED otherwise). load_json takes
+ * the text of a config.json (for a store filled with ornith_weights_put). The store must outlive
+ * the model. */
+ORNITH_API int ornith_model_open(ornith_ctx* ctx, const ornith_weights* ws, const char* model_dir, int act_dtype,
+                                 ornith_model** out);
+ORNITH_API int ornith_model_load_json(ornith_ctx* ctx, const ornith_weights* ws, const char* config_json, size_t len,
+                                      int act_dtype, ornith_model** out);
+typedef struct ornith_model_info {
+  int hidden_size, vocab_size, num_layers;
+  int act_dtype; /* element type of the hidden rows ornith_model_forward writes */
+  int max_rows;
+  char design[32];
+} ornith_model_info;
+ORNITH_API int ornith_model_describe(const ornith_model* m, ornith_model_info* out);
 ORNITH_API int ornith_model_destroy(ornith_model* m);
 /* Rows one forward call may carry (default 16: decode, verify, short prompt chunks). The
  * reference prefills in chunks of prefill_step_size (2048, src/generate.rs:90-136); raise
@@ -549,7 +569,8 @@ ORNITH_API int ornith_caches_reset(ornith_caches* c);
 ORNITH_API int ornith_caches_destroy(ornith_caches* c);
 ORNITH_API int ornith_caches_offset(const ornith_caches* c, int* offset_out);
 /* TextModel::forward_hidden (capture = 0) / forward_capture (capture = 1): T tokens
- * (device u32) through the trunk; writes the post-norm hidden rows bf16 [T, H] and
+ * (device u32) through the trunk; writes the post-norm hidden rows (bf16 [T, H]; f32 for a model
+ * opened in 32-bit) and
  * advances the caches by T. With capture, T <= max_window and every gated-delta layer
  * keeps a state snapshot per token so ornith_model_rewind can take rows back. */
 ORNITH_API int ornith_model_forward(ornith_model* m, ornith_caches* c, const uint32_t* d_tokens, int T,
@@ -559,6 +580,8 @@ ORNITH_API int ornith_model_forward(ornith_model* m, ornith_caches* c, const uin
 ORNITH_API int ornith_model_rewind(ornith_model* m, ornith_caches* c, int keep);
 /* lm_head.matmul: hidden bf16 [T, H] -> logits bf16 [T, vocab]. */
 ORNITH_API int ornith_model_logits(ornith_model* m, const void* d_hidden, int T, void* d_logits);
+/* the same head with its sums stored in 32-bit, f32 [T, vocab] (designs with a dense bf16 head) */
+ORNITH_API int ornith_model_logits_f32(ornith_model* m, const void* d_hidden, int T, float* d_logits);
 
 /* ---- FR-Spec: FrSpec (src/frspec.rs:38-158) ----------------------------------------- */
 typedef struct ornith_frspec ornith_frspec;

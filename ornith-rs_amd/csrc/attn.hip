@@ -647,29 +647,6 @@ __global__ __launch_bounds__(HD) void sdpa_merge_kernel(SdpaArgs p) {
 
 extern "C" {
 
-int ornith_rope_table(ornith_ctx* ctx, int npos, int dims, double theta, float* d_cos,
-                      float* d_sin) {
-  ORN_REQUIRE(ctx && d_cos && d_sin, "rope_table: null argument");
-  ORN_REQUIRE(npos >= 1 && dims >= 2 && dims % 2 == 0 && theta > 0, "rope_table: npos=%d dims=%d",
-              npos, dims);
-  const int half = dims / 2;
-  float* hc = (float*)malloc(sizeof(float) * (size_t)npos * half * 2);
-  if (!hc) return ornith_fail(ORNITH_ERR_INVALID, "rope_table: out of host memory");
-  float* hs = hc + (size_t)npos * half;
-  for (int i = 0; i < half; ++i) {
-    const double inv_freq = pow(theta, -(double)i / (double)half);
-    for (int pos = 0; pos < npos; ++pos) {
-      const double ang = (double)pos * inv_freq;
-      hc[(size_t)pos * half + i] = (float)cos(ang);
-      hs[(size_t)pos * half + i] = (float)sin(ang);
-    }
-  }
-  int rc = ornith_upload(ctx, d_cos, hc, sizeof(float) * (size_t)npos * half);
-  if (!rc) rc = ornith_upload(ctx, d_sin, hs, sizeof(float) * (size_t)npos * half);
-  free(hc);
-  return rc;
-}
-
 static int prep_args(ornith_ctx* ctx, const void* d_qg, const void* d_kx, const void* d_vx, const void* d_q_norm_w,
                      const void* d_k_norm_w, int T, int Hq, int Hkv, int hd, int rope_dims, float eps,
                      const float* d_cos, const float* d_sin, int table_npos, int offset, const int* d_offset, int cap,

@@ -1,5 +1,5 @@
-// Host-side model objects: the named-tensor store, the trunk, the MTP head, the
-// caches and the FR-Spec head. Mirrors WeightStore (/root/reference/src/weights.rs),
+// Host-side model objects: the named-tensor store, the designs and their layers, the MTP
+// head, the caches and the FR-Spec head. Mirrors WeightStore (/root/reference/src/weights.rs),
 // TextModel / DecoderLayer / GatedDeltaNet / Attention
 // (/root/reference/src/model/qwen3_5.rs), MtpHead (/root/reference/src/model/mtp.rs),
 // KvCache / GdnCache (/root/reference/src/model/cache.rs) and FrSpec
@@ -41,6 +41,11 @@ struct QuantTable {
   }
 };
 int quant_table_load(const std::string& model_dir, QuantTable* qt);
+
+namespace orn_json {
+struct JVal;
+}
+int text_config_from(const orn_json::JVal& cfg, ornith_text_config* c, int* mtp_layers);
 
 struct ornith_weights_files;  // the mapped shards behind a store opened from a directory
 struct ornith_weights;
@@ -102,6 +107,15 @@ int ws_tensor(const ornith_weights* ws, const std::string& name, int dtype, int6
 int ws_stacked(const ornith_weights* ws, const std::string& prefix, const std::string& suffix,
                int experts, int dtype, int64_t numel, const void** out);
 size_t ornith_dt_size(int dt);
+// A bf16 matrix [O, K] under its full name, as a dense projection.
+int ws_dense(const ornith_weights* ws, const std::string& name, int O, int K, ornith_linear* out);
+
+static const int kMaxRows = 16;  // activation rows a forward may carry unless the model is told otherwise
+
+// ---- layers ------------------------------------------------------------------------
+// A layer is a mixer (what looks across tokens) and a feed-forward, either of several kinds.
+enum MixerKind { MIX_GATED_DELTA, MIX_GATED_ATTN, MIX_MLSTM, MIX_DIFF_ATTN };
+enum FfKind { FF_MOE, FF_DENSE, FF_NONE };
 
 struct GdnLayer {
   ornith_linear in_proj_qkv, in_proj_z, out_proj, in_proj_a, in_proj_b;
@@ -111,17 +125,82 @@ struct AttnLayer {
   ornith_linear q_proj, k_proj, v_proj, o_proj;
   const void *q_norm, *k_norm;
 };
+// mlstm.hip: matrix memory with exponential gates
+struct MlstmLayer {
+  int heads, dim, vdim;
+  float gate_cap;
+  ornith_linear q, k, v, g, o, i, f;
+  const void *norm, *i_b, *f_b;
+};
+// diff_attn.hip: two softmax maps over the same values, rotary positions, a sliding window with
+// kept first tokens, one output gate a head
+struct DiffAttnLayer {
+  int heads, kv_heads, dim, vdim;
+  int window, keep_first;  // window 0: none
+  int rope;                // which of the model's rotation tables
+  float scale, diff, lambda;
+  ornith_linear q, k, v, g, o;
+};
+struct DenseFf {
+  int ff;
+  ornith_linear gate, up, down;
+};
+
+// What a layer keeps from token to token. The caches are laid out from this alone.
+struct CacheSpec {
+  int kv_heads = 0;                  // KV rows: kv_heads x capacity of
+  size_t k_row = 0, v_row = 0;       //   these many bytes
+  int conv_taps = 0;                 // convolution window: rows kept, and
+  size_t conv_row = 0;               //   bytes a row
+  size_t state = 0;                  // recurrent state: bytes a slot
+};
+
 struct Layer {
-  bool linear = false;
+  MixerKind mixer = MIX_GATED_ATTN;
+  FfKind ffn = FF_MOE;
   const void *input_ln = nullptr, *post_ln = nullptr;
+  CacheSpec keeps;
   GdnLayer gdn{};
   AttnLayer attn{};
+  MlstmLayer mlstm{};
+  DiffAttnLayer dattn{};
   ornith_moe_weights moe{};
+  DenseFf dense{};
+};
+
+// A rotation: cos / sin of position * base^(-2i/dims) / factor
+struct RopeTable {
+  int dims = 0;
+  double base = 0, factor = 1;
+  float *d_cos = nullptr, *d_sin = nullptr;  // f32 [rope_npos, dims/2]
+};
+
+// ---- designs -------------------------------------------------------------------------
+// One entry of the model registry. The entry whose `architecture` is config.json's
+// "architecture" loads the model; an entry without one takes the files that lack the key.
+struct ModelDesign {
+  const char* architecture;
+  const char* name;
+  bool runs_f32;  // also with activations and products in 32-bit
+  int (*load)(ornith_ctx* ctx, const ornith_weights* ws, const orn_json::JVal& cfg, int act_dtype, ornith_model** out);
+  size_t (*step_bytes)(const ornith_model* m, int rows);
+  // T tokens through the trunk, the caches' cursors still where they were (the caller moves them)
+  int (*forward)(ornith_model* m, ornith_caches* cc, const uint32_t* d_tokens, int T, bool capture, void* d_hidden);
+  int (*logits)(ornith_model* m, const void* d_hidden, int T, void* d_logits, int dtype);
+  // the recurrent slots are walked as a ring: a forward never writes the slot it starts from
+  bool state_ring;
+  ModelDesign* next;
+};
+struct DesignEntry {
+  explicit DesignEntry(ModelDesign* d);
 };
 
 struct ornith_model {
   ornith_ctx* ctx = nullptr;
-  ornith_text_config cfg{};
+  const ModelDesign* design = nullptr;
+  int act_dtype = ORNITH_BF16;  // hidden rows, activations, KV rows
+  ornith_text_config cfg{};     // every design fills hidden_size, vocab_size, num_hidden_layers, rms_norm_eps
+  float embed_scale = 1.f;
   ornith_linear embed_tokens{};
   ornith_linear lm_head{};
   const void* final_norm = nullptr;
@@ -131,24 +210,27 @@ struct ornith_model {
   void* ws_buf = nullptr;
   size_t ws_bytes = 0;
   // rope tables, grown on demand to the largest cache capacity seen
-  float *d_cos = nullptr, *d_sin = nullptr;
+  std::vector<RopeTable> ropes;
   int rope_npos = 0;
   int key_dim() const { return cfg.linear_num_key_heads * cfg.linear_key_head_dim; }
   int value_dim() const { return cfg.linear_num_value_heads * cfg.linear_value_head_dim; }
   int conv_dim() const { return 2 * key_dim() + value_dim(); }
+  // the table of such a rotation, made at the next model_ensure_rope
+  int rope_index(int dims, double base, double factor);
 };
 
 struct LayerCache {
-  // full attention
-  void *k = nullptr, *v = nullptr;  // bf16 [Hkv, cap, hd]
+  // attention
+  void *k = nullptr, *v = nullptr;  // [kv_heads, cap, row]
   // gated delta
   void* conv[2] = {nullptr, nullptr};  // bf16 [K-1+max_rows, D] each
-  float* state = nullptr;              // f32 [slots][Hv, Dv, Dk]
+  float* state = nullptr;              // f32 [slots][the layer's state]
 };
 
 struct ornith_caches {
   ornith_model* m = nullptr;
-  int capacity = 0, max_window = 0, conv_rows = 0;
+  int capacity = 0, max_window = 0, rows = 0;  // rows: the most a forward may carry
+  int slots = 0;                               // recurrent state slots
   bool growable = true;  // a forward past the capacity grows the KV tensors (else it is refused)
   std::vector<LayerCache> layers;
   // one set of cursors serves every layer: they all advance together
@@ -156,8 +238,11 @@ struct ornith_caches {
   int conv_cur = 0;   // which conv buffer holds the live window
   int conv_off = 0;   // first row of the live K-1 rows in it
   int state_cur = 0;  // slot holding the live recurrent state
+  int state_base = 0; // slot the last forward's first snapshot went to
   int last_T = 0;     // rows of the last forward (for rewind)
   bool last_capture = false;
+  // slot that receives the state after token t of the next forward
+  int state_out(int t) const { return m->design->state_ring ? (state_cur + 1 + t) % slots : t; }
 };
 
 struct ornith_frspec {

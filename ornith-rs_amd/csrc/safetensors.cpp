@@ -182,9 +182,14 @@ struct ornith_safetensors {
   }
 };
 
-// model.safetensors.index.json -> the shard paths, sorted and de-duplicated.
+// model.safetensors.index.json -> the shard paths, sorted and de-duplicated; a directory without
+// an index may hold everything in one model.safetensors.
 static int shards_from_index(const std::string& dir, std::vector<std::string>* out) {
-  const std::string idx_path = dir + "/model.safetensors.index.json";
+  const std::string idx_path = dir + "/model.safetensors.index.json", one = dir + "/model.safetensors";
+  if (access(idx_path.c_str(), F_OK) != 0 && access(one.c_str(), F_OK) == 0) {
+    out->push_back(one);
+    return ORNITH_OK;
+  }
   JVal idx;
   std::string err;
   if (!json_file(idx_path, &idx, &err)) return ornith_fail(ORNITH_ERR_IO, "%s", err.c_str());
@@ -263,7 +268,7 @@ int quant_table_load(const std::string& dir, QuantTable* qt) {
   return ORNITH_OK;
 }
 
-static int text_config_from(const JVal& cfg, ornith_text_config* c, int* mtp_layers) {
+int text_config_from(const JVal& cfg, ornith_text_config* c, int* mtp_layers) {
   // the text model's keys sit under `text_config` when the artifact also has a vision tower
   const JVal* t = cfg.get("text_config");
   if (!t) t = &cfg;
@@ -498,9 +503,16 @@ int ornith_weights_open(ornith_ctx* ctx, const char* model_dir, const char* cons
   std::unique_ptr<ornith_weights_files> files(new ornith_weights_files());
   int rc = ornith_safetensors_open_model(model_dir, extra, n_extra, &files->st);
   if (rc) return rc;
+  // a config that names its architecture describes plain tensors unless it has the block
+  JVal cfg;
+  std::string err;
   QuantTable qt;
-  rc = quant_table_load(model_dir, &qt);
-  if (rc) return rc;
+  const bool plain = json_file(std::string(model_dir) + "/config.json", &cfg, &err) && cfg.get("architecture") &&
+                     !cfg.get("quantization");
+  if (!plain) {
+    rc = quant_table_load(model_dir, &qt);
+    if (rc) return rc;
+  }
   for (auto& f : files->st->files) f->will_need();
   ornith_weights* w = new ornith_weights();
   w->ctx = ctx;

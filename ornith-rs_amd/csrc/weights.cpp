@@ -152,6 +152,20 @@ int ws_linear(const ornith_weights* ws, const std::string& path, ornith_linear* 
   return ORNITH_OK;
 }
 
+int ws_dense(const ornith_weights* ws, const std::string& name, int O, int K, ornith_linear* out) {
+  memset(out, 0, sizeof *out);
+  const void* w = nullptr;
+  int rc = ws_tensor(ws, name, ORNITH_DT_BF16, (int64_t)O * K, &w);
+  if (rc) return rc;
+  const std::vector<int64_t>& s = ws->find(name)->shape;
+  ORN_REQUIRE(s.size() == 2 && s[0] == O && s[1] == K, "%s: expected [%d, %d]", name.c_str(), O, K);
+  out->mode = ORNITH_LIN_DENSE;
+  out->O = O;
+  out->K = K;
+  out->d_w = w;
+  return ORNITH_OK;
+}
+
 int ws_tensor(const ornith_weights* ws, const std::string& name, int dtype, int64_t numel,
               const void** out) {
   ws->fault_rc = 0;
