@@ -99,6 +99,9 @@ ORNITH_API int ornith_device_info(ornith_ctx* ctx, char* name, size_t name_len, 
  *   "fuse_attn_prep" (ORNITH_FUSE_ATTN_PREP, default 1): ornith_attn_decode lets the attention
  *               launch do the prep of its own rows (norm, RoPE, KV append) at decode widths
  *               (0: a prep launch first); bit-identical
+ *   "mlstm_chunked" (ORNITH_MLSTM_CHUNKED, default 1): the mLSTM recurrence of calls of 64 rows
+ *               or more runs in 64-token chunks on the matrix cores (0: token by token); results
+ *               agree to rounding
  *   "fuse_moe_one" (ORNITH_FUSE_MOE_ONE, default 0): the MoE block's phases as ranges of
  *               workgroups of ONE launch that hand their intermediates over through memory
  *               (1: router + up + down, 2: up + down after a router launch). Bit-identical,
@@ -398,6 +401,96 @@ ORNITH_API int ornith_attn_decode(ornith_ctx* ctx, const void* d_qg, const void*
 ORNITH_API int ornith_sdpa_prefill_gated(ornith_ctx* ctx, const void* d_q_rot, const void* d_k_cache,
                                          const void* d_v_cache, const void* d_qg, int T, int Hq, int Hkv,
                                          int hd, int offset, int cap, float scale, void* d_out);
+
+/* ---- dense bf16 projections around a 32-bit residual stream ---------------------------
+ * No counterpart in the reference (its projections are quantized and its stream bf16). Element
+ * type of the activations per call: `act` = ORNITH_BF16, or ORNITH_F32 for everything in 32-bit
+ * (weights are bf16 numbers either way). Every row of a call below the gemm_rows option is summed
+ * exactly as it would be alone; bf16 calls from there on run as a tiled matrix-core GEMM. */
+#define ORNITH_PRE_NONE 0  /* d_x: act [M, K] */
+#define ORNITH_PRE_NORM 1  /* d_x: f32 [M, K]; rows = x / sqrt(mean(x^2) + eps) * (w_offset + w) */
+#define ORNITH_PRE_HEADS 2 /* d_x: f32 [M, K]: heads of head_dim values, each over its own root mean
+                              square, times w [K], times sigmoid(gate), gate: act [M, K] */
+#define ORNITH_OUT_ACT 0   /* y: act [M, O] */
+#define ORNITH_OUT_F32 1   /* y: f32 [M, O] */
+#define ORNITH_OUT_ADD 2   /* y: f32 [M, O], added to */
+typedef struct ornith_dense_call {
+  int act, pre;
+  const void* d_x;
+  const void* d_norm_w; /* bf16 [K] */
+  const void* d_gate;
+  float w_offset, eps;
+  int head_dim;
+  int M, K;
+  int n; /* matrices, at most 6, all [O, K] dense */
+  const ornith_linear* w[6];
+  void* d_y[6];
+  int out[6];
+  int gelu_pair; /* n == 2: d_y[0] (act) = gelu_tanh(w[0] row) * (w[1] row) */
+  void* d_rows;  /* act [M, K]: where the rows a prologue makes are kept for a GEMM (may be null below it) */
+} ornith_dense_call;
+ORNITH_API int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* call);
+/* the prologues alone */
+ORNITH_API int ornith_norm_rows(ornith_ctx* ctx, const float* d_x, const void* d_w, float w_offset, int rows, int n,
+                                float eps, int act, void* d_out);
+ORNITH_API int ornith_head_norm_gate(ornith_ctx* ctx, const float* d_x, const void* d_w, const void* d_gate, int rows,
+                                     int heads, int head_dim, float eps, int act, void* d_out);
+/* rows of a dense bf16 table times `scale`, f32; ids are clamped to the table */
+ORNITH_API int ornith_embed_rows(ornith_ctx* ctx, const ornith_linear* table, const uint32_t* d_ids, int n, float scale,
+                                 float* d_out);
+
+/* n floats to bf16 */
+ORNITH_API int ornith_round_bf16(ornith_ctx* ctx, const float* d_x, size_t n, void* d_out);
+
+/* ---- mLSTM: matrix memory with exponential gates and a running maximum --------------------
+ * Beck et al., "xLSTM: Extended Long Short-Term Memory". Per head, with q scaled by dim^(-1/2), log gates
+ * i = cap tanh((gi + bi) / cap), f = logsigmoid(cap tanh((gf + bf) / cap)) and m starting at 0:
+ *   m' = max(f + m, i);  S' = e^(f + m - m') S + e^(i - m') v k^T;  n' likewise with k alone
+ *   o = S' q / (max(|n' . q|, e^(-m')) + 1e-6)
+ * q, k: act [T, H*dim], v: act [T, H*vdim], gi, gf: f32 [T, H] (the raw projections), bi, bf: bf16 [H];
+ * o: f32 [T, H*vdim]. State: ornith_mlstm_state_floats(H, dim, vdim) floats a slot, all zero for a new
+ * sequence. The state after token t goes to slot slot_out(t) = (first_slot + t) mod n_slots of d_slots
+ * for every token (snapshots != 0) or, for the last token only, to slot first_slot; d_state_in must be
+ * none of the slots written. Calls of 64 rows or more (bf16, dim and vdim multiples of 8, dim <= 256,
+ * no snapshots; option mlstm_chunked) run in chunks of 64 tokens on the matrix cores, everything that enters the
+ * recurrence besides q, k, v in 32-bit or as two bf16 parts. */
+typedef struct ornith_mlstm_call {
+  int act;
+  const void *d_q, *d_k, *d_v;
+  const float *d_gi, *d_gf;
+  const void *d_bi, *d_bf;
+  float gate_cap;
+  int T, H, dim, vdim;
+  const float* d_state_in;
+  float* d_slots;
+  int n_slots, first_slot, snapshots;
+  float* d_o;
+} ornith_mlstm_call;
+ORNITH_API size_t ornith_mlstm_state_floats(int H, int dim, int vdim);
+ORNITH_API int ornith_mlstm(ornith_ctx* ctx, const ornith_mlstm_call* call);
+
+/* ---- differential attention over a KV cache --------------------------------------------
+ * Ye et al., "Differential Transformer". q: act [T, H, 2, dim], k: act [T, G, 2, dim] (map 1, map 2 of a
+ * head side by side), v: act [T, G, vdim], gate: f32 [T, H]; query head h reads KV head h / (H / G).
+ * Rotary positions on the first rope_dims dimensions of every map, pairs (2i, 2i+1), tables f32
+ * [table_npos, rope_dims/2]; keys are appended rotated to d_k_cache act [G, cap, 2*dim], values to
+ * d_v_cache act [G, cap, vdim] at rows [offset, offset + T). A query at position i sees key j <= i if
+ * i - j < window (window 0: any) or j < keep_first. With a1, a2 the two maps' softmax attention:
+ * o = a1 - lambda a2, over its root mean square, times (1 - diff) sigmoid(gate): act [T, H*vdim].
+ * bf16 calls of gemm_rows rows or more (dims multiples of 8, dim <= 128, vdim <= 256) run on the
+ * matrix cores; d_q_rot (act [T, H, 2, dim]) is needed from there on. */
+typedef struct ornith_diff_attn_call {
+  int act;
+  const void *d_q, *d_k, *d_v;
+  const float* d_gate;
+  const float *d_cos, *d_sin;
+  int rope_dims, table_npos;
+  int T, H, G, dim, vdim;
+  int offset, cap, window, keep_first;
+  float scale, lambda, diff, eps;
+  void *d_k_cache, *d_v_cache, *d_q_rot, *d_out;
+} ornith_diff_attn_call;
+ORNITH_API int ornith_diff_attn(ornith_ctx* ctx, const ornith_diff_attn_call* call);
 
 /* ---- greedy selection: src/ops/sample.rs ------------------------------------------ */
 /* greedy_token / the verify rows of generate_step_mtp (src/ops/sample.rs:134-147,

@@ -392,4 +392,4 @@ def argmax_rows(self, logits, rows, V, out):
 
 
 from .engine import *  # noqa: E402,F401,F403  (engine objects: WeightStore, TextModel, ...)
-from .engine import TextConfig, Sampler, MtpStats, WeightStore, Caches, TextModel, FrSpec, MtpHead, generate_step, generate_step_mtp, HISTORY_CYCLE, HISTORY_COMMITTED  # noqa: E402,F401
+from .engine import TextConfig, Sampler, MtpStats, WeightStore, Caches, TextModel, ModelInfo, FrSpec, MtpHead, generate_step, generate_step_mtp, HISTORY_CYCLE, HISTORY_COMMITTED  # noqa: E402,F401

@@ -1,6 +1,7 @@
 """Build recipe for the HIP library (gfx950 only).
 
     python ornith-rs_amd/build.py          # compile csrc/*.hip, *.cpp -> libornith_hip.so
+    python ornith-rs_amd/build.py Pigodra  # only what models of that design need -> build/libornith_Pigodra.so
 
 hipcc cross-compiles without a GPU. Every translation unit is compiled with
 -ffp-contract=off (the only fused multiply-adds are the explicit ones, so results
@@ -34,8 +35,20 @@ FLAGS = [
 FLAGS += os.environ.get("ORN_EXTRA_FLAGS", "").split()
 
 
-def sources():
+# What every design needs, and what each design of the registry adds (a design that is not listed
+# needs the whole library).
+CORE = ["runtime.hip", "weights.cpp", "safetensors.cpp", "model.cpp", "rope.cpp", "engine.cpp", "sample.hip", "sampler.hip"]
+DESIGNS = {"Pigodra": ["pigodra.cpp", "stack.cpp", "dense_rows.hip", "mlstm.hip", "diff_attn.hip"]}
+
+
+def sources(design=None):
+    if design is not None:
+        return CORE + DESIGNS[design]
     return sorted(f for f in os.listdir(CSRC) if f.endswith((".hip", ".cpp")))
+
+
+def library(design=None):
+    return LIB if design is None else os.path.join(OBJ, f"libornith_{design}.so")
 
 
 def _compile(src):
@@ -47,23 +60,43 @@ def _compile(src):
     return src, obj, r.returncode, err
 
 
-def build(verbose=True, jobs=8):
+def build(verbose=True, jobs=8, design=None):
     os.makedirs(OBJ, exist_ok=True)
     objs = []
     with concurrent.futures.ThreadPoolExecutor(max_workers=jobs) as ex:
-        for src, obj, rc, err in ex.map(_compile, sources()):
+        for src, obj, rc, err in ex.map(_compile, sources(design)):
             if verbose and err.strip():
                 print(f"[{src}]\n{err}", file=sys.stderr)
             if rc != 0:
                 raise RuntimeError(f"hipcc failed on {src}")
             objs.append(obj)
-    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB, *objs]
+    # linked beside its place and moved there whole, so that nobody loads half a library
+    out = library(design)
+    part = f"{out}.{os.getpid()}"
+    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-Wl,-z,defs", "-o", part, *objs]
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         print(r.stderr, file=sys.stderr)
         raise RuntimeError("link failed")
-    return LIB
+    os.replace(part, out)
+    return out
+
+
+def ensure(design=None):
+    """The path of a library that serves `design`: the whole one if it is there, else one of the
+    design's own parts, compiled if need be (one process at a time)."""
+    import fcntl
+    if design not in DESIGNS:
+        design = None
+    for path in (LIB, library(design)):
+        if os.path.exists(path):
+            return path
+    os.makedirs(OBJ, exist_ok=True)
+    with open(os.path.join(OBJ, ".lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        path = library(design)
+        return path if os.path.exists(path) else build(verbose=False, design=design)
 
 
 if __name__ == "__main__":
-    print(build())
+    print(build(design=sys.argv[1] if len(sys.argv) > 1 else None))

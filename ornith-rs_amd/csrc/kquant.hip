@@ -413,51 +413,13 @@ int pick_iters() {
   return forced > 8 ? 8 : forced;
 }
 
-int check_matrix(const ornith_kmatrix* w, const char* who) {
-  ORN_REQUIRE(w, "%s: null matrix", who);
-  ORN_REQUIRE(w->kind == ORNITH_Q4K || w->kind == ORNITH_Q6K, "%s: unknown k-quant kind %d", who,
-              w->kind);
-  ORN_REQUIRE(w->E >= 1 && w->O >= 1 && w->K >= 256, "%s: bad dims E=%d O=%d K=%d", who, w->E,
-              w->O, w->K);
-  ORN_REQUIRE(w->K % 256 == 0, "%s: %d is not a multiple of 256", who, w->K);
-  ORN_REQUIRE(w->d_qs && w->d_scales && w->d_dm, "%s: null tensor", who);
-  return ORNITH_OK;
-}
-
 }  // namespace
 
 extern "C" {
 
-int ornith_kmatrix_check(const ornith_kmatrix* w, size_t qs_bytes, size_t scales_bytes,
-                         size_t dm_bytes) {
-  if (w && w->kind == ORNITH_AFFINE4_G32) {
-    ORN_REQUIRE(w->E >= 1 && w->O >= 1 && w->K >= 32 && w->K % 32 == 0, "KMatrix: bad dims E=%d O=%d K=%d", w->E,
-                w->O, w->K);
-    ORN_REQUIRE(w->d_qs && w->d_scales && w->d_dm, "KMatrix: null tensor");
-    const size_t groups = (size_t)w->E * w->O * (w->K / 32);
-    ORN_REQUIRE(qs_bytes == groups * 16 && scales_bytes == groups * 2 && dm_bytes == groups * 2,
-                "affine4 sizes: %zu / %zu / %zu bytes, %zu groups want %zu / %zu / %zu", qs_bytes, scales_bytes,
-                dm_bytes, groups, groups * 16, groups * 2, groups * 2);
-    return ORNITH_OK;
-  }
-  int rc = check_matrix(w, "KMatrix");
-  if (rc) return rc;
-  const size_t blocks = (size_t)w->E * w->O * (w->K / 256);
-  const size_t cb = w->kind == ORNITH_Q4K ? 128 : 192, sb_ = w->kind == ORNITH_Q4K ? 12 : 16,
-               db = w->kind == ORNITH_Q4K ? 4 : 2;
-  const char* name = w->kind == ORNITH_Q4K ? "q4k" : "q6k";
-  ORN_REQUIRE(qs_bytes == blocks * cb, "%s qs size: %zu bytes, %zu blocks want %zu", name, qs_bytes,
-              blocks, blocks * cb);
-  ORN_REQUIRE(scales_bytes == blocks * sb_, "%s scales size: %zu bytes, want %zu", name,
-              scales_bytes, blocks * sb_);
-  ORN_REQUIRE(dm_bytes == blocks * db, "%s dm size: %zu bytes, want %zu", name, dm_bytes,
-              blocks * db);
-  return ORNITH_OK;
-}
-
 int ornith_kq_dequantize(ornith_ctx* ctx, const ornith_kmatrix* w, void* d_out, int out_dtype) {
   ORN_REQUIRE(ctx && d_out, "kq_dequantize: null argument");
-  int rc = check_matrix(w, "kq_dequantize");
+  int rc = kmatrix_check_dims(w, "kq_dequantize");
   if (rc) return rc;
   const int64_t blocks = (int64_t)w->E * w->O * (w->K / 256);
   dim3 grid((unsigned)((blocks + 63) / 64));
@@ -484,7 +446,7 @@ int kq_qmv_multi_prenorm(ornith_ctx* ctx, const ornith_kmatrix* const* ws, int n
   // are dead before the row loop's peak -- and the launch saved is worth 0.4 % at depth 1 and 1.7 %
   // at depth 3 in same-box A/B runs, so every width takes the norm in its head now.)
   for (int s = 0; s < n; ++s) {
-    if (check_matrix(ws[s], "kq_qmv_prenorm")) return -1;
+    if (kmatrix_check_dims(ws[s], "kq_qmv_prenorm")) return -1;
     if (ws[s]->E != 1 || ws[s]->kind != ws[0]->kind || ws[s]->K != ws[0]->K || !d_ys[s]) return -1;
   }
   KqArgs a{};
@@ -512,7 +474,7 @@ int ornith_kq_qmv_multi(ornith_ctx* ctx, const ornith_kmatrix* const* ws, int n,
   ORN_REQUIRE(M >= 1, "kq_qmv: M=%d", M);
   ORN_REQUIRE(((uintptr_t)d_x & 15) == 0, "kq_qmv: x must be 16-byte aligned");
   for (int s = 0; s < n; ++s) {
-    int rc = check_matrix(ws[s], "kq_qmv");
+    int rc = kmatrix_check_dims(ws[s], "kq_qmv");
     if (rc) return rc;
     ORN_REQUIRE(ws[s]->E == 1, "kq_qmv: matrix has %d experts; use gather_qmv", ws[s]->E);
     ORN_REQUIRE(ws[s]->kind == ws[0]->kind && ws[s]->K == ws[0]->K,
@@ -558,7 +520,7 @@ int ornith_kq_gather_qmv(ornith_ctx* ctx, const ornith_kmatrix* w, const void* d
                          int x_rows, const uint32_t* d_lhs, const uint32_t* d_rhs, int rows,
                          void* d_y, int y_dtype) {
   ORN_REQUIRE(ctx && d_x && d_y && d_lhs && d_rhs, "kq_gather_qmv: null argument");
-  int rc = check_matrix(w, "kq_gather_qmv");
+  int rc = kmatrix_check_dims(w, "kq_gather_qmv");
   if (rc) return rc;
   ORN_REQUIRE(rows >= 0 && rows <= 65535, "kq_gather_qmv: rows=%d", rows);
   ORN_REQUIRE(x_rows >= 1, "kq_gather_qmv: x_rows=%d", x_rows);

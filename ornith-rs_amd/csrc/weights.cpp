@@ -89,6 +89,17 @@ static int kq_from(const ornith_weights* ws, const std::string& path, bool route
   return ornith_kmatrix_check(out, w->bytes, s->bytes, d->bytes);
 }
 
+int kmatrix_check_dims(const ornith_kmatrix* w, const char* who) {
+  ORN_REQUIRE(w, "%s: null matrix", who);
+  ORN_REQUIRE(w->kind == ORNITH_Q4K || w->kind == ORNITH_Q6K, "%s: unknown k-quant kind %d", who,
+              w->kind);
+  ORN_REQUIRE(w->E >= 1 && w->O >= 1 && w->K >= 256, "%s: bad dims E=%d O=%d K=%d", who, w->E,
+              w->O, w->K);
+  ORN_REQUIRE(w->K % 256 == 0, "%s: %d is not a multiple of 256", who, w->K);
+  ORN_REQUIRE(w->d_qs && w->d_scales && w->d_dm, "%s: null tensor", who);
+  return ORNITH_OK;
+}
+
 int ws_kmatrix(const ornith_weights* ws, const std::string& path, ornith_kmatrix* out) {
   return kq_from(ws, path, true, out);
 }
@@ -179,6 +190,33 @@ int ws_tensor(const ornith_weights* ws, const std::string& name, int dtype, int6
 }
 
 extern "C" {
+
+int ornith_kmatrix_check(const ornith_kmatrix* w, size_t qs_bytes, size_t scales_bytes,
+                         size_t dm_bytes) {
+  if (w && w->kind == ORNITH_AFFINE4_G32) {
+    ORN_REQUIRE(w->E >= 1 && w->O >= 1 && w->K >= 32 && w->K % 32 == 0, "KMatrix: bad dims E=%d O=%d K=%d", w->E,
+                w->O, w->K);
+    ORN_REQUIRE(w->d_qs && w->d_scales && w->d_dm, "KMatrix: null tensor");
+    const size_t groups = (size_t)w->E * w->O * (w->K / 32);
+    ORN_REQUIRE(qs_bytes == groups * 16 && scales_bytes == groups * 2 && dm_bytes == groups * 2,
+                "affine4 sizes: %zu / %zu / %zu bytes, %zu groups want %zu / %zu / %zu", qs_bytes, scales_bytes,
+                dm_bytes, groups, groups * 16, groups * 2, groups * 2);
+    return ORNITH_OK;
+  }
+  int rc = kmatrix_check_dims(w, "KMatrix");
+  if (rc) return rc;
+  const size_t blocks = (size_t)w->E * w->O * (w->K / 256);
+  const size_t cb = w->kind == ORNITH_Q4K ? 128 : 192, sb_ = w->kind == ORNITH_Q4K ? 12 : 16,
+               db = w->kind == ORNITH_Q4K ? 4 : 2;
+  const char* name = w->kind == ORNITH_Q4K ? "q4k" : "q6k";
+  ORN_REQUIRE(qs_bytes == blocks * cb, "%s qs size: %zu bytes, %zu blocks want %zu", name, qs_bytes,
+              blocks, blocks * cb);
+  ORN_REQUIRE(scales_bytes == blocks * sb_, "%s scales size: %zu bytes, want %zu", name,
+              scales_bytes, blocks * sb_);
+  ORN_REQUIRE(dm_bytes == blocks * db, "%s dm size: %zu bytes, want %zu", name, dm_bytes,
+              blocks * db);
+  return ORNITH_OK;
+}
 
 int ornith_weights_create(ornith_ctx* ctx, ornith_weights** out) {
   ORN_REQUIRE(ctx && out, "weights_create: null argument");

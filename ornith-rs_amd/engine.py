@@ -3,6 +3,7 @@ WeightStore, TextModel (+ caches), FrSpec, MtpHead, generate_step, generate_step
 Names and argument meaning follow /root/reference/src/{weights,frspec,generate,
 mtp_generate}.rs and src/model/{qwen3_5,mtp}.rs so tests read like the reference's."""
 import ctypes as C
+import json
 import os
 
 import numpy as np
@@ -254,29 +255,64 @@ class Caches:
             self.h = None
 
 
-class TextModel:
-    """TextModel::load + forward_hidden / forward_capture / rewind."""
+class ModelInfo(C.Structure):
+    """ornith_model_info"""
+    _fields_ = [(n, C.c_int) for n in ("hidden_size", "vocab_size", "num_layers", "act_dtype", "max_rows")] + [
+        ("design", C.c_char * 32)]
 
-    def __init__(self, ctx, ws, cfg):
+
+class TextModel:
+    """A model of the registry: forward_hidden / forward_capture / rewind / logits.
+
+    TextModel(ctx, ws, text_config) is TextModel::load; open() and from_json() let config.json's
+    "architecture" pick the design."""
+
+    def __init__(self, ctx, ws, cfg, _handle=None):
         self.ctx, self.ws, self.cfg = ctx, ws, cfg
+        if _handle is None:
+            _handle = C.c_void_p()
+            _check(lib().ornith_model_load(ctx.h, ws.h, C.byref(cfg), C.byref(_handle)), "model_load")
+        self.h = _handle
+        self.info = ModelInfo()
+        _check(lib().ornith_model_describe(self.h, C.byref(self.info)), "model_describe")
+        if cfg is None:
+            self.cfg = self.info
+        self._hidden = np.float32 if self.info.act_dtype == F32 else np.uint16
+
+    @staticmethod
+    def open(ctx, ws, model_dir, act_dtype=BF16):
+        """The model <model_dir>/config.json describes, its weights from the store `ws`."""
         h = C.c_void_p()
-        _check(lib().ornith_model_load(ctx.h, ws.h, C.byref(cfg), C.byref(h)), "model_load")
-        self.h = h
+        _check(lib().ornith_model_open(ctx.h, ws.h, os.fsencode(model_dir), act_dtype, C.byref(h)), f"model_open({model_dir})")
+        return TextModel(ctx, ws, None, h)
+
+    @staticmethod
+    def from_json(ctx, ws, config, act_dtype=BF16):
+        """The same from a config dict (for a store filled with put)."""
+        text = json.dumps(config).encode()
+        h = C.c_void_p()
+        _check(lib().ornith_model_load_json(ctx.h, ws.h, text, C.c_size_t(len(text)), act_dtype, C.byref(h)), "model_load_json")
+        return TextModel(ctx, ws, None, h)
 
     def make_cache(self, capacity, max_window=4):
         return Caches(self, capacity, max_window)
 
     def forward(self, caches, tokens, capture=False):
-        """tokens: host uint32 array -> post-norm hidden rows as uint16 bf16 bits [T, H]."""
+        """tokens: host uint32 array -> post-norm hidden rows [T, H]: uint16 bf16 bits, or float32
+        for a model opened in 32-bit."""
         tokens = np.ascontiguousarray(tokens, dtype=np.uint32)
         T, H = len(tokens), self.cfg.hidden_size
-        dt, dh = self.ctx.to_device(tokens), self.ctx.alloc(T * H * 2)
+        dt, dh = self.ctx.to_device(tokens), self.ctx.alloc(T * H * np.dtype(self._hidden).itemsize)
         try:
-            _check(lib().ornith_model_forward(self.h, caches.h, dt.ptr, T, int(capture), dh.ptr), "model_forward")
-            return dh.download(np.uint16, (T, H))
+            self.forward_on_device(caches, dt, T, dh, capture)
+            return dh.download(self._hidden, (T, H))
         finally:
             dt.free()
             dh.free()
+
+    def forward_on_device(self, caches, tokens, T, hidden, capture=False):
+        """The step function itself: T token ids on the device -> hidden rows on the device."""
+        _check(lib().ornith_model_forward(self.h, caches.h, tokens.ptr, T, int(capture), hidden.ptr), "model_forward")
 
     def rewind(self, caches, keep):
         _check(lib().ornith_model_rewind(self.h, caches.h, keep), "model_rewind")
@@ -293,8 +329,23 @@ class TextModel:
         _check(lib().ornith_model_moe_weights(self.h, layer, C.byref(w)), "model_moe_weights")
         return w
 
+    def logits_f32_on_device(self, hidden, T, logits):
+        _check(lib().ornith_model_logits_f32(self.h, hidden.ptr, T, logits.ptr), "model_logits_f32")
+
+    def logits_f32(self, hidden):
+        """Hidden rows (as forward returns them) -> float32 logits [T, V]."""
+        hidden = np.ascontiguousarray(hidden, dtype=self._hidden)
+        T, V = hidden.shape[0], self.cfg.vocab_size
+        dh, dl = self.ctx.to_device(hidden), self.ctx.alloc(T * V * 4)
+        try:
+            self.logits_f32_on_device(dh, T, dl)
+            return dl.download(np.float32, (T, V))
+        finally:
+            dh.free()
+            dl.free()
+
     def logits(self, hidden):
-        hidden = np.ascontiguousarray(hidden, dtype=np.uint16)
+        hidden = np.ascontiguousarray(hidden, dtype=self._hidden)
         T, V = hidden.shape[0], self.cfg.vocab_size
         dh, dl = self.ctx.to_device(hidden), self.ctx.alloc(T * V * 2)
         try:
@@ -618,3 +669,62 @@ def add_rms_linear_multi(ctx, lins, res, y, wnorm, eps, M, h_out, normed_out, ys
 def add_rms_moe_block(ctx, w, res, y, wnorm, eps, T, h_out, normed_out, out):
     _check(lib().ornith_add_rms_moe_block(ctx.h, C.byref(w), res.ptr, y.ptr, wnorm.ptr, C.c_float(eps), T,
                                           h_out.ptr, normed_out.ptr, out.ptr), "add_rms_moe_block")
+
+
+# ---- dense projections around a 32-bit residual stream, mLSTM, differential attention ---------
+PRE_NONE, PRE_NORM, PRE_HEADS = range(3)
+OUT_ACT, OUT_F32, OUT_ADD = range(3)
+
+
+class DenseCall(C.Structure):
+    """ornith_dense_call"""
+    _fields_ = [("act", C.c_int), ("pre", C.c_int), ("d_x", C.c_void_p), ("d_norm_w", C.c_void_p), ("d_gate", C.c_void_p),
+                ("w_offset", C.c_float), ("eps", C.c_float), ("head_dim", C.c_int), ("M", C.c_int), ("K", C.c_int),
+                ("n", C.c_int), ("w", C.POINTER(LinearStruct) * 6), ("d_y", C.c_void_p * 6), ("out", C.c_int * 6),
+                ("gelu_pair", C.c_int), ("d_rows", C.c_void_p)]
+
+
+class MlstmCall(C.Structure):
+    """ornith_mlstm_call"""
+    _fields_ = [("act", C.c_int)] + [(n, C.c_void_p) for n in ("d_q", "d_k", "d_v", "d_gi", "d_gf", "d_bi", "d_bf")] + [
+        ("gate_cap", C.c_float), ("T", C.c_int), ("H", C.c_int), ("dim", C.c_int), ("vdim", C.c_int),
+        ("d_state_in", C.c_void_p), ("d_slots", C.c_void_p), ("n_slots", C.c_int), ("first_slot", C.c_int),
+        ("snapshots", C.c_int), ("d_o", C.c_void_p)]
+
+
+class DiffAttnCall(C.Structure):
+    """ornith_diff_attn_call"""
+    _fields_ = [("act", C.c_int)] + [(n, C.c_void_p) for n in ("d_q", "d_k", "d_v", "d_gate", "d_cos", "d_sin")] + [
+        (n, C.c_int) for n in ("rope_dims", "table_npos", "T", "H", "G", "dim", "vdim", "offset", "cap", "window",
+                               "keep_first")] + [(n, C.c_float) for n in ("scale", "lam", "diff", "eps")] + [
+        (n, C.c_void_p) for n in ("d_k_cache", "d_v_cache", "d_q_rot", "d_out")]
+
+
+def dense_rows(ctx, act, x, M, K, lins, ys, outs, pre=PRE_NONE, norm_w=None, gate=None, w_offset=0.0, eps=1e-6, head_dim=0,
+               gelu_pair=False, rows=None):
+    c = DenseCall(act=act, pre=pre, d_x=x.ptr, d_norm_w=norm_w.ptr if norm_w else None, d_gate=gate.ptr if gate else None,
+                  w_offset=w_offset, eps=eps, head_dim=head_dim, M=M, K=K, n=len(lins), gelu_pair=int(gelu_pair),
+                  d_rows=rows.ptr if rows else None)
+    for i, (l, y, o) in enumerate(zip(lins, ys, outs)):
+        c.w[i], c.d_y[i], c.out[i] = C.pointer(l.s), (y.ptr if y else None), o
+    _check(lib().ornith_dense_rows(ctx.h, C.byref(c)), "dense_rows")
+
+
+def mlstm_state_floats(H, dim, vdim):
+    f = lib().ornith_mlstm_state_floats
+    f.restype = C.c_size_t
+    return int(f(H, dim, vdim))
+
+
+def mlstm(ctx, **kw):
+    """ornith_mlstm; buffers by the call's field names without d_."""
+    names = {n for n, _ in MlstmCall._fields_}
+    c = MlstmCall(**{(k if k in names else "d_" + k): (v.ptr if hasattr(v, "ptr") else v) for k, v in kw.items()})
+    _check(lib().ornith_mlstm(ctx.h, C.byref(c)), "mlstm")
+
+
+def diff_attn(ctx, **kw):
+    """ornith_diff_attn; buffers by the call's field names without d_."""
+    names = {n for n, _ in DiffAttnCall._fields_}
+    c = DiffAttnCall(**{(k if k in names else "d_" + k): (v.ptr if hasattr(v, "ptr") else v) for k, v in kw.items()})
+    _check(lib().ornith_diff_attn(ctx.h, C.byref(c)), "diff_attn")
