@@ -649,6 +649,365 @@ def config5(args, orn, ctx, synth, np, model, ws, cfg, dev_name):
     return line
 
 
+# ---- a layer-list design beside the closest existing model (`--design Pigodra`) -------------------
+MFMA_PEAK_TFLOPS = 2500.0
+DESIGN_SIZES = {
+    # width, mLSTM (heads, dim, vdim), attention (heads, kv_heads, dim, vdim, window, kept), ff
+    2048: dict(mlstm=(8, 128, 256), attn=(16, 4, 64, 128, 2048, 64), ff=5632),
+    4096: dict(mlstm=(8, 256, 512), attn=(32, 8, 64, 128, 4096, 128), ff=11008)}
+
+
+def design_config(width, layers, vocab):
+    """`layers` layers of a Pigodra model of that width, every fourth one attention, every second one
+    with a feed-forward."""
+    z = DESIGN_SIZES[width]
+    H, d, dv = z["mlstm"]
+    h, g, ad, av, win, keep = z["attn"]
+    out = []
+    for i in range(layers):
+        if i % 4 == 3:
+            lay = {"type": "attention", "mixer": {"heads": h, "kv_heads": g, "dim": ad, "vdim": av, "diff": 0.55,
+                                                  "scale": ad ** -0.5, "mask": {"size": win, "keep_first": keep},
+                                                  "rot": {"base": 250000.0, "dims": ad // 2, "scaling": {"factor": 2.0}}}}
+        else:
+            lay = {"type": "mlstm", "mixer": {"heads": H, "dim": d, "vdim": dv, "gate_cap": 15.0}}
+        lay["mlp"] = {"kind": "dense", "ff": z["ff"]} if i % 2 else None
+        out.append(lay)
+    return {"architecture": "Pigodra", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "layers": out}
+
+
+def design_tensors(cfg, rng, np):
+    """(name, bf16 bits) of every tensor of such a model, random (blocks of one normal draw)."""
+    import util
+    block = util.f32_to_bf16(rng.standard_normal(1 << 22).astype(np.float32))
+    f32 = util.bf16_to_f32(block)
+
+    def mat(*shape, std=1.0):
+        n = int(np.prod(shape))
+        at = int(rng.integers(0, 1 << 20))
+        src = np.resize(f32[at:], n) * np.float32(std)
+        return util.f32_to_bf16(src).reshape(shape)
+
+    W, V = cfg["width"], cfg["vocab"]
+    yield "embed", mat(V, W)
+    yield "head", mat(V, W, std=W ** -0.5)
+    yield "final.norm", mat(W, std=0.1)
+    for i, lay in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", lay["mixer"]
+        yield p + "norm1", mat(W, std=0.1)
+        if lay["type"] == "mlstm":
+            nk, nv = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+            for n, o in (("q", nk), ("k", nk), ("v", nv), ("g", nv), ("i", m["heads"]), ("f", m["heads"])):
+                yield p + "mix." + n, mat(o, W, std=W ** -0.5)
+            yield p + "mix.i.b", mat(m["heads"], std=0.5)
+            yield p + "mix.f.b", util.f32_to_bf16(np.full(m["heads"], 3.0, np.float32))
+            yield p + "mix.norm", util.f32_to_bf16(np.ones(nv, np.float32))
+            yield p + "mix.o", mat(W, nv, std=0.5 * nv ** -0.5)
+        else:
+            nv = m["heads"] * m["vdim"]
+            for n, o in (("q", m["heads"] * 2 * m["dim"]), ("k", m["kv_heads"] * 2 * m["dim"]),
+                         ("v", m["kv_heads"] * m["vdim"]), ("g", m["heads"])):
+                yield p + "mix." + n, mat(o, W, std=W ** -0.5)
+            for n in ("lq1", "lk1", "lq2", "lk2"):
+                yield p + "mix." + n, mat(m["dim"], std=0.1)
+            yield p + "mix.o", mat(W, nv, std=0.5 * nv ** -0.5)
+        if lay["mlp"]:
+            ff = lay["mlp"]["ff"]
+            yield p + "norm2", mat(W, std=0.1)
+            yield p + "mlp.gate", mat(ff, W, std=W ** -0.5)
+            yield p + "mlp.up", mat(ff, W, std=W ** -0.5)
+            yield p + "mlp.down", mat(W, ff, std=0.5 * ff ** -0.5)
+
+
+def design_model_rates(orn, ctx, np, model, vocab, ctx_len, n_gen, rows):
+    """Prefill and decode rates of a model through the plain generation loop: a ctx_len-token prompt in
+    calls of `rows` rows, then n_gen greedy tokens; the second of two runs."""
+    model.set_max_rows(rows)
+    caches = model.make_cache(ctx_len + n_gen + 16, 1)
+    prompt = np.random.default_rng(5).integers(0, vocab, ctx_len).astype(np.uint32)
+    out = None
+    for _ in range(2):
+        caches.reset()
+        mark = {}
+
+        def progress(done, total):
+            ctx.sync()
+            mark["p0" if done == 0 else "p1"] = time.perf_counter()
+
+        toks = orn.generate_step(model, caches, prompt, n_gen, prefill_step=rows, progress=progress)
+        ctx.sync()
+        t = time.perf_counter()
+        out = {"prompt": ctx_len, "prefill_tok_s": round(ctx_len / (mark["p1"] - mark["p0"]), 1),
+               "decode_tok_s": round(len(toks) / (t - mark["p1"]), 1)}
+    caches.close()
+    return out
+
+
+def design_kernels(orn, ctx, np, width, only=None):
+    """Every kernel of the design at `width` beside the like kernel of the closest existing model (the
+    gated-delta / gated-attention hybrid) at the same width, both in turn on this device: microseconds
+    a launch and the fraction of its roofline (HBM bytes, or matrix-core flops where those are the longer
+    time). Weights are cycled through copies of > 512 MB in all, so no launch finds them cached."""
+    import util
+    z = DESIGN_SIZES[width]
+    rng = np.random.default_rng(7)
+    block = rng.standard_normal(1 << 20).astype(np.float32)
+    W, res, garbage = width, [], []
+
+    def dev(shape, dtype="bf16", std=1.0):
+        a = np.resize(block, int(np.prod(shape))) * np.float32(std)
+        b = ctx.to_device(util.f32_to_bf16(a) if dtype == "bf16" else a)
+        garbage.append(b)
+        return b
+
+    def dense(O, K, copies):
+        out = []
+        for _ in range(copies):
+            w = orn.Linear(orn.LinearStruct(orn.LIN_DENSE, O, K, orn.KMatrixStruct(), dev((O, K), std=K ** -0.5).ptr, None, None), [])
+            out.append(w)
+        return out
+
+    def kq(kind, O, K, copies):
+        km = util.HostLinear.kq(rng, kind, O, K)
+        out = [km.dev(orn, ctx) for _ in range(copies)]
+        garbage.extend(out)
+        return out
+
+    def copies_for(nbytes):
+        return max(2, min(24, int(-(-(600 << 20) // nbytes))))
+
+    def row(name, us, nbytes, flops=0.0, peer=False, note=""):
+        t_hbm, t_mm = nbytes / (HBM_PEAK_GBS * 1e3), flops / (MFMA_PEAK_TFLOPS * 1e6)
+        r = {"kernel": name, "us": round(us, 2), "GB_s": round(nbytes / us / 1e3, 1), "roofline_frac": round(max(t_hbm, t_mm) / us, 4)}
+        if flops:
+            r["TFLOP_s"] = round(flops / us / 1e6, 1)
+            r["bound"] = "mfma" if t_mm > t_hbm else "hbm"
+        if note:
+            r["note"] = note
+        log(("    like: " if peer else "  ") + json.dumps(r))
+        return r
+
+    def pair(name, mine, peer, peer_name):
+        res.append({"what": name, "design": mine, "closest": dict(peer, kernel=peer_name) if peer else None,
+                    "times_as_far": round(peer["roofline_frac"] / mine["roofline_frac"], 2) if peer else None})
+
+    def want(name):
+        return only is None or any(o in name for o in only)
+
+    def calls(fn, made):
+        """fn(ctx, call) over call structures made beforehand (the host must not be what is timed)"""
+        return lambda i: fn(ctx, made[i % len(made)])
+
+    t_of = lambda fn, n=200, warm=20: _time_loop(ctx, fn, n, warm)
+    H, d, dv = z["mlstm"]
+    nk, nv = H * d, H * dv
+    h, g, ad, av, win, keep = z["attn"]
+    ff = z["ff"]
+    Hk, Hv = 16, 32                  # the hybrid's gated-delta heads (its kernels are made for this many channels)
+    vd = Hv * 128
+    D = 2 * Hk * 128 + vd
+
+    # ---- projections into the mixers and back, decode
+    for T in (1, 4):
+        if want("decode projections"):
+            shapes = [nk, nk, nv, nv, H, H]
+            nb = sum(shapes) * W * 2
+            n = copies_for(nb)
+            ws = [dense(o, W, n) for o in shapes]
+            x, wn = dev((T, W), "f32"), dev((W,), std=0.1)
+            ys = [ctx.alloc(T * o * 4) for o in shapes]
+            outs = [orn.OUT_ACT] * 4 + [orn.OUT_F32] * 2
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [w[i % n] for w in ws], ys, outs, pre=orn.PRE_NORM, norm_w=wn, w_offset=1.0) for i in range(n)]))
+            mine = row(f"norm + q, k, v, gates (T = {T})", us, nb + T * W * 4 + T * sum(shapes) * 2)
+            nb2 = int((D + vd) * W * 0.5625)
+            n2 = copies_for(nb2)
+            a, b = kq(util.Q4K, D, W, n2), kq(util.Q4K, vd, W, n2)
+            xb, yb, hb, nn = dev((T, W)), dev((T, W)), ctx.alloc(T * W * 2), ctx.alloc(T * W * 2)
+            w1 = dev((W,))
+            o1, o2 = ctx.alloc(T * D * 2), ctx.alloc(T * vd * 2)
+            us = t_of(lambda i: orn.add_rms_linear_multi(ctx, [a[i % n2], b[i % n2]], xb, yb, w1, 1e-6, T, hb, nn, [o1, o2]))
+            pair(f"decode projections in, T = {T}", mine, row("x", us, nb2 + T * (D + vd) * 2, peer=True), "add + norm + in_proj qkv, z (Q4_K)")
+            n = copies_for(W * nv * 2)
+            wo = dense(W, nv, n)
+            o, gate, wn2, xs = dev((T, nv), "f32"), dev((T, nv)), dev((nv,)), dev((T, W), "f32")
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, o, T, nv, [wo[i % n]], [xs], [orn.OUT_ADD], pre=orn.PRE_HEADS, norm_w=wn2, gate=gate, head_dim=dv) for i in range(n)]))
+            mine = row(f"head norm, gate + output projection + sum (T = {T})", us, W * nv * 2 + T * nv * 6)
+            n2 = copies_for(int(W * vd * 0.5625))
+            a = kq(util.Q4K, W, vd, n2)
+            xo, yo = dev((T, vd)), ctx.alloc(T * W * 2)
+            us = t_of(lambda i: ctx.linear_matmul(a[i % n2], xo, T, yo))
+            pair(f"decode projection out, T = {T}", mine, row("x", us, int(W * vd * 0.5625), peer=True), "out_proj (Q4_K)")
+            n = copies_for(2 * ff * W * 2)
+            wg, wu, wd = dense(ff, W, n), dense(ff, W, n), dense(W, ff, n)
+            act = ctx.alloc(T * ff * 2)
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [wg[i % n], wu[i % n]], [act, None], [0, 0], pre=orn.PRE_NORM, norm_w=wn, w_offset=1.0, gelu_pair=True) for i in range(n)]))
+            mine = row(f"norm + gate, up + gelu (T = {T})", us, 2 * ff * W * 2)
+            us2 = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, act, T, ff, [wd[i % n]], [xs], [orn.OUT_ADD]) for i in range(n)]))
+            mine2 = row(f"down + sum (T = {T})", us2, ff * W * 2)
+            if W == 2048:
+                moes = [util.HostMoe(rng, E=64).dev(orn, ctx) for _ in range(4)]
+                xm, om, im = dev((T, W)), ctx.alloc(T * W * 2), ctx.alloc(T * 8 * 4)
+                sm = ctx.alloc(T * 8 * 2)
+                ctx.moe_block(moes[0], xm, T, om, im, sm)
+                U = len(np.unique(im.download(np.uint32, (T * 8,))))
+                us = t_of(lambda i: ctx.moe_block(moes[i % 4], xm, T, om))
+                peer = row("x", us, (U + 1) * EXPERT_BYTES + 110_000, peer=True)
+                both = row(f"feed-forward, both launches (T = {T})", mine["us"] + mine2["us"], 3 * ff * W * 2)
+                pair(f"decode feed-forward, T = {T}", both, peer, "MoE block (router, up, down)")
+            else:
+                pair(f"decode feed-forward in, T = {T}", mine, None, None)
+                pair(f"decode feed-forward out, T = {T}", mine2, None, None)
+        if want("decode recurrence"):
+            sf = orn.mlstm_state_floats(H, d, dv)
+            layers = 24
+            slots = [dev((T + 2, sf), "f32", 0.01) for _ in range(layers)]
+            q, k, v, gi, gf, b1 = dev((T, nk)), dev((T, nk)), dev((T, nv)), dev((T, H), "f32"), dev((T, H), "f32"), dev((H,))
+            o = ctx.alloc(T * nv * 4)
+            us = t_of(calls(orn.mlstm, [orn.mlstm_call(act=orn.BF16, q=q, k=k, v=v, gi=gi, gf=gf, bi=b1, bf=b1, gate_cap=15.0, T=T, H=H, dim=d, vdim=dv,
+                                          state_in=slots[i % layers].ptr.value + ((i // layers) % 2) * sf * 4, slots=slots[i % layers], n_slots=T + 2,
+                                          first_slot=1 - (i // layers) % 2, snapshots=0, o=o) for i in range(2 * layers)]))
+            mine = row(f"mLSTM step (T = {T})", us, 2 * sf * 4 + T * (2 * nk + nv) * 2 + T * nv * 4)
+            sd = Hv * 128 * 128
+            st = [dev((2, sd), "f32", 0.01) for _ in range(layers)]
+            conv, qkv, cw, wa, wb, xn = dev((3, D)), dev((T, D)), dev((D, 4)), dev((Hv, W), std=0.02), dev((Hv, W), std=0.02), dev((T, W))
+            al, dt, nw, zz = dev((Hv,)), dev((Hv,)), dev((128,)), dev((T, vd))
+            ci, gated = ctx.alloc((3 + T) * D * 2), ctx.alloc(T * vd * 2)
+            us = t_of(lambda i: orn.gdn_step(ctx, conv, qkv, cw, wa, wb, xn, W, al, dt, T, 4, Hk, 128, Hv, 128, st[i % layers], st[i % layers], False, nw, zz, ci, gated))
+            pair(f"decode recurrence, T = {T}", mine, row("x", us, 2 * sd * 4 + 2 * Hv * W * 2 + T * (D + 2 * vd) * 2 + 7 * D * 2, peer=True), "gdn_step")
+        if want("decode attention"):
+            for ctx_len in (256, win + keep):
+                caps = 24
+                off = ctx_len - T
+                kc, vc = [dev((g, ctx_len, 2 * ad)) for _ in range(caps)], [dev((g, ctx_len, av)) for _ in range(caps)]
+                q, k, v, gt = dev((T, h * 2 * ad)), dev((T, g * 2 * ad)), dev((T, g * av)), dev((T, h), "f32")
+                co, si = ctx.rope_table(ctx_len, ad // 2, 250000.0)
+                out, qr = ctx.alloc(T * h * av * 2), ctx.alloc(T * h * 2 * ad * 2)
+                us = t_of(calls(orn.diff_attn, [orn.diff_attn_call(act=orn.BF16, q=q, k=k, v=v, gate=gt, cos=co, sin=si, rope_dims=ad // 2, table_npos=ctx_len, T=T, H=h, G=g,
+                                                  dim=ad, vdim=av, offset=off, cap=ctx_len, window=win, keep_first=keep, scale=ad ** -0.5, lam=0.5, diff=0.55,
+                                                  eps=1e-6, k_cache=kc[i % caps], v_cache=vc[i % caps], q_rot=qr, out=out) for i in range(caps)]))
+                mine = row(f"attention, {ctx_len} keys (T = {T})", us, g * ctx_len * (2 * ad + av) * 2)
+                Hq, Hkv = W // 128, max(2, W // 1024)
+                kc2, vc2 = [dev((Hkv, ctx_len, 256)) for _ in range(caps)], [dev((Hkv, ctx_len, 256)) for _ in range(caps)]
+                qg, kx, vx, qw = dev((T, Hq * 512)), dev((T, Hkv * 256)), dev((T, Hkv * 256)), dev((256,))
+                co2, si2 = ctx.rope_table(ctx_len, 64, 1e7)
+                qr2, out2 = ctx.alloc(T * Hq * 512), ctx.alloc(T * Hq * 512)
+                us = t_of(lambda i: ctx.attn_decode(qg, kx, vx, qw, qw, T, Hq, Hkv, 256, 64, 1e-6, co2, si2, ctx_len, off, ctx_len, 1 / 16.0, qr2,
+                                                    kc2[i % caps], vc2[i % caps], out2))
+                pair(f"decode attention, {ctx_len} keys, T = {T}", mine, row("x", us, Hkv * ctx_len * 1024, peer=True), "attn_decode")
+    # ---- prefill
+    for T in (512, 4096):
+        reps = dict(n=20, warm=3)
+        if want("prefill GEMM"):
+            shapes = [nk, nk, nv, nv, H, H]
+            ws = [dense(o, W, 1)[0] for o in shapes]
+            x, wn, rows_ = dev((T, W)), dev((W,), std=0.1), ctx.alloc(T * max(W, nv) * 2)
+            ys = [ctx.alloc(T * o * 4) for o in shapes]
+            outs = [orn.OUT_ACT] * 4 + [orn.OUT_F32] * 2
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, ws, ys, outs) for i in range(1)]), **reps)
+            mine = row(f"q, k, v, gates (T = {T})", us, sum(shapes) * W * 2 + T * W * 2 + T * sum(shapes) * 2, 2.0 * T * W * sum(shapes))
+            a, b = kq(util.Q4K, D, W, 1), kq(util.Q4K, vd, W, 1)
+            o1, o2 = ctx.alloc(T * D * 2), ctx.alloc(T * vd * 2)
+            us = t_of(lambda i: ctx.linear_matmul_multi([a[0], b[0]], x, T, [o1, o2]), **reps)
+            peer = row("x", us, int((D + vd) * W * 0.5625) + T * (D + vd + W) * 2, 2.0 * T * W * (D + vd), peer=True)
+            pair(f"prefill GEMM in, T = {T}", mine, peer, "in_proj qkv, z (Q4_K)")
+            wg, wu, wd = dense(ff, W, 1)[0], dense(ff, W, 1)[0], dense(W, ff, 1)[0]
+            act, xs = ctx.alloc(T * ff * 2), dev((T, W), "f32")
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [wg, wu], [act, None], [0, 0], gelu_pair=True) for i in range(1)]), **reps)
+            pair(f"prefill GEMM gate, up + gelu, T = {T}", row(f"gate, up + gelu (T = {T})", us, 2 * ff * W * 2 + T * (W + ff) * 2, 4.0 * T * W * ff), peer, "in_proj qkv, z (Q4_K)")
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, act, T, ff, [wd], [xs], [orn.OUT_ADD]) for i in range(1)]), **reps)
+            mine = row(f"down + sum (T = {T})", us, ff * W * 2 + T * (ff * 2 + W * 8), 2.0 * T * W * ff)
+            a = kq(util.Q4K, W, vd, 1)
+            xo, yo = dev((T, vd)), ctx.alloc(T * W * 2)
+            us = t_of(lambda i: ctx.linear_matmul(a[0], xo, T, yo), **reps)
+            pair(f"prefill GEMM down + sum, T = {T}", mine, row("x", us, int(W * vd * 0.5625) + T * (W + vd) * 2, 2.0 * T * W * vd, peer=True), "out_proj (Q4_K)")
+        if want("prefill rows"):
+            xs, wn, out = dev((T, W), "f32"), dev((W,), std=0.1), ctx.alloc(T * max(W, nv) * 2)
+            us = t_of(lambda i: orn.norm_rows(ctx, xs, wn, 1.0, T, W, 1e-6, orn.BF16, out), **reps)
+            mine = row(f"norm rows (T = {T})", us, T * W * 6)
+            xb, h1, w1 = dev((T, W)), ctx.alloc(T * W * 2), dev((W,))
+            us = t_of(lambda i: ctx.add_rms_norm(xb, xb, w1, T, W, 1e-6, h1, out), **reps)
+            pair(f"prefill rows: norm, T = {T}", mine, row("x", us, T * W * 8, peer=True), "add_rms_norm")
+            o, gate, wn2 = dev((T, nv), "f32"), dev((T, nv)), dev((nv,))
+            us = t_of(lambda i: orn.head_norm_gate(ctx, o, wn2, gate, T, H, dv, 1e-6, orn.BF16, out), **reps)
+            mine = row(f"head norm, gate (T = {T})", us, T * nv * 8)
+            yb, zb, w3, o3 = dev((T * Hv, 128)), dev((T * Hv, 128)), dev((128,)), ctx.alloc(T * vd * 2)
+            us = t_of(lambda i: ctx.rms_norm_gated(yb, w3, zb, T * Hv, 128, 1e-6, o3), **reps)
+            pair(f"prefill rows: head norm, T = {T}", mine, row("x", us, T * vd * 6, peer=True), "rms_norm_gated")
+        if want("prefill recurrence"):
+            sf = orn.mlstm_state_floats(H, d, dv)
+            slots = dev((2, sf), "f32", 0.01)
+            q, k, v, gi, gf, b1 = dev((T, nk)), dev((T, nk)), dev((T, nv)), dev((T, H), "f32"), dev((T, H), "f32"), dev((H,))
+            o = ctx.alloc(T * nv * 4)
+            us = t_of(calls(orn.mlstm, [orn.mlstm_call(act=orn.BF16, q=q, k=k, v=v, gi=gi, gf=gf, bi=b1, bf=b1, gate_cap=15.0, T=T, H=H, dim=d, vdim=dv,
+                                          state_in=slots.ptr.value + (i % 2) * sf * 4, slots=slots, n_slots=2, first_slot=1 - i % 2, snapshots=0, o=o) for i in range(2)]), **reps)
+            mine = row(f"mLSTM in chunks (T = {T})", us, T * (2 * nk + nv) * 2 + T * nv * 4 + 2 * sf * 4, 2.0 * T * H * (2 * d * dv + 32 * (d + dv)))
+            qd, kdd, vdd = dev((T, Hk * 128), std=0.09), dev((T, Hk * 128), std=0.09), dev((T, vd))
+            gd = ctx.to_device(np.resize(np.abs(block) * np.float32(0.1) + np.float32(0.85), T * Hv).clip(0.5, 0.999).astype(np.float32))
+            bd, yd, sd = dev((T, Hv), std=0.3), ctx.alloc(T * vd * 2), dev((1, Hv * 128 * 128), "f32", 0.01)
+            us = t_of(lambda i: ctx.gdn_recurrence(qd, kdd, vdd, gd, bd, sd, T, Hk, Hv, 128, 128, yd, sd, False), **reps)
+            pair(f"prefill recurrence, T = {T}", mine, row("x", us, T * (2 * Hk * 128 + 2 * vd) * 2 + 2 * Hv * 128 * 128 * 4,
+                                                           2.0 * T * Hv * (2 * 128 * 128 + 32 * 256), peer=True), "gdn_recurrence (chunked)")
+        if want("prefill attention"):
+            q, k, v, gt = dev((T, h * 2 * ad)), dev((T, g * 2 * ad)), dev((T, g * av)), dev((T, h), "f32")
+            co, si = ctx.rope_table(T, ad // 2, 250000.0)
+            kc, vc = dev((g, T, 2 * ad)), dev((g, T, av))
+            out, qr = ctx.alloc(T * h * av * 2), ctx.alloc(T * h * 2 * ad * 2)
+            i_ = np.arange(T)
+            seen = float(np.sum(np.minimum(i_ + 1, win) + np.minimum(np.maximum(i_ - win + 1, 0), keep)))
+            us = t_of(calls(orn.diff_attn, [orn.diff_attn_call(act=orn.BF16, q=q, k=k, v=v, gate=gt, cos=co, sin=si, rope_dims=ad // 2, table_npos=T, T=T, H=h, G=g, dim=ad,
+                                              vdim=av, offset=0, cap=T, window=win, keep_first=keep, scale=ad ** -0.5, lam=0.5, diff=0.55, eps=1e-6,
+                                              k_cache=kc, v_cache=vc, q_rot=qr, out=out) for i in range(1)]), **reps)
+            mine = row(f"attention (T = {T}, rotation and append included)", us, T * (h * 2 * ad + g * (2 * ad + av) + h * av) * 2, 2.0 * seen * h * 2 * (ad + av))
+            Hq, Hkv = W // 128, max(2, W // 1024)
+            qg, kx, vx, qw = dev((T, Hq * 512)), dev((T, Hkv * 256)), dev((T, Hkv * 256)), dev((256,))
+            co2, si2 = ctx.rope_table(T, 64, 1e7)
+            kc2, vc2 = dev((Hkv, T, 256)), dev((Hkv, T, 256))
+            qr2, out2 = ctx.alloc(T * Hq * 512), ctx.alloc(T * Hq * 512)
+            us = t_of(lambda i: ctx.attn_decode(qg, kx, vx, qw, qw, T, Hq, Hkv, 256, 64, 1e-6, co2, si2, T, 0, T, 1 / 16.0, qr2, kc2, vc2, out2), **reps)
+            full = T * (T + 1) / 2
+            pair(f"prefill attention, T = {T}", mine, row("x", us, T * (Hq * 512 + 2 * Hkv * 256 + Hq * 256) * 2, 2.0 * full * Hq * 512, peer=True),
+                 "attn_decode at prefill width (prep + attention)")
+    for b in garbage:
+        b.free()
+    return res
+
+
+def design_bench(args, orn, ctx, synth, np, dev_name):
+    """`--design Pigodra`: prefill and decode rates of the design at layer sizes of real models (random
+    weights) beside the closest existing model at equal width and depth, and kernel by kernel."""
+    out = {"design": args.design, "device": dev_name, "data": "synthetic", "models": [], "kernels": []}
+    layers, vocab = 8, 32768
+    only = args.design_kernels.split(",") if args.design_kernels else None
+    for width in (int(w) for w in args.design_widths.split(",")):
+        log(f"width {width}: kernels")
+        out["kernels"].append({"width": width, "rows": design_kernels(orn, ctx, np, width, only)})
+        if args.design_no_models:
+            continue
+        cfg = design_config(width, layers, vocab)
+        ws = orn.WeightStore(ctx)
+        for n, a in design_tensors(cfg, np.random.default_rng(3), np):
+            ws.put(n, a, orn.DT_BF16)
+        model = orn.TextModel.from_json(ctx, ws, cfg)
+        e = {"width": width, "layers": layers, "weight_bytes": ws.stats()[1],
+             "design": [design_model_rates(orn, ctx, np, model, vocab, n, 128, 4096) for n in (128, 4096)]}
+        model.close()
+        ws.close()
+        # the hybrid's stepwise kernels are made for hidden size 2048: its width there
+        if width == 2048:
+            qc = dict(synth.FULL, num_hidden_layers=layers, vocab_size=vocab, num_experts=64)
+            sm = synth.SynthModel(qc, seed=9, with_mtp=False, with_oracle=False)
+            ws = sm.upload(orn, ctx, drop_host=True)
+            model = orn.TextModel(ctx, ws, sm.text_config(orn))
+            e["closest"] = [design_model_rates(orn, ctx, np, model, vocab, n, 128, 4096) for n in (128, 4096)]
+            e["closest_weight_bytes"] = ws.stats()[1]
+            model.close()
+            ws.close()
+        log(json.dumps(e))
+        out["models"].append(e)
+    print(json.dumps(out), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -689,6 +1048,12 @@ def main():
                     help="only the phase time stamps of the expert pair (needs the library built with -DORN_TIMING)")
     ap.add_argument("--warm-cold", action="store_true",
                     help="only the mat-vec timings on re-used, unread and just-read weights")
+    ap.add_argument("--design", choices=("Pigodra",), default=None,
+                    help="instead of the metric's workload: prefill and decode rates of that design at layer sizes of real "
+                         "models (random weights) beside the closest existing model, and every kernel of both")
+    ap.add_argument("--design-widths", default="2048,4096", help="with --design: model widths, commas between them")
+    ap.add_argument("--design-kernels", default="", help="with --design: only kernels whose group contains one of these words")
+    ap.add_argument("--design-no-models", action="store_true", help="with --design: the kernels only")
     args = ap.parse_args()
     if args.gpus != 1:
         sys.exit("bench.py: this build runs on exactly one GPU (one process, one stream); "
@@ -705,6 +1070,8 @@ def main():
         return ceiling(orn, ctx, np)
     if args.warm_cold:
         return warm_cold(orn, ctx, np)
+    if args.design:
+        return design_bench(args, orn, ctx, synth, np, dev_name)
     cfg = dict(synth.FULL, num_hidden_layers=args.layers)
     t0 = time.time()
     sm = synth.SynthModel(cfg, seed=2025)

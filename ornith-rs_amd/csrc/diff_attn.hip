@@ -364,7 +364,7 @@ __device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t&
 // leave the registers. They go to the matrix cores as two bf16 parts, so they count as 32-bit numbers.
 // KD: 32-channel steps of a map; VT: 16-channel tiles of the values.
 template <int KD, int VT>
-__global__ __launch_bounds__(256) void diff_prefill_kernel(DaArgs p) {
+__global__ __launch_bounds__(256, VT <= 8 ? 2 : 1) void diff_prefill_kernel(DaArgs p) {
   constexpr int DP = KD * 32, LK = 2 * DP + 8;
   __shared__ __attribute__((aligned(16))) bf16_t Ks[BKV][LK];
   __shared__ __attribute__((aligned(16))) bf16_t Vt[VT * 16][LV];
@@ -385,10 +385,6 @@ __global__ __launch_bounds__(256) void diff_prefill_kernel(DaArgs p) {
         x = *reinterpret_cast<const d_u32x4*>(reinterpret_cast<const bf16_t*>(p.q_rot) + (((size_t)tc * p.H + h) * 2 + m) * p.dim + d);
       qf[m][kk] = __builtin_bit_cast(d_bf16x8, x);
     }
-  // padding channels of the tiles stay zero (nothing below writes them)
-  for (int i = tid; i < BKV * LK / 8; i += 256) reinterpret_cast<uint4*>(&Ks[0][0])[i] = make_uint4(0, 0, 0, 0);
-  for (int i = tid; i < VT * 16 * LV / 8; i += 256) reinterpret_cast<uint4*>(&Vt[0][0])[i] = make_uint4(0, 0, 0, 0);
-
   d_f32x4 acc[2][VT];
   float mx[2], sum[2];
 #pragma unroll
@@ -405,27 +401,50 @@ __global__ __launch_bounds__(256) void diff_prefill_kernel(DaArgs p) {
   const int lo = p.window > 0 ? max(0, first - p.window + 1) : 0, wb0 = lo / BKV, wb1 = last / BKV;
   const int hb = min((p.keep + BKV - 1) / BKV, wb0);
   const int nblocks = hb + wb1 - wb0 + 1;
-  const int kch = p.dim / 8, vch = p.vdim / 8;
-  for (int ib = 0; ib < nblocks; ++ib) {
-    const int j0 = (ib < hb ? ib : wb0 + ib - hb) * BKV;
-    __syncthreads();
-    for (int i = tid; i < BKV * 2 * kch; i += 256) {
-      const int r = i / (2 * kch), c = i % (2 * kch), m = c >= kch ? 1 : 0;
-      *reinterpret_cast<d_u32x4*>(&Ks[r][m * DP + 8 * (c - m * kch)]) =
-          *reinterpret_cast<const d_u32x4*>(kc + (size_t)min(j0 + r, last) * kd + 8 * c);
-    }
-    for (int i = tid; i < (BKV / 2) * vch; i += 256) {
-      const int oct = i % vch, pr = i / vch;
-      const d_u32x4 a = *reinterpret_cast<const d_u32x4*>(vc + (size_t)min(j0 + 2 * pr, last) * p.vdim + 8 * oct);
-      const d_u32x4 b = *reinterpret_cast<const d_u32x4*>(vc + (size_t)min(j0 + 2 * pr + 1, last) * p.vdim + 8 * oct);
-      const int at = (2 * pr & 32) + vt_pos(2 * pr & 31);
+  // this thread's pieces of a key block: 16 bytes of a key row each, and pairs of value rows, turned on
+  // their way into LDS; the next block's are asked for before this one is worked on
+  constexpr int KI = 2 * KD, VI = VT / 4;
+  d_u32x4 kreg[KI], vreg[VI][2];
+  // value piece e: which eight channels, which two rows. Four neighbouring lanes read 64 bytes of a row,
+  // and the sixteen row pairs of a wavefront keep its LDS writes two to a bank
+  auto v_oct = [](int e) { return (e & 3) + 4 * (e >> 7); };
+  auto v_pair = [](int e) { return (e >> 2) & 31; };
+  auto fetch = [&](int j0) {
+    const d_u32x4 zero = {0, 0, 0, 0};
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        *reinterpret_cast<uint32_t*>(&Vt[8 * oct + 2 * e][at]) = (a[e] & 0xffffu) | (b[e] << 16);
-        *reinterpret_cast<uint32_t*>(&Vt[8 * oct + 2 * e + 1][at]) = (a[e] >> 16) | (b[e] & 0xffff0000u);
+    for (int i = 0; i < KI; ++i) {
+      const int e = tid + 256 * i, r = e / (8 * KD), c = e % (8 * KD), m = c / (4 * KD), d = 8 * (c % (4 * KD));
+      kreg[i] = d < p.dim ? *reinterpret_cast<const d_u32x4*>(kc + (size_t)min(j0 + r, last) * kd + m * p.dim + d) : zero;
+    }
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+      const int e = tid + 256 * i, d = 8 * v_oct(e), r = 2 * v_pair(e);
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+        vreg[i][b] = d < p.vdim ? *reinterpret_cast<const d_u32x4*>(vc + (size_t)min(j0 + r + b, last) * p.vdim + d) : zero;
+    }
+  };
+  auto block_at = [&](int ib) { return (ib < hb ? ib : wb0 + ib - hb) * BKV; };
+  fetch(block_at(0));
+  for (int ib = 0; ib < nblocks; ++ib) {
+    const int j0 = block_at(ib);
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < KI; ++i) {
+      const int e = tid + 256 * i, r = e / (8 * KD), c = e % (8 * KD);
+      *reinterpret_cast<d_u32x4*>(&Ks[r][8 * c]) = kreg[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+      const int e = tid + 256 * i, d = 8 * v_oct(e), r = 2 * v_pair(e), at = (r & 32) + vt_pos(r & 31);
+#pragma unroll
+      for (int w = 0; w < 4; ++w) {
+        *reinterpret_cast<uint32_t*>(&Vt[d + 2 * w][at]) = (vreg[i][0][w] & 0xffffu) | (vreg[i][1][w] << 16);
+        *reinterpret_cast<uint32_t*>(&Vt[d + 2 * w + 1][at]) = (vreg[i][0][w] >> 16) | (vreg[i][1][w] & 0xffff0000u);
       }
     }
     __syncthreads();
+    if (ib + 1 < nblocks) fetch(block_at(ib + 1));
     // scores: key j0 + 16 kt + 4 lg + r of this lane's query
     d_f32x4 sc[2][4];
 #pragma unroll

@@ -293,7 +293,9 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(ScanArgs p) {
 #pragma unroll
   for (int i = 0; i < 8; ++i) ones[i] = (__bf16)1.0f;
 
-  const int oct = tid & 7, pair = tid >> 3;  // eight channels, two tokens
+  // eight channels, two tokens: four neighbouring lanes read 64 bytes of a row, and the sixteen token
+  // pairs of a wavefront keep its LDS writes two to a bank
+  const int oct = (tid & 3) + 4 * (tid >> 7), pair = (tid >> 2) & 31;
   const bool kin = d0 + 8 * oct < p.dim, vin = j0 + 8 * oct < p.vdim;
   const bf16_t* kp = p.k + (size_t)h * p.dim + d0 + 8 * oct;
   const bf16_t* vp = p.v + (size_t)h * p.vdim + j0 + 8 * oct;
@@ -410,7 +412,7 @@ __global__ __launch_bounds__(256) void mlstm_out_kernel(OutArgs p) {
   const int t0 = c * C;
   // values, turned: a thread brings two tokens of eight channels
   for (int i = tid; i < (VB / 8) * (C / 2); i += 256) {
-    const int oct = i % (VB / 8), pair = i / (VB / 8);
+    const int oct = (i & 3) + 4 * (i >> 7), pair = (i >> 2) & 31;  // as in the scan
     const m_u32x4 zero = {0, 0, 0, 0};
     m_u32x4 a = zero, b = zero;
     if (jb + 8 * oct < p.vdim) {

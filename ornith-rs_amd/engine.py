@@ -700,13 +700,19 @@ class DiffAttnCall(C.Structure):
         (n, C.c_void_p) for n in ("d_k_cache", "d_v_cache", "d_q_rot", "d_out")]
 
 
-def dense_rows(ctx, act, x, M, K, lins, ys, outs, pre=PRE_NONE, norm_w=None, gate=None, w_offset=0.0, eps=1e-6, head_dim=0,
+def dense_call(act, x, M, K, lins, ys, outs, pre=PRE_NONE, norm_w=None, gate=None, w_offset=0.0, eps=1e-6, head_dim=0,
                gelu_pair=False, rows=None):
     c = DenseCall(act=act, pre=pre, d_x=x.ptr, d_norm_w=norm_w.ptr if norm_w else None, d_gate=gate.ptr if gate else None,
                   w_offset=w_offset, eps=eps, head_dim=head_dim, M=M, K=K, n=len(lins), gelu_pair=int(gelu_pair),
                   d_rows=rows.ptr if rows else None)
     for i, (l, y, o) in enumerate(zip(lins, ys, outs)):
         c.w[i], c.d_y[i], c.out[i] = C.pointer(l.s), (y.ptr if y else None), o
+    return c
+
+
+def dense_rows(ctx, *a, **kw):
+    """ornith_dense_rows; the arguments of dense_call, or a call made earlier."""
+    c = a[0] if a and isinstance(a[0], DenseCall) else dense_call(*a, **kw)
     _check(lib().ornith_dense_rows(ctx.h, C.byref(c)), "dense_rows")
 
 
@@ -716,15 +722,39 @@ def mlstm_state_floats(H, dim, vdim):
     return int(f(H, dim, vdim))
 
 
-def mlstm(ctx, **kw):
-    """ornith_mlstm; buffers by the call's field names without d_."""
-    names = {n for n, _ in MlstmCall._fields_}
-    c = MlstmCall(**{(k if k in names else "d_" + k): (v.ptr if hasattr(v, "ptr") else v) for k, v in kw.items()})
+def _fields(cls, kw):
+    names = {n for n, _ in cls._fields_}
+    return cls(**{(k if k in names else "d_" + k): (v.ptr if hasattr(v, "ptr") else v) for k, v in kw.items()})
+
+
+def mlstm(ctx, call=None, **kw):
+    """ornith_mlstm; buffers by the call's field names without d_ (or a MlstmCall made earlier)."""
+    c = call or _fields(MlstmCall, kw)
     _check(lib().ornith_mlstm(ctx.h, C.byref(c)), "mlstm")
 
 
-def diff_attn(ctx, **kw):
-    """ornith_diff_attn; buffers by the call's field names without d_."""
-    names = {n for n, _ in DiffAttnCall._fields_}
-    c = DiffAttnCall(**{(k if k in names else "d_" + k): (v.ptr if hasattr(v, "ptr") else v) for k, v in kw.items()})
+def mlstm_call(**kw):
+    return _fields(MlstmCall, kw)
+
+
+def diff_attn_call(**kw):
+    return _fields(DiffAttnCall, kw)
+
+
+def diff_attn(ctx, call=None, **kw):
+    """ornith_diff_attn; buffers by the call's field names without d_ (or a DiffAttnCall made earlier)."""
+    c = call or _fields(DiffAttnCall, kw)
     _check(lib().ornith_diff_attn(ctx.h, C.byref(c)), "diff_attn")
+
+
+def norm_rows(ctx, x, w, w_offset, rows, n, eps, act, out):
+    _check(lib().ornith_norm_rows(ctx.h, x.ptr, w.ptr, C.c_float(w_offset), rows, n, C.c_float(eps), act, out.ptr), "norm_rows")
+
+
+def head_norm_gate(ctx, x, w, gate, rows, heads, head_dim, eps, act, out):
+    _check(lib().ornith_head_norm_gate(ctx.h, x.ptr, w.ptr, gate.ptr, rows, heads, head_dim, C.c_float(eps), act, out.ptr),
+           "head_norm_gate")
+
+
+def embed_rows(ctx, table, ids, n, scale, out):
+    _check(lib().ornith_embed_rows(ctx.h, C.byref(table.s), ids.ptr, n, C.c_float(scale), out.ptr), "embed_rows")
