@@ -317,31 +317,35 @@ int run_decode(ornith_ctx* ctx, const DaArgs& p) {
 }
 
 // ---- prefill widths ----------------------------------------------------------------------
-// queries rotated into q_rot, keys rotated and values as they are into the cache; a thread takes two
-// elements (one pair), grid.x the rows
+// queries rotated into q_rot, keys rotated and values as they are into the cache; a thread takes eight
+// elements (four pairs), grid.x the rows
 __global__ __launch_bounds__(NT) void diff_prep_kernel(DaArgs p) {
-  const int t = blockIdx.x, pos = p.offset + t, pairs = p.dim / 2;
-  const int nq = p.H * 2 * pairs, nk = p.G * 2 * pairs, nv = p.G * p.vdim / 2;
+  const int t = blockIdx.x, pos = p.offset + t, per = p.dim / 8, vper = p.vdim / 8;
+  const int nq = p.H * 2 * per, nk = p.G * 2 * per, nv = p.G * vper;
+  const float* ct = p.cos_t + (size_t)pos * p.rope_half;
+  const float* st = p.sin_t + (size_t)pos * p.rope_half;
   for (int i = threadIdx.x; i < nq + nk + nv; i += NT) {
     if (i >= nq + nk) {
-      const int e = 2 * (i - nq - nk), g = e / p.vdim, c = e % p.vdim;
-      *reinterpret_cast<uint32_t*>(reinterpret_cast<bf16_t*>(p.v_cache) + ((size_t)g * p.cap + pos) * p.vdim + c) =
-          *reinterpret_cast<const uint32_t*>(reinterpret_cast<const bf16_t*>(p.v) + (size_t)t * p.G * p.vdim + e);
+      const int e = i - nq - nk, g = e / vper, c = 8 * (e % vper);
+      *reinterpret_cast<uint4*>(reinterpret_cast<bf16_t*>(p.v_cache) + ((size_t)g * p.cap + pos) * p.vdim + c) =
+          *reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(p.v) + ((size_t)t * p.G + g) * p.vdim + c);
       continue;
     }
     const bool is_q = i < nq;
-    const int a = is_q ? i : i - nq, row = a / pairs, d = 2 * (a % pairs);
+    const int a = is_q ? i : i - nq, row = a / per, d = 8 * (a % per);
     const bf16_t* src = is_q ? reinterpret_cast<const bf16_t*>(p.q) + (size_t)t * p.H * 2 * p.dim
                              : reinterpret_cast<const bf16_t*>(p.k) + (size_t)t * p.G * 2 * p.dim;
-    uint32_t w = *reinterpret_cast<const uint32_t*>(src + (size_t)row * p.dim + d);
-    if (d < 2 * p.rope_half) {
-      const size_t at = (size_t)pos * p.rope_half + (d >> 1);
-      const float c = p.cos_t[at], s = p.sin_t[at], x = dm_bf2f_lo(w), y = dm_bf2f_hi(w);
-      w = dm_f2bf2(dm_fma(-y, s, x * c), dm_fma(x, s, y * c));
-    }
+    const uint4 in = *reinterpret_cast<const uint4*>(src + (size_t)row * p.dim + d);
+    uint32_t w[4] = {in.x, in.y, in.z, in.w};
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (d + 2 * e < 2 * p.rope_half) {
+        const float c = ct[(d >> 1) + e], s = st[(d >> 1) + e], x = dm_bf2f_lo(w[e]), y = dm_bf2f_hi(w[e]);
+        w[e] = dm_f2bf2(dm_fma(-y, s, x * c), dm_fma(x, s, y * c));
+      }
     bf16_t* dst = is_q ? reinterpret_cast<bf16_t*>(p.q_rot) + ((size_t)t * p.H * 2 + row) * p.dim + d
                        : reinterpret_cast<bf16_t*>(p.k_cache) + ((size_t)(row >> 1) * p.cap + pos) * 2 * p.dim + (row & 1) * p.dim + d;
-    *reinterpret_cast<uint32_t*>(dst) = w;
+    *reinterpret_cast<uint4*>(dst) = make_uint4(w[0], w[1], w[2], w[3]);
   }
 }
 
@@ -364,7 +368,7 @@ __device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t&
 // leave the registers. They go to the matrix cores as two bf16 parts, so they count as 32-bit numbers.
 // KD: 32-channel steps of a map; VT: 16-channel tiles of the values.
 template <int KD, int VT>
-__global__ __launch_bounds__(256, VT <= 8 ? 2 : 1) void diff_prefill_kernel(DaArgs p) {
+__global__ __launch_bounds__(256, VT <= 8 && KD <= 2 ? 2 : 1) void diff_prefill_kernel(DaArgs p) {
   constexpr int DP = KD * 32, LK = 2 * DP + 8;
   __shared__ __attribute__((aligned(16))) bf16_t Ks[BKV][LK];
   __shared__ __attribute__((aligned(16))) bf16_t Vt[VT * 16][LV];
@@ -383,6 +387,7 @@ __global__ __launch_bounds__(256, VT <= 8 ? 2 : 1) void diff_prefill_kernel(DaAr
       d_u32x4 x = {0, 0, 0, 0};
       if (d < p.dim)
         x = *reinterpret_cast<const d_u32x4*>(reinterpret_cast<const bf16_t*>(p.q_rot) + (((size_t)tc * p.H + h) * 2 + m) * p.dim + d);
+      if (p.scale < 0.f) x ^= 0x80008000u;  // the scale's sign, so that a row's largest score is its largest product
       qf[m][kk] = __builtin_bit_cast(d_bf16x8, x);
     }
   d_f32x4 acc[2][VT];
@@ -396,92 +401,160 @@ __global__ __launch_bounds__(256, VT <= 8 ? 2 : 1) void diff_prefill_kernel(DaAr
   }
   const bf16_t* kc = reinterpret_cast<const bf16_t*>(p.k_cache) + (size_t)g * p.cap * kd;
   const bf16_t* vc = reinterpret_cast<const bf16_t*>(p.v_cache) + (size_t)g * p.cap * p.vdim;
-  const float s2 = p.scale * 1.44269504088896341f;
+  const float s2 = __builtin_fmaxf(__builtin_fabsf(p.scale) * 1.44269504088896341f, 1e-30f);
   // key blocks: the kept first tokens that lie before the window of the first row, then the window
   const int lo = p.window > 0 ? max(0, first - p.window + 1) : 0, wb0 = lo / BKV, wb1 = last / BKV;
   const int hb = min((p.keep + BKV - 1) / BKV, wb0);
   const int nblocks = hb + wb1 - wb0 + 1;
   // this thread's pieces of a key block: 16 bytes of a key row each, and pairs of value rows, turned on
-  // their way into LDS; the next block's are asked for before this one is worked on
+  // their way into LDS; the next block's are asked for before this one is worked on. Value piece e: four
+  // neighbouring lanes read 64 bytes of a row, and the sixteen row pairs of a wavefront keep its LDS
+  // writes two to a bank. Offsets inside a block are made once: a block costs the vector ALU nothing here.
   constexpr int KI = 2 * KD, VI = VT / 4;
   d_u32x4 kreg[KI], vreg[VI][2];
-  // value piece e: which eight channels, which two rows. Four neighbouring lanes read 64 bytes of a row,
-  // and the sixteen row pairs of a wavefront keep its LDS writes two to a bank
-  auto v_oct = [](int e) { return (e & 3) + 4 * (e >> 7); };
-  auto v_pair = [](int e) { return (e >> 2) & 31; };
+  int krow[KI], kcol[KI], vrow[VI], vcol[VI], koff[KI], voff[VI][2];
+  bool kin[KI], vin[VI];
+#pragma unroll
+  for (int i = 0; i < KI; ++i) {
+    const int e = tid + 256 * i, c = e % (8 * KD), m = c / (4 * KD), d = 8 * (c % (4 * KD));
+    krow[i] = e / (8 * KD);
+    kin[i] = d < p.dim;
+    kcol[i] = kin[i] ? m * p.dim + d : 0;
+    koff[i] = krow[i] * kd + kcol[i];
+  }
+#pragma unroll
+  for (int i = 0; i < VI; ++i) {
+    const int e = tid + 256 * i, d = 8 * ((e & 3) + 4 * (e >> 7));
+    vrow[i] = 2 * ((e >> 2) & 31);
+    vin[i] = d < p.vdim;
+    vcol[i] = vin[i] ? d : 0;
+#pragma unroll
+    for (int b = 0; b < 2; ++b) voff[i][b] = (vrow[i] + b) * p.vdim + vcol[i];
+  }
   auto fetch = [&](int j0) {
-    const d_u32x4 zero = {0, 0, 0, 0};
+    const bf16_t* kb = kc + (size_t)j0 * kd;
+    const bf16_t* vb = vc + (size_t)j0 * p.vdim;
+    if (j0 + BKV - 1 <= last) {
 #pragma unroll
-    for (int i = 0; i < KI; ++i) {
-      const int e = tid + 256 * i, r = e / (8 * KD), c = e % (8 * KD), m = c / (4 * KD), d = 8 * (c % (4 * KD));
-      kreg[i] = d < p.dim ? *reinterpret_cast<const d_u32x4*>(kc + (size_t)min(j0 + r, last) * kd + m * p.dim + d) : zero;
-    }
+      for (int i = 0; i < KI; ++i) kreg[i] = *reinterpret_cast<const d_u32x4*>(kb + koff[i]);
 #pragma unroll
-    for (int i = 0; i < VI; ++i) {
-      const int e = tid + 256 * i, d = 8 * v_oct(e), r = 2 * v_pair(e);
+      for (int i = 0; i < VI; ++i)
 #pragma unroll
-      for (int b = 0; b < 2; ++b)
-        vreg[i][b] = d < p.vdim ? *reinterpret_cast<const d_u32x4*>(vc + (size_t)min(j0 + r + b, last) * p.vdim + d) : zero;
+        for (int b = 0; b < 2; ++b) vreg[i][b] = *reinterpret_cast<const d_u32x4*>(vb + voff[i][b]);
+    } else {  // the block the call's last keys end in: nothing is read past them
+      const int n = last - j0;
+#pragma unroll
+      for (int i = 0; i < KI; ++i) kreg[i] = *reinterpret_cast<const d_u32x4*>(kb + min(krow[i], n) * kd + kcol[i]);
+#pragma unroll
+      for (int i = 0; i < VI; ++i)
+#pragma unroll
+        for (int b = 0; b < 2; ++b) vreg[i][b] = *reinterpret_cast<const d_u32x4*>(vb + min(vrow[i] + b, n) * p.vdim + vcol[i]);
     }
   };
   auto block_at = [&](int ib) { return (ib < hb ? ib : wb0 + ib - hb) * BKV; };
+  const unsigned win = p.window > 0 ? (unsigned)p.window : 0x7fffffffu;
+  // padding channels of the tiles stay zero
+  if (p.dim < DP)
+    for (int i = tid; i < BKV * LK / 8; i += 256) reinterpret_cast<uint4*>(&Ks[0][0])[i] = make_uint4(0, 0, 0, 0);
+  if (p.vdim < VT * 16)
+    for (int i = tid; i < VT * 16 * LV / 8; i += 256) reinterpret_cast<uint4*>(&Vt[0][0])[i] = make_uint4(0, 0, 0, 0);
   fetch(block_at(0));
   for (int ib = 0; ib < nblocks; ++ib) {
     const int j0 = block_at(ib);
     __syncthreads();
 #pragma unroll
-    for (int i = 0; i < KI; ++i) {
-      const int e = tid + 256 * i, r = e / (8 * KD), c = e % (8 * KD);
-      *reinterpret_cast<d_u32x4*>(&Ks[r][8 * c]) = kreg[i];
-    }
+    for (int i = 0; i < KI; ++i)
+      if (kin[i]) *reinterpret_cast<d_u32x4*>(&Ks[krow[i]][8 * ((tid + 256 * i) % (8 * KD))]) = kreg[i];
 #pragma unroll
-    for (int i = 0; i < VI; ++i) {
-      const int e = tid + 256 * i, d = 8 * v_oct(e), r = 2 * v_pair(e), at = (r & 32) + vt_pos(r & 31);
+    for (int i = 0; i < VI; ++i)
+      if (vin[i]) {
+        const int at = (vrow[i] & 32) + vt_pos(vrow[i] & 31);
 #pragma unroll
-      for (int w = 0; w < 4; ++w) {
-        *reinterpret_cast<uint32_t*>(&Vt[d + 2 * w][at]) = (vreg[i][0][w] & 0xffffu) | (vreg[i][1][w] << 16);
-        *reinterpret_cast<uint32_t*>(&Vt[d + 2 * w + 1][at]) = (vreg[i][0][w] >> 16) | (vreg[i][1][w] & 0xffff0000u);
+        for (int w = 0; w < 4; ++w) {
+          *reinterpret_cast<uint32_t*>(&Vt[vcol[i] + 2 * w][at]) = __builtin_amdgcn_perm(vreg[i][1][w], vreg[i][0][w], 0x05040100u);
+          *reinterpret_cast<uint32_t*>(&Vt[vcol[i] + 2 * w + 1][at]) = __builtin_amdgcn_perm(vreg[i][1][w], vreg[i][0][w], 0x07060302u);
+        }
       }
-    }
     __syncthreads();
     if (ib + 1 < nblocks) fetch(block_at(ib + 1));
-    // scores: key j0 + 16 kt + 4 lg + r of this lane's query
+    // scores: key j0 + 16 kt + 4 lg + r of this lane's query. All fragments of a map are asked for before
+    // the first is used, the second map's before the first map's products (left to itself the compiler
+    // puts every read right before its use, an LDS latency a product)
     d_f32x4 sc[2][4];
+    constexpr int GK = KD <= 2 ? 4 : VT <= 8 ? 2 : 1;  // key tiles asked for together
+    d_bf16x8 kf[2][GK][KD];
+    auto key_frags = [&](int step) {  // step: map, then group of key tiles
+      const int m = step / (4 / GK), k0 = step % (4 / GK) * GK;
 #pragma unroll
-    for (int m = 0; m < 2; ++m)
+      for (int kt = 0; kt < GK; ++kt)
 #pragma unroll
-      for (int kt = 0; kt < 4; ++kt) {
-        d_f32x4 s = {0.f, 0.f, 0.f, 0.f};
+        for (int kk = 0; kk < KD; ++kk)
+          kf[step & 1][kt][kk] = *reinterpret_cast<const d_bf16x8*>(&Ks[16 * (k0 + kt) + l16][m * DP + 32 * kk + 8 * lg]);
+    };
+    auto products = [&](int step) {
+      const int m = step / (4 / GK), k0 = step % (4 / GK) * GK;
 #pragma unroll
-        for (int kk = 0; kk < KD; ++kk) {
-          const d_bf16x8 kf = *reinterpret_cast<const d_bf16x8*>(&Ks[16 * kt + l16][m * DP + 32 * kk + 8 * lg]);
-          s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[m][kk], s, 0, 0, 0);
-        }
-        sc[m][kt] = s;
-      }
+      for (int kt = 0; kt < GK; ++kt) sc[m][k0 + kt] = d_f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kk = 0; kk < KD; ++kk)
+#pragma unroll
+        for (int kt = 0; kt < GK; ++kt)
+          sc[m][k0 + kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[step & 1][kt][kk], qf[m][kk], sc[m][k0 + kt], 0, 0, 0);
+    };
+    constexpr int STEPS = 2 * (4 / GK);
+    key_frags(0);
+#pragma unroll
+    for (int step = 0; step < STEPS; ++step) {
+      __builtin_amdgcn_sched_barrier(0);
+      if (step + 1 < STEPS) key_frags(step + 1);
+      __builtin_amdgcn_sched_barrier(0);
+      products(step);
+    }
+    // the first value fragments come in under the softmax
+    constexpr int AHEAD = VT <= 8 ? 2 : 1;
+    d_bf16x8 vf[AHEAD + 1][2];
+    auto value_frags = [&](int v) {
+#pragma unroll
+      for (int a = 0; a < 2; ++a) vf[v % (AHEAD + 1)][a] = *reinterpret_cast<const d_bf16x8*>(&Vt[16 * v + l16][32 * a + 8 * lg]);
+    };
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int v = 0; v < AHEAD; ++v) value_frags(v);
+    __builtin_amdgcn_sched_barrier(0);
     // every row of the tile sees the whole block: inside everyone's window, before everyone
     const bool whole = j0 + BKV - 1 <= first && (p.window <= 0 || last - j0 < p.window || j0 + BKV <= p.keep);
-    d_bf16x8 ph[2][2], pl[2][2];
-#pragma unroll
-    for (int m = 0; m < 2; ++m) {
-      float top = -DM_INF;
+    if (!whole) {
+      const bool kept = j0 < p.keep;
 #pragma unroll
       for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          float s = sc[m][kt][r] * s2;
-          if (!whole) {
-            const int j = j0 + 16 * kt + 4 * lg + r;
-            const bool see = j <= pos && (p.window <= 0 || pos - j < p.window || j < p.keep);
-            s = see ? s : -DM_INF;
-          }
-          sc[m][kt][r] = s;
-          top = __builtin_fmaxf(top, s);
+          const int j = j0 + 16 * kt + 4 * lg + r, back = pos - j;
+          bool see = (unsigned)back < win;
+          if (kept) see = see | ((j < p.keep) & (back >= 0));
+#pragma unroll
+          for (int m = 0; m < 2; ++m) sc[m][kt][r] = see ? sc[m][kt][r] : -DM_INF;
         }
-      top = dm_max_groups16(top);
-      const float mn = __builtin_fmaxf(mx[m], top), ref = mn == -DM_INF ? 0.f : mn;
-      const float alpha = dm_exp2_hw(mx[m] - ref);
-      mx[m] = mn;
+    }
+    d_bf16x8 ph[2][2], pl[2][2];
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      float top = sc[m][0][0];
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) top = __builtin_fmaxf(top, sc[m][kt][r]);
+      top = dm_max_groups16(top) * s2;
+      // the reference point of a row's exponentials moves only when its maximum has grown by 2^8 (the
+      // weights stay below 2^8 then, the sums far inside fp32's range)
+      if (__any(top > mx[m] + 8.0f)) {
+        const float mn = __builtin_fmaxf(mx[m], top), alpha = mn == -DM_INF ? 0.f : dm_exp2_hw(mx[m] - mn);
+        mx[m] = mn;
+        sum[m] *= alpha;
+#pragma unroll
+        for (int v = 0; v < VT; ++v) acc[m][v] *= alpha;
+      }
+      const float ref = mx[m] == -DM_INF ? 0.f : mx[m];
       float l = 0.f;
 #pragma unroll
       for (int a = 0; a < 2; ++a) {
@@ -491,7 +564,7 @@ __global__ __launch_bounds__(256, VT <= 8 ? 2 : 1) void diff_prefill_kernel(DaAr
           float e[4];
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
-            e[r] = dm_exp2_hw(sc[m][2 * a + b][r] - ref);
+            e[r] = dm_exp2_hw(dm_fma(sc[m][2 * a + b][r], s2, -ref));
             l += e[r];
           }
           split2(e[0], e[1], hi[2 * b], lo2[2 * b]);
@@ -501,23 +574,22 @@ __global__ __launch_bounds__(256, VT <= 8 ? 2 : 1) void diff_prefill_kernel(DaAr
         ph[m][a] = __builtin_bit_cast(d_bf16x8, hv);
         pl[m][a] = __builtin_bit_cast(d_bf16x8, lv);
       }
-      sum[m] = dm_fma(sum[m], alpha, l);
-      if (__any(alpha != 1.0f)) {
-#pragma unroll
-        for (int v = 0; v < VT; ++v) acc[m][v] *= alpha;
-      }
+      sum[m] += l;
     }
 #pragma unroll
-    for (int v = 0; v < VT; ++v)
+    for (int v = 0; v < VT; ++v) {
+      if (v + AHEAD < VT) value_frags(v + AHEAD);
+      __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int a = 0; a < 2; ++a) {
-        const d_bf16x8 vf = *reinterpret_cast<const d_bf16x8*>(&Vt[16 * v + l16][32 * a + 8 * lg]);
+      for (int a = 0; a < 2; ++a)
 #pragma unroll
-        for (int m = 0; m < 2; ++m) {
-          acc[m][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[m][a], acc[m][v], 0, 0, 0);
-          acc[m][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[m][a], acc[m][v], 0, 0, 0);
-        }
-      }
+        for (int m = 0; m < 2; ++m) acc[m][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[v % (AHEAD + 1)][a], ph[m][a], acc[m][v], 0, 0, 0);
+#pragma unroll
+      for (int a = 0; a < 2; ++a)
+#pragma unroll
+        for (int m = 0; m < 2; ++m) acc[m][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[v % (AHEAD + 1)][a], pl[m][a], acc[m][v], 0, 0, 0);
+      __builtin_amdgcn_sched_barrier(0);
+    }
   }
   // a1 - lambda a2, its norm over the head (padding channels are zero), the gate
   const float i1 = 1.0f / dm_sum_groups16(sum[0]), i2 = p.lambda / dm_sum_groups16(sum[1]);

@@ -26,8 +26,12 @@ def gelu_tanh(z):
     return 0.5 * z * (1.0 + np.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3)))
 
 
-def dense_ff(h, gate, up, down):
-    return (gelu_tanh(h @ gate.T) * (h @ up.T)) @ down.T
+def exact(x):
+    return x
+
+
+def dense_ff(h, gate, up, down, r=exact):
+    return r(gelu_tanh(h @ gate.T) * (h @ up.T)) @ down.T
 
 
 def soft_cap(x, cap):
@@ -53,13 +57,13 @@ def mlstm_cell(q, k, v, log_i, log_f, state):
     return out, (S, n, m)
 
 
-def mlstm_mixer(h, w, p, mx, eps, state):
-    """state: list of per-head cell states or None for a new sequence."""
+def mlstm_mixer(h, w, p, mx, eps, state, r=exact):
+    """state: list of per-head cell states or None for a new sequence. r: see Run."""
     H, d, dv, cap = mx["heads"], mx["dim"], mx["vdim"], mx["gate_cap"]
     T = len(h)
-    q = (h @ w[p + "q"].T).reshape(T, H, d) * d ** -0.5
-    k = (h @ w[p + "k"].T).reshape(T, H, d)
-    v = (h @ w[p + "v"].T).reshape(T, H, dv)
+    q = r(h @ w[p + "q"].T).reshape(T, H, d) * d ** -0.5
+    k = r(h @ w[p + "k"].T).reshape(T, H, d)
+    v = r(h @ w[p + "v"].T).reshape(T, H, dv)
     li = soft_cap(h @ w[p + "i"].T + w[p + "i.b"], cap)
     lf = log_sigmoid(soft_cap(h @ w[p + "f"].T + w[p + "f.b"], cap))
     state = state or [(np.zeros((d, dv)), np.zeros(d), 0.0) for _ in range(H)]
@@ -67,7 +71,7 @@ def mlstm_mixer(h, w, p, mx, eps, state):
     for a in range(H):
         out[:, a], s = mlstm_cell(q[:, a], k[:, a], v[:, a], li[:, a], lf[:, a], state[a])
         new.append(s)
-    out = rms(out, eps).reshape(T, H * dv) * w[p + "norm"] * sigmoid(h @ w[p + "g"].T)
+    out = r(rms(out, eps).reshape(T, H * dv) * w[p + "norm"] * sigmoid(r(h @ w[p + "g"].T)))
     return out @ w[p + "o"].T, new
 
 
@@ -99,24 +103,24 @@ def diff_lambda(lq1, lk1, lq2, lk2, diff):
     return math.exp(float(np.sum(lq1 * lk1))) - math.exp(float(np.sum(lq2 * lk2))) + diff
 
 
-def diff_attention_mixer(h, w, p, mx, eps, cache):
+def diff_attention_mixer(h, w, p, mx, eps, cache, r=exact):
     """cache: (list of keys [G, 2, dim], list of values [G, vdim]) or None; one entry a position."""
     H, G, d, dv = mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
     rot, mask = mx["rot"], mx.get("mask") or {}
     factor = (rot.get("scaling") or {}).get("factor", 1.0)
     K, V = ([], []) if cache is None else (list(cache[0]), list(cache[1]))
     T = len(h)
-    q = (h @ w[p + "q"].T).reshape(T, H, 2, d)
-    k = (h @ w[p + "k"].T).reshape(T, G, 2, d)
-    v = (h @ w[p + "v"].T).reshape(T, G, dv)
+    q = r(h @ w[p + "q"].T).reshape(T, H, 2, d)
+    k = r(h @ w[p + "k"].T).reshape(T, G, 2, d)
+    v = r(h @ w[p + "v"].T).reshape(T, G, dv)
     lam = diff_lambda(*(np.asarray(w[p + n], np.float64) for n in ("lq1", "lk1", "lq2", "lk2")), mx["diff"])
     gate = sigmoid(h @ w[p + "g"].T)
     out = np.empty((T, H, dv))
     for t in range(T):
         i = len(K)
-        K.append(rope_interleaved(k[t], i, rot["dims"], rot["base"], factor))
+        K.append(r(rope_interleaved(k[t], i, rot["dims"], rot["base"], factor)))
         V.append(v[t])
-        qr = rope_interleaved(q[t], i, rot["dims"], rot["base"], factor)
+        qr = r(rope_interleaved(q[t], i, rot["dims"], rot["base"], factor))
         Ka, Va = np.array(K), np.array(V)
         for a in range(H):
             g = a // (H // G)
@@ -124,16 +128,19 @@ def diff_attention_mixer(h, w, p, mx, eps, cache):
                              mask.get("keep_first", 0)) for n in (0, 1))
             o = rms(a1 - lam * a2, eps) * (1.0 - mx["diff"])
             out[t, a] = o * gate[t, a]
-    return out.reshape(T, H * dv) @ w[p + "o"].T, (K, V)
+    return r(out.reshape(T, H * dv)) @ w[p + "o"].T, (K, V)
 
 
 MIXERS = {"mlstm": mlstm_mixer, "attention": diff_attention_mixer}
 
 
 class Run:
-    """One sequence through the model; feed() takes its next tokens and returns the logits at each."""
+    """One sequence through the model; feed() takes its next tokens and returns the logits at each.
+    r: what happens to every activation that is stored between operations (nothing; a rounding or a
+    disturbance of its size, to learn what it does to the logits)."""
 
-    def __init__(self, cfg, w):
+    def __init__(self, cfg, w, r=exact):
+        self.r = r
         self.cfg, self.w = cfg, {n: np.asarray(a, np.float64) for n, a in w.items()}
         self.state = [None] * len(cfg["layers"])
 
@@ -143,13 +150,13 @@ class Run:
         x = w["embed"][np.asarray(tokens)] * cfg["embedding"]["scale"]
         for i, layer in enumerate(cfg["layers"]):
             p = f"l{i}."
-            y, self.state[i] = MIXERS[layer["type"]](norm_zero_centred(x, w[p + "norm1"], eps), w, p + "mix.",
-                                                     layer["mixer"], eps, self.state[i])
+            y, self.state[i] = MIXERS[layer["type"]](self.r(norm_zero_centred(x, w[p + "norm1"], eps)), w, p + "mix.",
+                                                     layer["mixer"], eps, self.state[i], self.r)
             x = x + y
             if layer["mlp"] is not None:
-                x = x + dense_ff(norm_zero_centred(x, w[p + "norm2"], eps), w[p + "mlp.gate"], w[p + "mlp.up"],
-                                 w[p + "mlp.down"])
+                x = x + dense_ff(self.r(norm_zero_centred(x, w[p + "norm2"], eps)), w[p + "mlp.gate"], w[p + "mlp.up"],
+                                 w[p + "mlp.down"], self.r)
             if trail is not None:
                 trail.append(x)
-        self.hidden = norm_zero_centred(x, w["final.norm"], eps)
+        self.hidden = self.r(norm_zero_centred(x, w["final.norm"], eps))
         return self.hidden @ w["head"].T
