@@ -453,12 +453,22 @@ __global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* x, cons
   }
 }
 
-// x = table[id] * scale, fp32
+// x = table[id] * scale, fp32: a workgroup takes 1024 values of a row
 __global__ __launch_bounds__(NT) void embed_rows_kernel(const bf16_t* table, const uint32_t* ids, float scale, int V, int n,
                                                         float* out) {
-  const bf16_t* src = table + (size_t)min(ids[blockIdx.x], (uint32_t)(V - 1)) * n;
-  float* dst = out + (size_t)blockIdx.x * n;
-  for (int i = threadIdx.x; i < n; i += NT) dst[i] = dm_bf2f(src[i]) * scale;
+  const bf16_t* src = table + (size_t)min(ids[blockIdx.y], (uint32_t)(V - 1)) * n;
+  float* dst = out + (size_t)blockIdx.y * n;
+  const int i = 4 * (blockIdx.x * NT + threadIdx.x);
+  if (n % 4 == 0) {
+    if (i >= n) return;
+    float v[4];
+    act_load<4>(src + i, v);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] *= scale;
+    act_store4(dst + i, v);
+  } else {
+    for (int e = i; e < min(i + 4, n); ++e) dst[e] = dm_bf2f(src[e]) * scale;
+  }
 }
 
 __global__ __launch_bounds__(NT) void round_bf16_kernel(const float* x, size_t n, bf16_t* out) {
@@ -685,8 +695,8 @@ int ornith_head_norm_gate(ornith_ctx* ctx, const float* d_x, const void* d_w, co
 
 int ornith_embed_rows(ornith_ctx* ctx, const ornith_linear* table, const uint32_t* d_ids, int n, float scale, float* d_out) {
   ORN_REQUIRE(ctx && table && d_ids && d_out, "embed_rows: null argument");
-  ORN_REQUIRE(table->mode == ORNITH_LIN_DENSE && table->d_w && n >= 1, "embed_rows: table mode %d, n=%d", table->mode, n);
-  hipLaunchKernelGGL(embed_rows_kernel, dim3(n), dim3(NT), 0, ctx->stream, (const bf16_t*)table->d_w, d_ids, scale, table->O,
+  ORN_REQUIRE(table->mode == ORNITH_LIN_DENSE && table->d_w && n >= 1 && n <= 65535, "embed_rows: table mode %d, n=%d", table->mode, n);
+  hipLaunchKernelGGL(embed_rows_kernel, dim3((table->K + 4 * NT - 1) / (4 * NT), n), dim3(NT), 0, ctx->stream, (const bf16_t*)table->d_w, d_ids, scale, table->O,
                      table->K, d_out);
   ORN_LAUNCH_CHECK("embed_rows_kernel");
   return ORNITH_OK;

@@ -31,16 +31,31 @@ __device__ __forceinline__ void visible(const DaArgs& p, int pos, int& head, int
   head = min(p.keep, lo);
 }
 
-// element d of one map's row at position pos, rotated
+// element d of one map's row at position pos, rotated: what it is made of (loads only), then itself
 template <typename A>
-__device__ __forceinline__ float rotated(const A* row, int d, int pos, const DaArgs& p) {
-  const float x = act_f(row[d]);
-  if (d >= 2 * p.rope_half) return x;
-  const float y = act_f(row[d ^ 1]);
-  const size_t at = (size_t)pos * p.rope_half + (d >> 1);
-  const float c = p.cos_t[at], s = p.sin_t[at];
-  return (d & 1) ? dm_fma(y, s, x * c) : dm_fma(-y, s, x * c);
-}
+struct Turn {
+  A x, y;
+  float c, s;
+  bool on;
+  __device__ __forceinline__ void load(const A* row, int d, int pos, const DaArgs& p) {
+    on = d < 2 * p.rope_half;
+    x = row[d];
+    y = x;
+    c = 1.f;
+    s = 0.f;
+    if (on) {
+      y = row[d ^ 1];
+      const size_t at = (size_t)pos * p.rope_half + (d >> 1);
+      c = p.cos_t[at];
+      s = p.sin_t[at];
+    }
+  }
+  __device__ __forceinline__ A value(int d) const {
+    if (!on) return x;
+    const float a = act_f(x), b = act_f(y);
+    return act_of<A>((d & 1) ? dm_fma(b, s, a * c) : dm_fma(-b, s, a * c));
+  }
+};
 
 constexpr int NT = 256;
 
@@ -79,63 +94,91 @@ __global__ __launch_bounds__(NT) void diff_decode_kernel(DaArgs p, int KB, int t
   A* ks = reinterpret_cast<A*>(os + rows * ost);  // [KB][kst]
   A* vs = ks + (size_t)KB * kst;                  // [KB][vst]
 
-  // keys and values of the block: cached rows, or the call's own
+  // what is staged: the group's queries, rotated (row 2 r + map of head g R + r), the block's cached keys
+  // and values, and the call's own
   const A* kc = reinterpret_cast<const A*>(p.k_cache) + (size_t)g * p.cap * kd;
   const A* vc = reinterpret_cast<const A*>(p.v_cache) + (size_t)g * p.cap * p.vdim;
   auto key_at = [&](int i) { const int u = u0 + i; return u < head ? u : lo + (u - head); };
-  if constexpr (VEC) {
-    constexpr int E = 16 / (int)sizeof(A);
-    const int kch = kd / E, vch = p.vdim / E;
-    for (int i = tid; i < nk * kch; i += NT) {
-      const int r = i / kch, c = i % kch, j = key_at(r);
-      if (j < p.offset) *reinterpret_cast<uint4*>(&ks[r * kst + c * E]) = *reinterpret_cast<const uint4*>(kc + (size_t)j * kd + c * E);
-    }
-    for (int i = tid; i < nk * vch; i += NT) {
-      const int r = i / vch, c = i % vch, j = key_at(r);
-      const A* src = j < p.offset ? vc + (size_t)j * p.vdim : reinterpret_cast<const A*>(p.v) + ((size_t)(j - p.offset) * p.G + g) * p.vdim;
-      *reinterpret_cast<uint4*>(&vs[r * vst + c * E]) = *reinterpret_cast<const uint4*>(src + c * E);
-    }
-  } else {
-    for (int i = tid; i < nk * kd; i += NT) {
-      const int r = i / kd, c = i % kd, j = key_at(r);
-      if (j < p.offset) ks[r * kst + c] = kc[(size_t)j * kd + c];
-    }
-    for (int i = tid; i < nk * p.vdim; i += NT) {
-      const int r = i / p.vdim, c = i % p.vdim, j = key_at(r);
-      vs[r * vst + c] = j < p.offset ? vc[(size_t)j * p.vdim + c]
-                                     : reinterpret_cast<const A*>(p.v)[((size_t)(j - p.offset) * p.G + g) * p.vdim + c];
-    }
-  }
-  // the queries of the group, rotated and scaled: row 2 r + map of head g R + r
-  for (int i = tid; i < rows * qd; i += NT) {
-    const int r = i / qd, d = i % qd;
-    const A* src = reinterpret_cast<const A*>(p.q) + (((size_t)t * p.H + g * R + (r >> 1)) * 2 + (r & 1)) * p.dim;
-    // (as the prefill path keeps them: rotated, an activation again)
-    qs[i] = d < p.dim ? act_f(act_of<A>(rotated(src, d, pos, p))) : 0.f;
-  }
   // the call's own keys among the block's: always its last ones
-  {
-    const int first_new = max(0, nk - (pos - p.offset + 1));
-    int r0 = nk;
-    for (int r = first_new; r < nk; ++r)
-      if (key_at(r) >= p.offset) {
-        r0 = r;
-        break;
-      }
-    for (int i = tid; i < (nk - r0) * kd; i += NT) {
-      const int r = r0 + i / kd, c = i % kd, j = key_at(r);
-      const A* src = reinterpret_cast<const A*>(p.k) + (((size_t)(j - p.offset) * p.G + g) * 2 + (c >= p.dim ? 1 : 0)) * p.dim;
-      const int d = c >= p.dim ? c - p.dim : c;
-      const A x = act_of<A>(rotated(src, d, j, p));
-      ks[r * kst + c] = x;
-      if (j == pos) reinterpret_cast<A*>(p.k_cache)[((size_t)g * p.cap + j) * kd + c] = x;
+  int r_new = nk;
+  for (int r = max(0, nk - (pos - p.offset + 1)); r < nk; ++r)
+    if (key_at(r) >= p.offset) {
+      r_new = r;
+      break;
     }
-    // this query's own value row
-    if (r0 < nk && key_at(nk - 1) == pos)
-      for (int c = tid; c < p.vdim; c += NT)
-        reinterpret_cast<A*>(p.v_cache)[((size_t)g * p.cap + pos) * p.vdim + c] =
-            reinterpret_cast<const A*>(p.v)[((size_t)t * p.G + g) * p.vdim + c];
+  const int n_new = (nk - r_new) * kd, n_q = rows * qd;
+  auto q_row = [&](int r) { return reinterpret_cast<const A*>(p.q) + (((size_t)t * p.H + g * R + (r >> 1)) * 2 + (r & 1)) * p.dim; };
+  auto new_row = [&](int j, int m) { return reinterpret_cast<const A*>(p.k) + (((size_t)(j - p.offset) * p.G + g) * 2 + m) * p.dim; };
+  // (queries as the prefill path keeps them: rotated, an activation again)
+  auto put_q = [&](int i, const Turn<A>& u) { const int d = i % qd; qs[i] = d < p.dim ? act_f(u.value(d)) : 0.f; };
+  auto load_q = [&](int i, Turn<A>& u) { const int d = i % qd; if (d < p.dim) u.load(q_row(i / qd), d, pos, p); };
+  auto load_new = [&](int i, Turn<A>& u) {
+    const int c = i % kd, m = c >= p.dim ? 1 : 0, j = key_at(r_new + i / kd);
+    u.load(new_row(j, m), c - m * p.dim, j, p);
+  };
+  auto put_new = [&](int i, const Turn<A>& u) {
+    const int r = r_new + i / kd, c = i % kd, j = key_at(r);
+    const A x = u.value(c >= p.dim ? c - p.dim : c);
+    ks[r * kst + c] = x;
+    if (j == pos) reinterpret_cast<A*>(p.k_cache)[((size_t)g * p.cap + j) * kd + c] = x;
+  };
+  auto v_row = [&](int j) {
+    return j < p.offset ? vc + (size_t)j * p.vdim : reinterpret_cast<const A*>(p.v) + ((size_t)(j - p.offset) * p.G + g) * p.vdim;
+  };
+  // everything a thread stages first is asked for before any of it is waited for
+  constexpr int QB = 2;
+  Turn<A> qu[QB], nu;
+#pragma unroll
+  for (int b = 0; b < QB; ++b)
+    if (tid + NT * b < n_q) load_q(tid + NT * b, qu[b]);
+  if (tid < n_new) load_new(tid, nu);
+  if constexpr (VEC) {
+    constexpr int E = 16 / (int)sizeof(A), B = 4;
+    const int kch = kd / E, vch = p.vdim / E, nkc = r_new * kch, nvc = nk * vch;
+    uint4 kr[B], vr[B];
+    auto k_piece = [&](int i) { return *reinterpret_cast<const uint4*>(kc + (size_t)key_at(i / kch) * kd + (i % kch) * E); };
+    auto v_piece = [&](int i) { return *reinterpret_cast<const uint4*>(v_row(key_at(i / vch)) + (i % vch) * E); };
+#pragma unroll
+    for (int b = 0; b < B; ++b)
+      if (tid + NT * b < nkc) kr[b] = k_piece(tid + NT * b);
+#pragma unroll
+    for (int b = 0; b < B; ++b)
+      if (tid + NT * b < nvc) vr[b] = v_piece(tid + NT * b);
+#pragma unroll
+    for (int b = 0; b < B; ++b) {
+      const int i = tid + NT * b;
+      if (i < nkc) *reinterpret_cast<uint4*>(&ks[(i / kch) * kst + (i % kch) * E]) = kr[b];
+    }
+#pragma unroll
+    for (int b = 0; b < B; ++b) {
+      const int i = tid + NT * b;
+      if (i < nvc) *reinterpret_cast<uint4*>(&vs[(i / vch) * vst + (i % vch) * E]) = vr[b];
+    }
+    for (int i = tid + NT * B; i < nkc; i += NT) *reinterpret_cast<uint4*>(&ks[(i / kch) * kst + (i % kch) * E]) = k_piece(i);
+    for (int i = tid + NT * B; i < nvc; i += NT) *reinterpret_cast<uint4*>(&vs[(i / vch) * vst + (i % vch) * E]) = v_piece(i);
+  } else {
+    for (int i = tid; i < r_new * kd; i += NT) ks[(i / kd) * kst + i % kd] = kc[(size_t)key_at(i / kd) * kd + i % kd];
+    for (int i = tid; i < nk * p.vdim; i += NT) vs[(i / p.vdim) * vst + i % p.vdim] = v_row(key_at(i / p.vdim))[i % p.vdim];
   }
+#pragma unroll
+  for (int b = 0; b < QB; ++b)
+    if (tid + NT * b < n_q) put_q(tid + NT * b, qu[b]);
+  for (int i = tid + NT * QB; i < n_q; i += NT) {
+    Turn<A> u{};
+    load_q(i, u);
+    put_q(i, u);
+  }
+  if (tid < n_new) put_new(tid, nu);
+  for (int i = tid + NT; i < n_new; i += NT) {
+    Turn<A> u;
+    load_new(i, u);
+    put_new(i, u);
+  }
+  // this query's own value row
+  if (r_new < nk && key_at(nk - 1) == pos)
+    for (int c = tid; c < p.vdim; c += NT)
+      reinterpret_cast<A*>(p.v_cache)[((size_t)g * p.cap + pos) * p.vdim + c] =
+          reinterpret_cast<const A*>(p.v)[((size_t)t * p.G + g) * p.vdim + c];
   __syncthreads();
 
   // scores: a thread takes one key and every (NT / KB)-th row
@@ -148,6 +191,7 @@ __global__ __launch_bounds__(NT) void diff_decode_kernel(DaArgs p, int KB, int t
         const float* qr = qs + r * qd;
         s = 0.f;
         if constexpr (VEC) {
+#pragma unroll 8
           for (int d = 0; d < p.dim; d += 4) {
             float kv[4];
             act_load<4>(kr + d, kv);
@@ -191,7 +235,7 @@ __global__ __launch_bounds__(NT) void diff_decode_kernel(DaArgs p, int KB, int t
 #pragma unroll
       for (int e = 0; e < W; ++e) o[e] = 0.f;
       const float* pr = sc + r * KB;
-#pragma unroll 4
+#pragma unroll 16
       for (int key = 0; key < nk; ++key) {
         const float w = pr[key];
         if constexpr (VEC) {
