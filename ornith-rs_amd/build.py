@@ -84,18 +84,18 @@ def build(verbose=True, jobs=8, design=None):
 
 def ensure(design=None):
     """The path of a library that serves `design`: the whole one if it is there, else one of the
-    design's own parts, compiled if need be (one process at a time)."""
+    design's own parts, compiled if it is missing or older than its sources (one process at a time)."""
     import fcntl
     if design not in DESIGNS:
         design = None
-    for path in (LIB, library(design)):
-        if os.path.exists(path):
-            return path
+    if os.path.exists(LIB):
+        return LIB
     os.makedirs(OBJ, exist_ok=True)
     with open(os.path.join(OBJ, ".lock"), "w") as lock:
         fcntl.flock(lock, fcntl.LOCK_EX)
         path = library(design)
-        return path if os.path.exists(path) else build(verbose=False, design=design)
+        newest = max(os.path.getmtime(os.path.join(CSRC, f)) for f in os.listdir(CSRC))
+        return path if os.path.exists(path) and os.path.getmtime(path) >= newest else build(verbose=False, design=design)
 
 
 if __name__ == "__main__":
