@@ -764,7 +764,8 @@ def design_kernels(orn, ctx, np, width, only=None):
     def dense(O, K, copies):
         out = []
         for _ in range(copies):
-            w = orn.Linear(orn.LinearStruct(orn.LIN_DENSE, O, K, orn.KMatrixStruct(), dev((O, K), std=K ** -0.5).ptr, None, None), [])
+            w = orn.Linear(orn.LinearStruct(orn.LIN_DENSE, O, K, orn.KMatrixStruct(), dev((O, K), std=K ** -0.5).ptr,
+                    None, None), [])
             out.append(w)
         return out
 
@@ -779,7 +780,8 @@ def design_kernels(orn, ctx, np, width, only=None):
 
     def row(name, us, nbytes, flops=0.0, peer=False, note=""):
         t_hbm, t_mm = nbytes / (HBM_PEAK_GBS * 1e3), flops / (MFMA_PEAK_TFLOPS * 1e6)
-        r = {"kernel": name, "us": round(us, 2), "GB_s": round(nbytes / us / 1e3, 1), "roofline_frac": round(max(t_hbm, t_mm) / us, 4)}
+        r = {"kernel": name, "us": round(us, 2), "GB_s": round(nbytes / us / 1e3, 1), "roofline_frac": round(max(t_hbm,
+                t_mm) / us, 4)}
         if flops:
             r["TFLOP_s"] = round(flops / us / 1e6, 1)
             r["bound"] = "mfma" if t_mm > t_hbm else "hbm"
@@ -818,7 +820,8 @@ def design_kernels(orn, ctx, np, width, only=None):
             x, wn = dev((T, W), "f32"), dev((W,), std=0.1)
             ys = [ctx.alloc(T * o * 4) for o in shapes]
             outs = [orn.OUT_ACT] * 4 + [orn.OUT_F32] * 2
-            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [w[i % n] for w in ws], ys, outs, pre=orn.PRE_NORM, norm_w=wn, w_offset=1.0) for i in range(n)]))
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [w[i % n] for w in ws], ys, outs,
+                    pre=orn.PRE_NORM, norm_w=wn, w_offset=1.0) for i in range(n)]))
             mine = row(f"norm + q, k, v, gates (T = {T})", us, nb + T * W * 4 + T * sum(shapes) * 2)
             nb2 = int((D + vd) * W * 0.5625)
             n2 = copies_for(nb2)
@@ -826,12 +829,15 @@ def design_kernels(orn, ctx, np, width, only=None):
             xb, yb, hb, nn = dev((T, W)), dev((T, W)), ctx.alloc(T * W * 2), ctx.alloc(T * W * 2)
             w1 = dev((W,))
             o1, o2 = ctx.alloc(T * D * 2), ctx.alloc(T * vd * 2)
-            us = t_of(lambda i: orn.add_rms_linear_multi(ctx, [a[i % n2], b[i % n2]], xb, yb, w1, 1e-6, T, hb, nn, [o1, o2]))
-            pair(f"decode projections in, T = {T}", mine, row("x", us, nb2 + T * (D + vd) * 2, peer=True), "add + norm + in_proj qkv, z (Q4_K)")
+            us = t_of(lambda i: orn.add_rms_linear_multi(ctx, [a[i % n2], b[i % n2]], xb, yb, w1, 1e-6, T, hb, nn, [o1,
+                    o2]))
+            pair(f"decode projections in, T = {T}", mine, row("x", us, nb2 + T * (D + vd) * 2, peer=True),
+                    "add + norm + in_proj qkv, z (Q4_K)")
             n = copies_for(W * nv * 2)
             wo = dense(W, nv, n)
             o, gate, wn2, xs = dev((T, nv), "f32"), dev((T, nv)), dev((nv,)), dev((T, W), "f32")
-            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, o, T, nv, [wo[i % n]], [xs], [orn.OUT_ADD], pre=orn.PRE_HEADS, norm_w=wn2, gate=gate, head_dim=dv) for i in range(n)]))
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, o, T, nv, [wo[i % n]], [xs], [orn.OUT_ADD],
+                    pre=orn.PRE_HEADS, norm_w=wn2, gate=gate, head_dim=dv) for i in range(n)]))
             mine = row(f"head norm, gate + output projection + sum (T = {T})", us, W * nv * 2 + T * nv * 6)
             n2 = copies_for(int(W * vd * 0.5625))
             a = kq(util.Q4K, W, vd, n2)
@@ -841,9 +847,11 @@ def design_kernels(orn, ctx, np, width, only=None):
             n = copies_for(2 * ff * W * 2)
             wg, wu, wd = dense(ff, W, n), dense(ff, W, n), dense(W, ff, n)
             act = ctx.alloc(T * ff * 2)
-            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [wg[i % n], wu[i % n]], [act, None], [0, 0], pre=orn.PRE_NORM, norm_w=wn, w_offset=1.0, gelu_pair=True) for i in range(n)]))
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [wg[i % n], wu[i % n]], [act, None], [0,
+                    0], pre=orn.PRE_NORM, norm_w=wn, w_offset=1.0, gelu_pair=True) for i in range(n)]))
             mine = row(f"norm + gate, up + gelu (T = {T})", us, 2 * ff * W * 2)
-            us2 = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, act, T, ff, [wd[i % n]], [xs], [orn.OUT_ADD]) for i in range(n)]))
+            us2 = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, act, T, ff, [wd[i % n]], [xs],
+                    [orn.OUT_ADD]) for i in range(n)]))
             mine2 = row(f"down + sum (T = {T})", us2, ff * W * 2)
             if W == 2048:
                 moes = [util.HostMoe(rng, E=64).dev(orn, ctx) for _ in range(4)]
@@ -862,19 +870,24 @@ def design_kernels(orn, ctx, np, width, only=None):
             sf = orn.mlstm_state_floats(H, d, dv)
             layers = 24
             slots = [dev((T + 2, sf), "f32", 0.01) for _ in range(layers)]
-            q, k, v, gi, gf, b1 = dev((T, nk)), dev((T, nk)), dev((T, nv)), dev((T, H), "f32"), dev((T, H), "f32"), dev((H,))
+            q, k, v, gi, gf, b1 = dev((T, nk)), dev((T, nk)), dev((T, nv)), dev((T, H), "f32"), dev((T, H),
+                    "f32"), dev((H,))
             o = ctx.alloc(T * nv * 4)
-            us = t_of(calls(orn.mlstm, [orn.mlstm_call(act=orn.BF16, q=q, k=k, v=v, gi=gi, gf=gf, bi=b1, bf=b1, gate_cap=15.0, T=T, H=H, dim=d, vdim=dv,
+            us = t_of(calls(orn.mlstm, [orn.mlstm_call(act=orn.BF16, q=q, k=k, v=v, gi=gi, gf=gf, bi=b1, bf=b1,
+                    gate_cap=15.0, T=T, H=H, dim=d, vdim=dv,
                                           state_in=slots[i % layers].ptr.value + ((i // layers) % 2) * sf * 4, slots=slots[i % layers], n_slots=T + 2,
                                           first_slot=1 - (i // layers) % 2, snapshots=0, o=o) for i in range(2 * layers)]))
             mine = row(f"mLSTM step (T = {T})", us, 2 * sf * 4 + T * (2 * nk + nv) * 2 + T * nv * 4)
             sd = Hv * 128 * 128
             st = [dev((2, sd), "f32", 0.01) for _ in range(layers)]
-            conv, qkv, cw, wa, wb, xn = dev((3, D)), dev((T, D)), dev((D, 4)), dev((Hv, W), std=0.02), dev((Hv, W), std=0.02), dev((T, W))
+            conv, qkv, cw, wa, wb, xn = dev((3, D)), dev((T, D)), dev((D, 4)), dev((Hv, W), std=0.02), dev((Hv, W),
+                    std=0.02), dev((T, W))
             al, dt, nw, zz = dev((Hv,)), dev((Hv,)), dev((128,)), dev((T, vd))
             ci, gated = ctx.alloc((3 + T) * D * 2), ctx.alloc(T * vd * 2)
-            us = t_of(lambda i: orn.gdn_step(ctx, conv, qkv, cw, wa, wb, xn, W, al, dt, T, 4, Hk, 128, Hv, 128, st[i % layers], st[i % layers], False, nw, zz, ci, gated))
-            pair(f"decode recurrence, T = {T}", mine, row("x", us, 2 * sd * 4 + 2 * Hv * W * 2 + T * (D + 2 * vd) * 2 + 7 * D * 2, peer=True), "gdn_step")
+            us = t_of(lambda i: orn.gdn_step(ctx, conv, qkv, cw, wa, wb, xn, W, al, dt, T, 4, Hk, 128, Hv, 128,
+                    st[i % layers], st[i % layers], False, nw, zz, ci, gated))
+            pair(f"decode recurrence, T = {T}", mine, row("x", us,
+                    2 * sd * 4 + 2 * Hv * W * 2 + T * (D + 2 * vd) * 2 + 7 * D * 2, peer=True), "gdn_step")
         if want("decode attention"):
             for ctx_len in (256, win + keep):
                 caps = 24
@@ -883,7 +896,8 @@ def design_kernels(orn, ctx, np, width, only=None):
                 q, k, v, gt = dev((T, h * 2 * ad)), dev((T, g * 2 * ad)), dev((T, g * av)), dev((T, h), "f32")
                 co, si = ctx.rope_table(ctx_len, ad // 2, 250000.0)
                 out, qr = ctx.alloc(T * h * av * 2), ctx.alloc(T * h * 2 * ad * 2)
-                us = t_of(calls(orn.diff_attn, [orn.diff_attn_call(act=orn.BF16, q=q, k=k, v=v, gate=gt, cos=co, sin=si, rope_dims=ad // 2, table_npos=ctx_len, T=T, H=h, G=g,
+                us = t_of(calls(orn.diff_attn, [orn.diff_attn_call(act=orn.BF16, q=q, k=k, v=v, gate=gt, cos=co, sin=si,
+                        rope_dims=ad // 2, table_npos=ctx_len, T=T, H=h, G=g,
                                                   dim=ad, vdim=av, offset=off, cap=ctx_len, window=win, keep_first=keep, scale=ad ** -0.5, lam=0.5, diff=0.55,
                                                   eps=1e-6, k_cache=kc[i % caps], v_cache=vc[i % caps], q_rot=qr, out=out) for i in range(caps)]))
                 mine = row(f"attention, {ctx_len} keys (T = {T})", us, g * ctx_len * (2 * ad + av) * 2)
@@ -892,9 +906,11 @@ def design_kernels(orn, ctx, np, width, only=None):
                 qg, kx, vx, qw = dev((T, Hq * 512)), dev((T, Hkv * 256)), dev((T, Hkv * 256)), dev((256,))
                 co2, si2 = ctx.rope_table(ctx_len, 64, 1e7)
                 qr2, out2 = ctx.alloc(T * Hq * 512), ctx.alloc(T * Hq * 512)
-                us = t_of(lambda i: ctx.attn_decode(qg, kx, vx, qw, qw, T, Hq, Hkv, 256, 64, 1e-6, co2, si2, ctx_len, off, ctx_len, 1 / 16.0, qr2,
+                us = t_of(lambda i: ctx.attn_decode(qg, kx, vx, qw, qw, T, Hq, Hkv, 256, 64, 1e-6, co2, si2, ctx_len, off,
+                        ctx_len, 1 / 16.0, qr2,
                                                     kc2[i % caps], vc2[i % caps], out2))
-                pair(f"decode attention, {ctx_len} keys, T = {T}", mine, row("x", us, Hkv * ctx_len * 1024, peer=True), "attn_decode")
+                pair(f"decode attention, {ctx_len} keys, T = {T}", mine, row("x", us, Hkv * ctx_len * 1024, peer=True),
+                        "attn_decode")
     # ---- prefill
     for T in (512, 4096):
         reps = dict(n=20, warm=3)
@@ -905,7 +921,8 @@ def design_kernels(orn, ctx, np, width, only=None):
             ys = [ctx.alloc(T * o * 4) for o in shapes]
             outs = [orn.OUT_ACT] * 4 + [orn.OUT_F32] * 2
             us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, ws, ys, outs) for i in range(1)]), **reps)
-            mine = row(f"q, k, v, gates (T = {T})", us, sum(shapes) * W * 2 + T * W * 2 + T * sum(shapes) * 2, 2.0 * T * W * sum(shapes))
+            mine = row(f"q, k, v, gates (T = {T})", us, sum(shapes) * W * 2 + T * W * 2 + T * sum(shapes) * 2,
+                    2.0 * T * W * sum(shapes))
             a, b = kq(util.Q4K, D, W, 1), kq(util.Q4K, vd, W, 1)
             o1, o2 = ctx.alloc(T * D * 2), ctx.alloc(T * vd * 2)
             us = t_of(lambda i: ctx.linear_matmul_multi([a[0], b[0]], x, T, [o1, o2]), **reps)
@@ -913,14 +930,18 @@ def design_kernels(orn, ctx, np, width, only=None):
             pair(f"prefill GEMM in, T = {T}", mine, peer, "in_proj qkv, z (Q4_K)")
             wg, wu, wd = dense(ff, W, 1)[0], dense(ff, W, 1)[0], dense(W, ff, 1)[0]
             act, xs = ctx.alloc(T * ff * 2), dev((T, W), "f32")
-            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [wg, wu], [act, None], [0, 0], gelu_pair=True) for i in range(1)]), **reps)
-            pair(f"prefill GEMM gate, up + gelu, T = {T}", row(f"gate, up + gelu (T = {T})", us, 2 * ff * W * 2 + T * (W + ff) * 2, 4.0 * T * W * ff), peer, "in_proj qkv, z (Q4_K)")
-            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, act, T, ff, [wd], [xs], [orn.OUT_ADD]) for i in range(1)]), **reps)
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [wg, wu], [act, None], [0, 0],
+                    gelu_pair=True) for i in range(1)]), **reps)
+            pair(f"prefill GEMM gate, up + gelu, T = {T}", row(f"gate, up + gelu (T = {T})", us,
+                    2 * ff * W * 2 + T * (W + ff) * 2, 4.0 * T * W * ff), peer, "in_proj qkv, z (Q4_K)")
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, act, T, ff, [wd], [xs],
+                    [orn.OUT_ADD]) for i in range(1)]), **reps)
             mine = row(f"down + sum (T = {T})", us, ff * W * 2 + T * (ff * 2 + W * 8), 2.0 * T * W * ff)
             a = kq(util.Q4K, W, vd, 1)
             xo, yo = dev((T, vd)), ctx.alloc(T * W * 2)
             us = t_of(lambda i: ctx.linear_matmul(a[0], xo, T, yo), **reps)
-            pair(f"prefill GEMM down + sum, T = {T}", mine, row("x", us, int(W * vd * 0.5625) + T * (W + vd) * 2, 2.0 * T * W * vd, peer=True), "out_proj (Q4_K)")
+            pair(f"prefill GEMM down + sum, T = {T}", mine, row("x", us, int(W * vd * 0.5625) + T * (W + vd) * 2,
+                    2.0 * T * W * vd, peer=True), "out_proj (Q4_K)")
         if want("prefill rows"):
             xs, wn, out = dev((T, W), "f32"), dev((W,), std=0.1), ctx.alloc(T * max(W, nv) * 2)
             us = t_of(lambda i: orn.norm_rows(ctx, xs, wn, 1.0, T, W, 1e-6, orn.BF16, out), **reps)
@@ -937,16 +958,21 @@ def design_kernels(orn, ctx, np, width, only=None):
         if want("prefill recurrence"):
             sf = orn.mlstm_state_floats(H, d, dv)
             slots = dev((2, sf), "f32", 0.01)
-            q, k, v, gi, gf, b1 = dev((T, nk)), dev((T, nk)), dev((T, nv)), dev((T, H), "f32"), dev((T, H), "f32"), dev((H,))
+            q, k, v, gi, gf, b1 = dev((T, nk)), dev((T, nk)), dev((T, nv)), dev((T, H), "f32"), dev((T, H),
+                    "f32"), dev((H,))
             o = ctx.alloc(T * nv * 4)
-            us = t_of(calls(orn.mlstm, [orn.mlstm_call(act=orn.BF16, q=q, k=k, v=v, gi=gi, gf=gf, bi=b1, bf=b1, gate_cap=15.0, T=T, H=H, dim=d, vdim=dv,
+            us = t_of(calls(orn.mlstm, [orn.mlstm_call(act=orn.BF16, q=q, k=k, v=v, gi=gi, gf=gf, bi=b1, bf=b1,
+                    gate_cap=15.0, T=T, H=H, dim=d, vdim=dv,
                                           state_in=slots.ptr.value + (i % 2) * sf * 4, slots=slots, n_slots=2, first_slot=1 - i % 2, snapshots=0, o=o) for i in range(2)]), **reps)
-            mine = row(f"mLSTM in chunks (T = {T})", us, T * (2 * nk + nv) * 2 + T * nv * 4 + 2 * sf * 4, 2.0 * T * H * (2 * d * dv + 32 * (d + dv)))
+            mine = row(f"mLSTM in chunks (T = {T})", us, T * (2 * nk + nv) * 2 + T * nv * 4 + 2 * sf * 4,
+                    2.0 * T * H * (2 * d * dv + 32 * (d + dv)))
             qd, kdd, vdd = dev((T, Hk * 128), std=0.09), dev((T, Hk * 128), std=0.09), dev((T, vd))
-            gd = ctx.to_device(np.resize(np.abs(block) * np.float32(0.1) + np.float32(0.85), T * Hv).clip(0.5, 0.999).astype(np.float32))
+            gd = ctx.to_device(np.resize(np.abs(block) * np.float32(0.1) + np.float32(0.85), T * Hv).clip(0.5,
+                    0.999).astype(np.float32))
             bd, yd, sd = dev((T, Hv), std=0.3), ctx.alloc(T * vd * 2), dev((1, Hv * 128 * 128), "f32", 0.01)
             us = t_of(lambda i: ctx.gdn_recurrence(qd, kdd, vdd, gd, bd, sd, T, Hk, Hv, 128, 128, yd, sd, False), **reps)
-            pair(f"prefill recurrence, T = {T}", mine, row("x", us, T * (2 * Hk * 128 + 2 * vd) * 2 + 2 * Hv * 128 * 128 * 4,
+            pair(f"prefill recurrence, T = {T}", mine, row("x", us,
+                    T * (2 * Hk * 128 + 2 * vd) * 2 + 2 * Hv * 128 * 128 * 4,
                                                            2.0 * T * Hv * (2 * 128 * 128 + 32 * 256), peer=True), "gdn_recurrence (chunked)")
         if want("prefill attention"):
             q, k, v, gt = dev((T, h * 2 * ad)), dev((T, g * 2 * ad)), dev((T, g * av)), dev((T, h), "f32")
@@ -955,18 +981,22 @@ def design_kernels(orn, ctx, np, width, only=None):
             out, qr = ctx.alloc(T * h * av * 2), ctx.alloc(T * h * 2 * ad * 2)
             i_ = np.arange(T)
             seen = float(np.sum(np.minimum(i_ + 1, win) + np.minimum(np.maximum(i_ - win + 1, 0), keep)))
-            us = t_of(calls(orn.diff_attn, [orn.diff_attn_call(act=orn.BF16, q=q, k=k, v=v, gate=gt, cos=co, sin=si, rope_dims=ad // 2, table_npos=T, T=T, H=h, G=g, dim=ad,
+            us = t_of(calls(orn.diff_attn, [orn.diff_attn_call(act=orn.BF16, q=q, k=k, v=v, gate=gt, cos=co, sin=si,
+                    rope_dims=ad // 2, table_npos=T, T=T, H=h, G=g, dim=ad,
                                               vdim=av, offset=0, cap=T, window=win, keep_first=keep, scale=ad ** -0.5, lam=0.5, diff=0.55, eps=1e-6,
                                               k_cache=kc, v_cache=vc, q_rot=qr, out=out) for i in range(1)]), **reps)
-            mine = row(f"attention (T = {T}, rotation and append included)", us, T * (h * 2 * ad + g * (2 * ad + av) + h * av) * 2, 2.0 * seen * h * 2 * (ad + av))
+            mine = row(f"attention (T = {T}, rotation and append included)", us,
+                    T * (h * 2 * ad + g * (2 * ad + av) + h * av) * 2, 2.0 * seen * h * 2 * (ad + av))
             Hq, Hkv = W // 128, max(2, W // 1024)
             qg, kx, vx, qw = dev((T, Hq * 512)), dev((T, Hkv * 256)), dev((T, Hkv * 256)), dev((256,))
             co2, si2 = ctx.rope_table(T, 64, 1e7)
             kc2, vc2 = dev((Hkv, T, 256)), dev((Hkv, T, 256))
             qr2, out2 = ctx.alloc(T * Hq * 512), ctx.alloc(T * Hq * 512)
-            us = t_of(lambda i: ctx.attn_decode(qg, kx, vx, qw, qw, T, Hq, Hkv, 256, 64, 1e-6, co2, si2, T, 0, T, 1 / 16.0, qr2, kc2, vc2, out2), **reps)
+            us = t_of(lambda i: ctx.attn_decode(qg, kx, vx, qw, qw, T, Hq, Hkv, 256, 64, 1e-6, co2, si2, T, 0, T,
+                    1 / 16.0, qr2, kc2, vc2, out2), **reps)
             full = T * (T + 1) / 2
-            pair(f"prefill attention, T = {T}", mine, row("x", us, T * (Hq * 512 + 2 * Hkv * 256 + Hq * 256) * 2, 2.0 * full * Hq * 512, peer=True),
+            pair(f"prefill attention, T = {T}", mine, row("x", us, T * (Hq * 512 + 2 * Hkv * 256 + Hq * 256) * 2,
+                    2.0 * full * Hq * 512, peer=True),
                  "attn_decode at prefill width (prep + attention)")
     for b in garbage:
         b.free()

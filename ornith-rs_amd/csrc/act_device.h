@@ -55,7 +55,7 @@ __device__ __forceinline__ float dm_tanh(float x) {
   return a < 0.25f ? s : (x < 0.0f ? -t : t);
 }
 
-// the tanh form of gelu
+// gelu by its tanh approximation
 __device__ __forceinline__ float dm_gelu_tanh(float z) {
   const float u = 0.7978845608028654f * dm_fma(0.044715f * z * z, z, z);
   return 0.5f * z * (1.0f + dm_tanh(u));

@@ -75,7 +75,7 @@ struct Call : ornith_dense_call {
     d_x = x;
     eps = m->cfg.rms_norm_eps;
   }
-  Call& norm(const void* w, void* rows) {  // weights stored around zero
+  Call& norm(const void* w, void* rows) {  // weights as their distance from one
     pre = ORNITH_PRE_NORM;
     d_norm_w = w;
     w_offset = 1.f;

@@ -3,13 +3,13 @@
     bin/trace_run --model DIR --dtype bfloat16|float32 --out DIR --max-tokens N
 
 DIR holds config.json and model.safetensors (or shards and their index); config.json picks the design.
-Steps come on standard input, one JSON object a line:
+Standard input holds a step a line, as JSON:
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+    {"step": 3, "entries": [{"id": "x", "tokens": [11, 4], "want": [1]}], "end": ["x"]}
 
-An entry brings a request's next tokens; "want" lists the places among them whose logits are written to
-<out>/<step>.f32 (float32, [wanted, vocab], in the order of the entries); "end" lists the requests whose
-caches are given back after the step. `done <step>` on standard output ends a step. Nothing is sampled.
+"tokens" continue request "x"; "want" are indexes into them, and the float32 logits at those go to
+<out>/<step>.f32, row after row; "end" names requests that need their caches no more. A finished step is
+reported as `done <step>` on standard output. Nothing is sampled.
 
 It drives the library's own step function and caches, one request after the other: a request's caches are
 taken from a pool at its first tokens, reset, and returned to the pool at its end."""
@@ -105,7 +105,7 @@ def main(argv=None):
     ap.add_argument("--model", required=True, help="folder with config.json and the weights")
     ap.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16")
     ap.add_argument("--out", required=True, help="folder for the logits")
-    ap.add_argument("--max-tokens", type=int, default=4096, help="the most tokens live requests hold at any time")
+    ap.add_argument("--max-tokens", type=int, default=4096, help="tokens the caches are laid out for")
     a = ap.parse_args(argv)
     orn = _library(a.model)
     try:

@@ -87,12 +87,12 @@ def rope_interleaved(x, pos, dims, base, factor):
 
 
 def visible(i, j, size, keep_first):
-    """Sliding window with kept first tokens; size 0: no window."""
+    """What position i may look at: its window (size 0: everything before it) and the sequence's start."""
     return j <= i and (not size or i - j < size or j < keep_first)
 
 
 def attend(q, keys, values, i, scale, size, keep_first):
-    """Ordinary softmax attention of the query at position i over what it sees."""
+    """Softmax average of the values that position i sees."""
     js = [j for j in range(len(keys)) if visible(i, j, size, keep_first)]
     s = np.array([float(q @ keys[j]) * scale for j in js])
     e = np.exp(s - s.max())

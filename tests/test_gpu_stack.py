@@ -31,11 +31,13 @@ def _close(got, want, act, what, slack=1.0):
     rms = np.sqrt(np.mean(want ** 2)) + 1e-30
     bound = slack * (3e-6 * (np.abs(want) + 3 * rms) if act == 0 else 2.0 ** -8 * np.abs(want) + 1e-2 * rms)
     err = np.abs(got - want)
-    assert np.all(np.isfinite(got)) and np.all(err <= bound), (what, float(err.max()), float((err / bound).max()), float(rms))
+    assert np.all(np.isfinite(got)) and np.all(err <= bound), (what, float(err.max()), float((err / bound).max()),
+            float(rms))
 
 
 @pytest.mark.parametrize("act", [0, 1])
-@pytest.mark.parametrize("M,K", [(1, 96), (2, 200), (3, 90), (5, 1032), (33, 200), (130, 96), (200, 264), (37, 91), (1, 9000), (2, 4104)])
+@pytest.mark.parametrize("M,K", [(1, 96), (2, 200), (3, 90), (5, 1032), (33, 200), (130, 96), (200, 264), (37, 91), (1,
+        9000), (2, 4104)])
 def test_dense_rows(orn, ctx, act, M, K):
     """All prologues and tails at decode and GEMM widths; widths that are no multiple of 8, ragged
     tiles, more than one matrix, rows longer than a thread's registers hold."""
@@ -50,7 +52,8 @@ def test_dense_rows(orn, ctx, act, M, K):
     gate = _bf(gate) if act else gate
     wn = _bf(0.3 * rng.standard_normal(K))
     rows = {orn.PRE_NONE: xa.astype(np.float64), orn.PRE_NORM: R.norm_zero_centred(x32.astype(np.float64), wn, 1e-5),
-            orn.PRE_HEADS: (R.rms(x32.astype(np.float64).reshape(M, -1, head), 1e-5).reshape(M, K) * wn) * R.sigmoid(gate.astype(np.float64))}
+            orn.PRE_HEADS: (R.rms(x32.astype(np.float64).reshape(M, -1, head), 1e-5).reshape(M,
+                    K) * wn) * R.sigmoid(gate.astype(np.float64))}
     d_x, d_g, d_wn = ctx.to_device(x32), _dev(ctx, gate, act), ctx.to_device(util.f32_to_bf16(wn))
     d_xa, d_rows = _dev(ctx, xa, act), ctx.alloc(M * K * 4)
     adt, es = (orn.F32, 4) if act == 0 else (orn.BF16, 2)
@@ -70,12 +73,15 @@ def test_dense_rows(orn, ctx, act, M, K):
         for y in ys:
             y.free()
         if pre != orn.PRE_HEADS:
-            g, u = (orn.Linear.dense(ctx, util.f32_to_bf16(_bf(rng.standard_normal((70, K)) * K ** -0.5))) for _ in range(2))
+            g, u = (orn.Linear.dense(ctx, util.f32_to_bf16(_bf(rng.standard_normal((70,
+                    K)) * K ** -0.5))) for _ in range(2))
             gw, uw = (util.bf16_to_f32(l.keep[0].download(np.uint16, (70, K))).astype(np.float64) for l in (g, u))
             y = ctx.alloc(M * 70 * 4)
-            orn.dense_rows(ctx, adt, d_xa if pre == orn.PRE_NONE else d_x, M, K, [g, u], [y, None], [0, 0], pre=pre, norm_w=d_wn,
+            orn.dense_rows(ctx, adt, d_xa if pre == orn.PRE_NONE else d_x, M, K, [g, u], [y, None], [0, 0], pre=pre,
+                    norm_w=d_wn,
                            w_offset=1.0, eps=1e-5, gelu_pair=True, rows=d_rows)
-            _close(_get(y, (M, 70), act), R.gelu_tanh(h @ gw.T) * (h @ uw.T), act, ("gelu pair", pre), slack=6.0 if act == 0 else 1.5)
+            _close(_get(y, (M, 70), act), R.gelu_tanh(h @ gw.T) * (h @ uw.T), act, ("gelu pair", pre),
+                    slack=6.0 if act == 0 else 1.5)
             for b in (y, g, u):
                 b.free()
     for b in [d_x, d_g, d_wn, d_xa, d_rows] + lins:
@@ -109,13 +115,15 @@ def test_dense_rows_of_a_call_are_those_of_single_rows(orn, ctx):
 def test_rows_of_the_prologues_alone(orn, ctx, act, heads, head):
     rng = np.random.default_rng(heads * 1000 + head)
     T, n = 9, heads * head
-    x, gate, w = rng.standard_normal((T, n)).astype(np.float32), _bf(rng.standard_normal((T, n))), _bf(rng.standard_normal(n))
+    x, gate, w = rng.standard_normal((T, n)).astype(np.float32), _bf(rng.standard_normal((T,
+            n))), _bf(rng.standard_normal(n))
     d, g, dw, out = ctx.to_device(x), _dev(ctx, gate, act), ctx.to_device(util.f32_to_bf16(w)), ctx.alloc(T * n * 4)
     adt = orn.F32 if act == 0 else orn.BF16
     orn.norm_rows(ctx, d, dw, 1.0, T, n, 1e-4, adt, out)
     _close(_get(out, (T, n), act), R.norm_zero_centred(x.astype(np.float64), w, 1e-4), act, "norm")
     orn.head_norm_gate(ctx, d, dw, g, T, heads, head, 1e-4, adt, out)
-    _close(_get(out, (T, n), act), R.rms(x.astype(np.float64).reshape(T, heads, head), 1e-4).reshape(T, n) * w * R.sigmoid(gate.astype(np.float64)),
+    _close(_get(out, (T, n), act), R.rms(x.astype(np.float64).reshape(T, heads, head), 1e-4).reshape(T,
+            n) * w * R.sigmoid(gate.astype(np.float64)),
            act, "head norm")
     for b in (d, g, dw, out):
         b.free()
@@ -137,15 +145,18 @@ class Memory:
     def inputs(self, rng, T):
         f = (lambda a: _bf(a)) if self.act else (lambda a: a.astype(np.float32))
         return dict(q=f(rng.standard_normal((T, self.H, self.dim))), k=f(rng.standard_normal((T, self.H, self.dim))),
-                    v=f(rng.standard_normal((T, self.H, self.vdim))), gi=(2 * rng.standard_normal((T, self.H))).astype(np.float32),
+                    v=f(rng.standard_normal((T, self.H, self.vdim))), gi=(2 * rng.standard_normal((T,
+                            self.H))).astype(np.float32),
                     gf=(2 * rng.standard_normal((T, self.H)) + 2).astype(np.float32))
 
     def step(self, x, snapshots=False):
         """The call's outputs [T, H, vdim]; the state moves to the next slot (or the last snapshot's)."""
         T = len(x["q"])
-        d = {n: (_dev(self.ctx, x[n], self.act) if n in "qkv" else self.ctx.to_device(x[n])) for n in ("q", "k", "v", "gi", "gf")}
+        d = {n: (_dev(self.ctx, x[n], self.act) if n in "qkv" else self.ctx.to_device(x[n])) for n in ("q", "k", "v",
+                "gi", "gf")}
         o, first = self.ctx.alloc(T * self.H * self.vdim * 4), (self.cur + 1) % self.n
-        self.orn.mlstm(self.ctx, act=self.act, bi=self.d_b[0], bf=self.d_b[1], gate_cap=self.cap, T=T, H=self.H, dim=self.dim,
+        self.orn.mlstm(self.ctx, act=self.act, bi=self.d_b[0], bf=self.d_b[1], gate_cap=self.cap, T=T, H=self.H,
+                dim=self.dim,
                        vdim=self.vdim, state_in=self.slots.ptr.value + self.cur * self.floats * 4, slots=self.slots, n_slots=self.n,
                        first_slot=first, snapshots=int(snapshots), o=o, **d)
         self.cur = (first + T - 1) % self.n if snapshots else first
@@ -159,7 +170,8 @@ class Memory:
         for h in range(self.H):
             li = R.soft_cap(x["gi"][:, h].astype(np.float64) + self.bi[h], self.cap)
             lf = R.log_sigmoid(R.soft_cap(x["gf"][:, h].astype(np.float64) + self.bf[h], self.cap))
-            out[:, h], self.ref[h] = R.mlstm_cell(x["q"][:, h].astype(np.float64) * self.dim ** -0.5, x["k"][:, h].astype(np.float64),
+            out[:, h], self.ref[h] = R.mlstm_cell(x["q"][:, h].astype(np.float64) * self.dim ** -0.5, x["k"][:,
+                    h].astype(np.float64),
                                                   x["v"][:, h].astype(np.float64), li, lf, self.ref[h])
         return out
 
@@ -169,7 +181,8 @@ class Memory:
         a = self.slots.download(np.float32, (self.n, self.H, self.floats // self.H))[self.cur if slot is None else slot]
         rows = a[:, :(self.vdim + 1) * ds].reshape(self.H, self.vdim + 1, ds)
         assert np.all(rows[:, :, self.dim:] == 0)
-        return [(rows[h, :self.vdim, :self.dim].T, rows[h, self.vdim, :self.dim], a[h, (self.vdim + 1) * ds]) for h in range(self.H)]
+        return [(rows[h, :self.vdim, :self.dim].T, rows[h, self.vdim, :self.dim], a[h,
+                (self.vdim + 1) * ds]) for h in range(self.H)]
 
     def check_state(self, what, tol):
         for h, (S, n, m) in enumerate(self.state()):
@@ -187,11 +200,13 @@ def _near(got, want, tol, what):
     """Relative to the size of the head's row (outputs of one head share their denominator)."""
     scale = np.sqrt(np.mean(want ** 2, axis=-1, keepdims=True)) + 1e-3 * np.sqrt(np.mean(want ** 2)) + 1e-12
     err = np.abs(got - want) / scale
-    assert np.all(np.isfinite(got)) and err.max() <= tol, (what, float(err.max()), np.unravel_index(err.argmax(), err.shape))
+    assert np.all(np.isfinite(got)) and err.max() <= tol, (what, float(err.max()), np.unravel_index(err.argmax(),
+            err.shape))
 
 
 @pytest.mark.parametrize("act", [0, 1])
-@pytest.mark.parametrize("H,dim,vdim,cap", [(1, 16, 16, 5.0), (3, 10, 14, 4.0), (2, 72, 136, 9.0), (2, 136, 40, 15.0), (1, 256, 192, 8.0),
+@pytest.mark.parametrize("H,dim,vdim,cap", [(1, 16, 16, 5.0), (3, 10, 14, 4.0), (2, 72, 136, 9.0), (2, 136, 40, 15.0), (1,
+        256, 192, 8.0),
                                             (2, 24, 300, 6.0), (1, 300, 20, 6.0)])
 def test_mlstm_portions(orn, ctx, act, H, dim, vdim, cap):
     """Calls of many lengths one after the other, around the chunk's edges and the sixteen-column
@@ -221,7 +236,8 @@ def test_mlstm_finds_a_far_key(orn, ctx, act, far):
     x["q"][-1] = x["k"][at]
     for cut in (T, T - 1):
         m2 = Memory(orn, ctx, H, dim, vdim, 12.0, act, seed=9, f_bias=9.0)
-        got = np.concatenate([m2.step({n: a[:cut] for n, a in x.items()})] + ([m2.step({n: a[cut:] for n, a in x.items()})] if cut < T else []))
+        got = np.concatenate([m2.step({n: a[:cut] for n, a in x.items()})] + ([m2.step({n: a[cut:] for n,
+                a in x.items()})] if cut < T else []))
         want = m2.want(x)
         _near(got[-1:], want[-1:], 2e-3, (far, cut))
         lost = {n: a.copy() for n, a in x.items()}
@@ -271,7 +287,8 @@ def test_mlstm_snapshots(orn, ctx, act):
 class Attention:
     """One attention layer's cache on the device and in the reference (ref: a diff_attention over raw rows)."""
 
-    def __init__(self, orn, ctx, act, H, G, dim, vdim, size, keep, rot, base=1000.0, factor=1.0, scale=None, diff=0.45, lam=0.6, cap=700):
+    def __init__(self, orn, ctx, act, H, G, dim, vdim, size, keep, rot, base=1000.0, factor=1.0, scale=None, diff=0.45,
+            lam=0.6, cap=700):
         self.orn, self.ctx, self.act = orn, ctx, act
         self.p = dict(H=H, G=G, dim=dim, vdim=vdim)
         self.size, self.keep, self.rot, self.base, self.factor = size, keep, rot, base, factor
@@ -289,14 +306,17 @@ class Attention:
     def inputs(self, rng, T, std=1.0):
         f = (lambda a: _bf(a)) if self.act else (lambda a: a.astype(np.float32))
         p = self.p
-        return dict(q=f(std * rng.standard_normal((T, p["H"], 2, p["dim"]))), k=f(std * rng.standard_normal((T, p["G"], 2, p["dim"]))),
-                    v=f(rng.standard_normal((T, p["G"], p["vdim"]))), gate=rng.standard_normal((T, p["H"])).astype(np.float32))
+        return dict(q=f(std * rng.standard_normal((T, p["H"], 2, p["dim"]))), k=f(std * rng.standard_normal((T, p["G"], 2,
+                p["dim"]))),
+                    v=f(rng.standard_normal((T, p["G"], p["vdim"]))), gate=rng.standard_normal((T,
+                            p["H"])).astype(np.float32))
 
     def step(self, x):
         T, p = len(x["q"]), self.p
         d = {n: (_dev(self.ctx, x[n], self.act) if n != "gate" else self.ctx.to_device(x[n])) for n in x}
         out, qr = self.ctx.alloc(T * p["H"] * p["vdim"] * 4), self.ctx.alloc(T * p["H"] * 2 * p["dim"] * 4)
-        self.orn.diff_attn(self.ctx, act=self.act, cos=self.d_cos, sin=self.d_sin, rope_dims=self.rot, table_npos=self.cap, T=T,
+        self.orn.diff_attn(self.ctx, act=self.act, cos=self.d_cos, sin=self.d_sin, rope_dims=self.rot,
+                table_npos=self.cap, T=T,
                            offset=self.offset, cap=self.cap, window=self.size, keep_first=self.keep, scale=self.scale, lam=self.lam,
                            diff=self.diff, eps=1e-5, k_cache=self.kc, v_cache=self.vc, q_rot=qr, out=out, **d, **p)
         self.offset += T
@@ -331,7 +351,8 @@ class Attention:
 
 SHAPES = [  # H, G, dim, vdim, size, keep, rot
     (2, 1, 16, 16, 5, 2, 8), (4, 4, 32, 64, 64, 0, 32), (6, 2, 24, 40, 65, 3, 4), (4, 1, 72, 136, 100, 70, 72),
-    (2, 2, 128, 256, 33, 128, 64), (2, 1, 14, 9, 20, 7, 6), (3, 1, 6, 10, 1, 1, 2), (2, 1, 8, 8, 0, 0, 0), (4, 2, 64, 128, 1000, 20, 32)]
+    (2, 2, 128, 256, 33, 128, 64), (2, 1, 14, 9, 20, 7, 6), (3, 1, 6, 10, 1, 1, 2), (2, 1, 8, 8, 0, 0, 0), (4, 2, 64, 128,
+            1000, 20, 32)]
 
 
 @pytest.mark.parametrize("act", [0, 1])
@@ -340,7 +361,8 @@ def test_attention_portions(orn, ctx, act, shape):
     """Portions of many lengths (decode and matrix-core widths) into one cache of garbage, windows shorter
     and longer than a key block, kept tokens fewer and more than a block, grouped heads."""
     H, G, dim, vdim, size, keep, rot = shape
-    att, rng = Attention(orn, ctx, act, H, G, dim, vdim, size, keep, rot, factor=2.0), np.random.default_rng(dim * 31 + vdim)
+    att, rng = Attention(orn, ctx, act, H, G, dim, vdim, size, keep, rot,
+            factor=2.0), np.random.default_rng(dim * 31 + vdim)
     for T in (1, 2, 40, 1, 64, 33, 3, 100, 1, 7):
         x = att.inputs(rng, T)
         _close(att.step(x), att.want(x), act, (shape, T), slack=4.0 if act == 0 else 1.5)
@@ -355,7 +377,8 @@ def test_attention_edges(orn, ctx, act, size, keep):
     with a window one longer or shorter, or one kept token more or fewer, is far away at these rows."""
     H, G, dim, vdim, rot = 2, 1, 24, 24, 8
     n = 230
-    spots = sorted({j for j in (0, keep - 1, keep, keep + 1, 63, 64, n - 1 - size, n - size, n - size + 1, n - 2) if 0 <= j < n - 1})
+    spots = sorted({j for j in (0, keep - 1, keep, keep + 1, 63, 64, n - 1 - size, n - size, n - size + 1,
+            n - 2) if 0 <= j < n - 1})
     for spot in spots:
         rng = np.random.default_rng(spot)
         att = Attention(orn, ctx, act, H, G, dim, vdim, size, keep, rot)
@@ -368,7 +391,8 @@ def test_attention_edges(orn, ctx, act, size, keep):
         seen = R.visible(n - 1, spot, size, keep)
         for cut in (n, n - 1):
             a2 = Attention(orn, ctx, act, H, G, dim, vdim, size, keep, rot)
-            got = np.concatenate([a2.step({k: a[:cut] for k, a in x.items()})] + ([a2.step({k: a[cut:] for k, a in x.items()})] if cut < n else []))
+            got = np.concatenate([a2.step({k: a[:cut] for k, a in x.items()})] + ([a2.step({k: a[cut:] for k,
+                    a in x.items()})] if cut < n else []))
             _close(got[-3:], want[-3:], act, (spot, cut), slack=4.0 if act == 0 else 1.5)
             a2.close()
         for other in ((size + 1, keep), (max(size - 1, 1), keep), (size, keep + 1), (size, max(keep - 1, 0))):
@@ -399,13 +423,16 @@ def test_attention_of_single_rows_does_not_depend_on_the_call(orn, ctx):
 def test_refusals(orn, ctx):
     """Calls the kernels cannot run come back as errors from the host."""
     b = ctx.alloc(1 << 16)
-    ok = dict(act=1, q=b, k=b, v=b, gate=b, cos=b, sin=b, rope_dims=4, table_npos=64, T=1, H=2, G=1, dim=8, vdim=8, offset=0, cap=64,
+    ok = dict(act=1, q=b, k=b, v=b, gate=b, cos=b, sin=b, rope_dims=4, table_npos=64, T=1, H=2, G=1, dim=8, vdim=8,
+            offset=0, cap=64,
               window=4, keep_first=0, scale=1.0, lam=0.5, diff=0.5, eps=1e-6, k_cache=b, v_cache=b, q_rot=b, out=b)
-    for bad in (dict(H=3, G=2), dict(rope_dims=3), dict(rope_dims=10), dict(offset=64), dict(offset=60, T=5), dict(table_npos=0), dict(window=-1)):
+    for bad in (dict(H=3, G=2), dict(rope_dims=3), dict(rope_dims=10), dict(offset=64), dict(offset=60, T=5),
+            dict(table_npos=0), dict(window=-1)):
         with pytest.raises(orn.OrnithError):
             orn.diff_attn(ctx, **dict(ok, **bad))
     s = orn.mlstm_state_floats(1, 8, 8) * 4
-    ok = dict(act=1, q=b, k=b, v=b, gi=b, gf=b, bi=b, bf=b, gate_cap=4.0, T=1, H=1, dim=8, vdim=8, state_in=b, slots=b, n_slots=2,
+    ok = dict(act=1, q=b, k=b, v=b, gi=b, gf=b, bi=b, bf=b, gate_cap=4.0, T=1, H=1, dim=8, vdim=8, state_in=b, slots=b,
+            n_slots=2,
               first_slot=1, snapshots=0, o=b)
     for bad in (dict(dim=513), dict(first_slot=2), dict(first_slot=0), dict(T=2, snapshots=1), dict(gate_cap=0.0)):
         with pytest.raises(orn.OrnithError):

@@ -62,7 +62,8 @@ class Want:
         rng = np.random.default_rng(99)
         self.act, self.logits = act, R.Run(cfg, w).feed(toks)
         size = 2.0 ** -22 if act == 0 else 2.0 ** -9
-        moved = [_err(R.Run(cfg, w, lambda x: x * (1 + size * rng.uniform(-1, 1, np.shape(x)))).feed(toks), self.logits) for _ in range(4)]
+        moved = [_err(R.Run(cfg, w, lambda x: x * (1 + size * rng.uniform(-1, 1, np.shape(x)))).feed(toks),
+                self.logits) for _ in range(4)]
         self.limit = np.maximum(LIMIT[act], 3 * np.max(moved, axis=0))
 
     def check(self, got, what, at=0):
@@ -70,7 +71,8 @@ class Want:
         rows = at if isinstance(at, list) else slice(at, at + len(got))
         e = _err(np.asarray(got, np.float64), self.logits[rows]) / self.limit[rows]
         # (four disturbed runs do not find every touchy position)
-        assert e.max() < 2 and np.sum(e > 1) <= max(1, len(e) // 50), (what, float(e.max()), int(e.argmax()), int(np.sum(e > 1)))
+        assert e.max() < 2 and np.sum(e > 1) <= max(1, len(e) // 50), (what, float(e.max()), int(e.argmax()),
+                int(np.sum(e > 1)))
 
 
 @pytest.mark.parametrize("act", [0, 1])
@@ -156,7 +158,8 @@ def test_rewind(orn, ctx, name):
         Want(cfg, w, follow, 0).check(d.feed(toks[50:60]), (name, keep), at=40 + keep)
         d.feed(toks[44:47], capture=True)
         d.model.rewind(d.caches, 3)
-        Want(cfg, w, np.concatenate([follow, toks[44:48]]), 0).check(d.feed(toks[47:48]), (name, keep, "again"), at=len(follow) + 3)
+        Want(cfg, w, np.concatenate([follow, toks[44:48]]), 0).check(d.feed(toks[47:48]), (name, keep, "again"),
+                at=len(follow) + 3)
     d.close()
 
 
@@ -202,7 +205,8 @@ def _write_model(tmp_path, cfg, w, orn):
     os.mkdir(d)
     with open(os.path.join(d, "config.json"), "w") as f:
         json.dump(cfg, f)
-    synth.write_safetensors(os.path.join(d, "model.safetensors"), {n: (util.f32_to_bf16(a), orn.DT_BF16) for n, a in w.items()})
+    synth.write_safetensors(os.path.join(d, "model.safetensors"), {n: (util.f32_to_bf16(a), orn.DT_BF16) for n,
+            a in w.items()})
     return d
 
 
