@@ -848,7 +848,7 @@ def design_kernels(orn, ctx, np, width, only=None):
             wg, wu, wd = dense(ff, W, n), dense(ff, W, n), dense(W, ff, n)
             act = ctx.alloc(T * ff * 2)
             us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [wg[i % n], wu[i % n]], [act, None], [0,
-                    0], pre=orn.PRE_NORM, norm_w=wn, w_offset=1.0, gelu_pair=True) for i in range(n)]))
+                    0], pre=orn.PRE_NORM, norm_w=wn, w_offset=1.0, pair_act=orn.PAIR_GELU) for i in range(n)]))
             mine = row(f"norm + gate, up + gelu (T = {T})", us, 2 * ff * W * 2)
             us2 = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, act, T, ff, [wd[i % n]], [xs],
                     [orn.OUT_ADD]) for i in range(n)]))
@@ -931,7 +931,7 @@ def design_kernels(orn, ctx, np, width, only=None):
             wg, wu, wd = dense(ff, W, 1)[0], dense(ff, W, 1)[0], dense(W, ff, 1)[0]
             act, xs = ctx.alloc(T * ff * 2), dev((T, W), "f32")
             us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, x, T, W, [wg, wu], [act, None], [0, 0],
-                    gelu_pair=True) for i in range(1)]), **reps)
+                    pair_act=orn.PAIR_GELU) for i in range(1)]), **reps)
             pair(f"prefill GEMM gate, up + gelu, T = {T}", row(f"gate, up + gelu (T = {T})", us,
                     2 * ff * W * 2 + T * (W + ff) * 2, 4.0 * T * W * ff), peer, "in_proj qkv, z (Q4_K)")
             us = t_of(calls(orn.dense_rows, [orn.dense_call(orn.BF16, act, T, ff, [wd], [xs],

@@ -102,6 +102,7 @@ ORNITH_API int ornith_device_info(ornith_ctx* ctx, char* name, size_t name_len, 
  *   "mlstm_chunked" (ORNITH_MLSTM_CHUNKED, default 1): the mLSTM recurrence of calls of 64 rows
  *               or more runs in 64-token chunks on the matrix cores (0: token by token); results
  *               agree to rounding
+ *   "retention_chunked" (ORNITH_RETENTION_CHUNKED, default 1): likewise for the retention recurrence
  *   "fuse_moe_one" (ORNITH_FUSE_MOE_ONE, default 0): the MoE block's phases as ranges of
  *               workgroups of ONE launch that hand their intermediates over through memory
  *               (1: router + up + down, 2: up + down after a router launch). Bit-identical,
@@ -366,6 +367,12 @@ ORNITH_API int ornith_rope_table(ornith_ctx* ctx, int npos, int dims, double the
 /* the same with every frequency divided by `factor` (linear position scaling) */
 ORNITH_API int ornith_rope_table_scaled(ornith_ctx* ctx, int npos, int dims, double theta, double factor,
                                         float* d_cos, float* d_sin);
+/* YaRN (Peng et al., "YaRN: Efficient Context Window Extension of Large Language Models"): with
+ * d(t) = dims ln(original / (2 pi t)) / (2 ln theta) the pair that turns t times over `original` positions,
+ * pairs below floor(d(fast)) keep their frequency, pairs above ceil(d(slow)) get a factor-th of it, a linear
+ * ramp lies between; cos and sin are multiplied by 0.1 ln(factor) + 1. */
+ORNITH_API int ornith_rope_table_yarn(ornith_ctx* ctx, int npos, int dims, double theta, double factor, double original,
+                                      double fast, double slow, float* d_cos, float* d_sin);
 /* Attention::forward up to the cache write (src/model/qwen3_5.rs:439-463): per-head
  * rms_norm of q and k (weights [hd]), partial RoPE at position offset + t, append of
  * K and V at rows [offset, offset+T) of the caches bf16 [Hkv, cap, hd]
@@ -410,10 +417,15 @@ ORNITH_API int ornith_sdpa_prefill_gated(ornith_ctx* ctx, const void* d_q_rot, c
 #define ORNITH_PRE_NONE 0  /* d_x: act [M, K] */
 #define ORNITH_PRE_NORM 1  /* d_x: f32 [M, K]; rows = x / sqrt(mean(x^2) + eps) * (w_offset + w) */
 #define ORNITH_PRE_HEADS 2 /* d_x: f32 [M, K]: heads of head_dim values, each over its own root mean
-                              square, times w [K], times sigmoid(gate), gate: act [M, K] */
+                              square, times w [K] (no w: as it is), times gate_act(gate), gate: act [M, K] */
+#define ORNITH_GATE_SIGMOID 0
+#define ORNITH_GATE_SILU 1
 #define ORNITH_OUT_ACT 0   /* y: act [M, O] */
 #define ORNITH_OUT_F32 1   /* y: f32 [M, O] */
-#define ORNITH_OUT_ADD 2   /* y: f32 [M, O], added to */
+#define ORNITH_OUT_ADD 2   /* y: f32 [M, O], add_scale times the sum added to it */
+#define ORNITH_PAIR_NONE 0
+#define ORNITH_PAIR_GELU 1 /* n == 2: d_y[0] (act) = gelu_tanh(w[0] row) * (w[1] row) */
+#define ORNITH_PAIR_SILU 2 /* the same with z sigmoid(z) */
 typedef struct ornith_dense_call {
   int act, pre;
   const void* d_x;
@@ -426,18 +438,24 @@ typedef struct ornith_dense_call {
   const ornith_linear* w[6];
   void* d_y[6];
   int out[6];
-  int gelu_pair; /* n == 2: d_y[0] (act) = gelu_tanh(w[0] row) * (w[1] row) */
+  int pair_act;  /* ORNITH_PAIR_* */
   void* d_rows;  /* act [M, K]: where the rows a prologue makes are kept for a GEMM (may be null below it) */
+  int gate_act;  /* ORNITH_GATE_* */
+  float add_scale;
+  float soft_cap; /* > 0: sums stored (not added) become soft_cap tanh(sum / soft_cap) */
 } ornith_dense_call;
 ORNITH_API int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* call);
 /* the prologues alone */
 ORNITH_API int ornith_norm_rows(ornith_ctx* ctx, const float* d_x, const void* d_w, float w_offset, int rows, int n,
                                 float eps, int act, void* d_out);
-ORNITH_API int ornith_head_norm_gate(ornith_ctx* ctx, const float* d_x, const void* d_w, const void* d_gate, int rows,
-                                     int heads, int head_dim, float eps, int act, void* d_out);
+ORNITH_API int ornith_head_norm_gate(ornith_ctx* ctx, const float* d_x, const void* d_w, const void* d_gate, int gate_act,
+                                     int rows, int heads, int head_dim, float eps, int act, void* d_out);
 /* rows of a dense bf16 table times `scale`, f32; ids are clamped to the table */
 ORNITH_API int ornith_embed_rows(ornith_ctx* ctx, const ornith_linear* table, const uint32_t* d_ids, int n, float scale,
                                  float* d_out);
+/* rows of a dense bf16 table, each over its root mean square times (w_offset + w), f32 */
+ORNITH_API int ornith_embed_norm_rows(ornith_ctx* ctx, const ornith_linear* table, const uint32_t* d_ids, int n,
+                                      const void* d_w, float w_offset, float eps, float* d_out);
 
 /* n floats to bf16 */
 ORNITH_API int ornith_round_bf16(ornith_ctx* ctx, const float* d_x, size_t n, void* d_out);
@@ -491,6 +509,64 @@ typedef struct ornith_diff_attn_call {
   void *d_k_cache, *d_v_cache, *d_q_rot, *d_out;
 } ornith_diff_attn_call;
 ORNITH_API int ornith_diff_attn(ornith_ctx* ctx, const ornith_diff_attn_call* call);
+
+/* ---- retention: linear attention with a fixed decay a head -------------------------------
+ * Sun et al., "Retentive Network: A Successor to Transformer for Large Language Models". Per head, with q and
+ * k turned by their position on the first rope_dims dimensions (dimension i pairs with i + rope_dims/2; tables
+ * f32 [table_npos, rope_dims/2], row = position) and k then scaled by dim^(-1/2):
+ *   S' = decay S + k v^T;  o = S'^T q
+ * q, k: act [T, H*dim], v: act [T, H*vdim] at positions offset ..; d_decay: f32 [H][ORNITH_DECAY_POWERS], the
+ * powers 0, 1, .. of each head's decay (ornith_decay_powers makes them); o: f32 [T, H*vdim]. State and slots as
+ * in ornith_mlstm, ornith_retention_state_floats floats a slot. Calls of 64 rows or more (bf16, dim, vdim
+ * multiples of 8, dim <= 256, no snapshots; option retention_chunked) run in chunks of 64 tokens on the matrix
+ * cores, everything that enters the recurrence besides v in two bf16 parts. */
+#define ORNITH_DECAY_POWERS 65
+typedef struct ornith_retention_call {
+  int act;
+  const void *d_q, *d_k, *d_v;
+  const float *d_cos, *d_sin;
+  int rope_dims, table_npos, offset;
+  const float* d_decay;
+  int T, H, dim, vdim;
+  const float* d_state_in;
+  float* d_slots;
+  int n_slots, first_slot, snapshots;
+  float* d_o;
+} ornith_retention_call;
+ORNITH_API size_t ornith_retention_state_floats(int H, int dim, int vdim);
+ORNITH_API int ornith_decay_powers(ornith_ctx* ctx, int H, const double* decay, float* d_out);
+ORNITH_API int ornith_retention(ornith_ctx* ctx, const ornith_retention_call* call);
+
+/* ---- latent attention over a cache of low-rank rows ----------------------------------------
+ * DeepSeek-AI, "DeepSeek-V2: A Strong, Economical, and Efficient Mixture-of-Experts Language Model" (MLA). One
+ * row a token and no heads: down f32 [T, rank + rot_dim] gives the latent c = down[:rank] over its root mean
+ * square times d_down_norm (bf16 [rank]), kept in d_c_cache act [cap, rank], and a key part turned by its
+ * position (pairs (2i, 2i+1), tables f32 [table_npos, rot_dim/2]), kept in d_r_cache act [cap, rot_dim], at
+ * rows [offset, offset + T). d_down null: those rows are there already. q: act [T, H, dim + rot_dim], the last
+ * rot_dim of a head turned here. A head's unturned keys are uk c (uk [H*dim, rank]), its values uv c
+ * (uv [H*vdim, rank]);
+ *   score_ij = scale (q_i . uk c_j + turned q_i . r_j),  j <= i and i - j < window (window 0: any j <= i)
+ *   o_i = sum_j e^score_ij uv c_j / (sum_j e^score_ij + e^sink), times sigmoid(gate): act [T, H*vdim]
+ * sink: bf16 [H] or null (none); gate: f32 [T, H] or null (1). bf16 calls of gemm_rows rows or more (sizes
+ * multiples of 8, dim and rot_dim rounded up to 32 at most 256 together, vdim <= 256) make keys and values of
+ * the rows in sight and run flash attention on the matrix cores; others take queries and results through
+ * uk and uv instead and read the cached rows as they are. */
+typedef struct ornith_latent_attn_call {
+  int act;
+  const void* d_q;
+  const float* d_down;
+  const void* d_down_norm;
+  const ornith_linear *uk, *uv;
+  const float* d_gate;
+  const void* d_sink;
+  const float *d_cos, *d_sin;
+  int table_npos;
+  int T, H, dim, rot_dim, vdim, rank;
+  int offset, cap, window;
+  float scale, eps;
+  void *d_c_cache, *d_r_cache, *d_out;
+} ornith_latent_attn_call;
+ORNITH_API int ornith_latent_attn(ornith_ctx* ctx, const ornith_latent_attn_call* call);
 
 /* ---- greedy selection: src/ops/sample.rs ------------------------------------------ */
 /* greedy_token / the verify rows of generate_step_mtp (src/ops/sample.rs:134-147,
@@ -616,8 +692,8 @@ ORNITH_API int ornith_model_load(ornith_ctx* ctx, const ornith_weights* ws,
 ORNITH_API int ornith_text_config_load(const char* model_dir, ornith_text_config* out,
                                        int* mtp_layers);
 /* The model registry: config.json's "architecture" names the design ("Pigodra": mLSTM and
- * differential-attention layers over a 32-bit residual stream; no such key: the Qwen3.5 keys of
- * ornith_text_config_load). act_dtype: ORNITH_BF16, or ORNITH_F32 for activations, products and
+ * differential-attention layers over a 32-bit residual stream; "Ranavik": retention and latent-attention
+ * layers side by side with their feed-forwards; no such key: the Qwen3.5 keys of ornith_text_config_load). act_dtype: ORNITH_BF16, or ORNITH_F32 for activations, products and
  * KV rows in 32-bit where the design runs so (ORNITH_ERR_UNSUPPORTED otherwise). load_json takes
  * the text of a config.json (for a store filled with ornith_weights_put). The store must outlive
  * the model. */

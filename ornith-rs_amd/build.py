@@ -38,7 +38,11 @@ FLAGS += os.environ.get("ORN_EXTRA_FLAGS", "").split()
 # What every design needs, and what each design of the registry adds (a design that is not listed
 # needs the whole library).
 CORE = ["runtime.hip", "weights.cpp", "safetensors.cpp", "model.cpp", "rope.cpp", "engine.cpp", "sample.hip", "sampler.hip"]
-DESIGNS = {"Pigodra": ["pigodra.cpp", "stack.cpp", "dense_rows.hip", "mlstm.hip", "diff_attn.hip"]}
+DESIGNS = {
+    "Pigodra": ["pigodra.cpp", "stack.cpp", "dense_rows.hip", "mix_mlstm.cpp", "mlstm.hip", "mix_diff_attn.cpp", "diff_attn.hip"],
+    "Ranavik": ["ranavik.cpp", "stack.cpp", "dense_rows.hip", "mix_retention.cpp", "retention.hip", "mix_latent_attn.cpp",
+                "latent_attn.hip"],
+}
 
 
 def sources(design=None):

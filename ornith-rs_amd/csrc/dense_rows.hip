@@ -1,6 +1,6 @@
 // Dense bf16 projections of the designs with a 32-bit residual stream, with what surrounds them
 // in the same launch: the norm or the per-head norm and gate that makes their input in the head,
-// the residual sum or the gated gelu in the tail.
+// the residual sum, the gated pair's activation or the soft cap in the tail.
 //
 // Decode widths (and 32-bit models at every width): a wavefront takes pairs of output rows over up
 // to four activation rows; every workgroup makes the input rows itself (they are a few KB and come
@@ -20,7 +20,8 @@ struct RowsArgs {
   const void* x;
   const bf16_t* wn;
   const void* gate;
-  float w_offset, eps;
+  float w_offset, eps, add_scale, soft_cap;
+  int gate_act, pair_act;
   int head, M, K;
   int n;
   const bf16_t* w[kSegs];
@@ -28,6 +29,23 @@ struct RowsArgs {
   int O[kSegs];
   int out[kSegs];
 };
+
+__device__ __forceinline__ float gate_of(int kind, float z) {
+  const float s = dm_sigmoid_f32(z);
+  return kind == ORNITH_GATE_SILU ? z * s : s;
+}
+__device__ __forceinline__ float pair_of(int kind, float gate, float up) {
+  return (kind == ORNITH_PAIR_SILU ? gate * dm_sigmoid_f32(gate) : dm_gelu_tanh(gate)) * up;
+}
+// a sum as it is stored
+__device__ __forceinline__ float stored(const RowsArgs& p, float v) {
+  return p.soft_cap > 0.f ? p.soft_cap * dm_tanh(v / p.soft_cap) : v;
+}
+// four norm weights; none: ones
+__device__ __forceinline__ void norm_weights(const bf16_t* w, float (&v)[4]) {
+  v[0] = v[1] = v[2] = v[3] = 1.0f;
+  if (w) act_load<4>(w, v);
+}
 
 // ---- decode widths ------------------------------------------------------------------------
 constexpr int NT = 256, NR = 2, NU = 4;
@@ -189,7 +207,7 @@ __global__ __launch_bounds__(NT) void dense_rows_kernel(RowsArgs p, int groups) 
         if (i >= K) return;
         const float4 x4 = value(m, c, i);
         float v[4] = {x4.x, x4.y, x4.z, x4.w}, wv[4];
-        act_load<4>(p.wn + i, wv);
+        norm_weights(p.wn ? p.wn + i : nullptr, wv);
         if constexpr (PRE == ORNITH_PRE_NORM) {
 #pragma unroll
           for (int e = 0; e < 4; ++e) v[e] = (v[e] * rinv) * (p.w_offset + wv[e]);
@@ -198,7 +216,7 @@ __global__ __launch_bounds__(NT) void dense_rows_kernel(RowsArgs p, int groups) 
           float gv[4] = {};
           if (m0 + m < p.M) act_load<4>(reinterpret_cast<const A*>(p.gate) + (size_t)(m0 + m) * K + i, gv);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v[e] = ((v[e] * hinv) * wv[e]) * dm_sigmoid_f32(gv[e]);
+          for (int e = 0; e < 4; ++e) v[e] = ((v[e] * hinv) * wv[e]) * gate_of(p.gate_act, gv[e]);
         }
         act_store4(&xs[m * Kp + i], v);
       };
@@ -230,9 +248,9 @@ __global__ __launch_bounds__(NT) void dense_rows_kernel(RowsArgs p, int groups) 
         const float rinv = dm_rsqrt((((aux[0] + aux[1]) + aux[2]) + aux[3]) / (float)head + p.eps);
         for (int i = tid; i < head; i += NT) {
           float v = live ? src[h0 + i] * rinv : 0.f;
-          const float wv = dm_bf2f(p.wn[h0 + i]);
+          const float wv = p.wn ? dm_bf2f(p.wn[h0 + i]) : 1.0f;
           if constexpr (PRE == ORNITH_PRE_NORM) v = v * (p.w_offset + wv);
-          else v = (v * wv) * dm_sigmoid_f32(live ? act_f(gsrc[h0 + i]) : 0.f);
+          else v = (v * wv) * gate_of(p.gate_act, live ? act_f(gsrc[h0 + i]) : 0.f);
           xs[m * Kp + h0 + i] = act_of<A>(v);
         }
       }
@@ -302,15 +320,15 @@ __global__ __launch_bounds__(NT) void dense_rows_kernel(RowsArgs p, int groups) 
       for (int m = 0; m < MR; ++m) {
         if (m0 + m >= p.M) continue;
         if constexpr (PAIR) {
-          reinterpret_cast<A*>(y)[(size_t)(m0 + m) * O + o_now] = act_of<A>(dm_gelu_tanh(v[0][m]) * v[1][m]);
+          reinterpret_cast<A*>(y)[(size_t)(m0 + m) * O + o_now] = act_of<A>(pair_of(p.pair_act, v[0][m], v[1][m]));
         } else {
 #pragma unroll
           for (int r = 0; r < NR; ++r) {
             if (o_now + r >= O) continue;
             const size_t at = (size_t)(m0 + m) * O + o_now + r;
-            if (kind == ORNITH_OUT_ACT) reinterpret_cast<A*>(y)[at] = act_of<A>(v[r][m]);
-            else if (kind == ORNITH_OUT_F32) reinterpret_cast<float*>(y)[at] = v[r][m];
-            else reinterpret_cast<float*>(y)[at] += v[r][m];
+            if (kind == ORNITH_OUT_ACT) reinterpret_cast<A*>(y)[at] = act_of<A>(stored(p, v[r][m]));
+            else if (kind == ORNITH_OUT_F32) reinterpret_cast<float*>(y)[at] = stored(p, v[r][m]);
+            else reinterpret_cast<float*>(y)[at] += p.add_scale * v[r][m];
           }
         }
       }
@@ -421,10 +439,10 @@ __global__ __launch_bounds__(NT) void norm_rows_kernel(const float* x, const bf1
   }
 }
 
-// one wavefront a head of a row: act(x / rms_head * w * sigmoid(gate))
+// one wavefront a head of a row: act(x / rms_head * w * gate_act(gate))
 template <typename A>
-__global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* x, const bf16_t* w, const A* gate, float eps,
-                                                            int heads, int head, int total, A* out) {
+__global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* x, const bf16_t* w, const A* gate, int gate_act,
+                                                            float eps, int heads, int head, int total, A* out) {
   const int hr = blockIdx.x * (NT / 64) + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (hr >= total) return;
   const size_t base = (size_t)hr * head;
@@ -439,17 +457,17 @@ __global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* x, cons
     for (int i = 4 * lane; i < head; i += 256) {
       const float4 x4 = *reinterpret_cast<const float4*>(x + base + i);
       float wv[4], gv[4];
-      act_load<4>(w + w0 + i, wv);
+      norm_weights(w ? w + w0 + i : nullptr, wv);
       act_load<4>(gate + base + i, gv);
-      const float v[4] = {((x4.x * inv) * wv[0]) * dm_sigmoid_f32(gv[0]), ((x4.y * inv) * wv[1]) * dm_sigmoid_f32(gv[1]),
-                          ((x4.z * inv) * wv[2]) * dm_sigmoid_f32(gv[2]), ((x4.w * inv) * wv[3]) * dm_sigmoid_f32(gv[3])};
+      const float v[4] = {((x4.x * inv) * wv[0]) * gate_of(gate_act, gv[0]), ((x4.y * inv) * wv[1]) * gate_of(gate_act, gv[1]),
+                          ((x4.z * inv) * wv[2]) * gate_of(gate_act, gv[2]), ((x4.w * inv) * wv[3]) * gate_of(gate_act, gv[3])};
       act_store4(out + base + i, v);
     }
   } else {
     for (int i = lane; i < head; i += 64) a = dm_fma(x[base + i], x[base + i], a);
     const float inv = dm_rsqrt(dm_wave_sum<64>(a) / (float)head + eps);
     for (int i = lane; i < head; i += 64)
-      out[base + i] = act_of<A>(((x[base + i] * inv) * dm_bf2f(w[w0 + i])) * dm_sigmoid_f32(act_f(gate[base + i])));
+      out[base + i] = act_of<A>(((x[base + i] * inv) * (w ? dm_bf2f(w[w0 + i]) : 1.0f)) * gate_of(gate_act, act_f(gate[base + i])));
   }
 }
 
@@ -469,6 +487,57 @@ __global__ __launch_bounds__(NT) void embed_rows_kernel(const bf16_t* table, con
   } else {
     for (int e = i; e < min(i + 4, n); ++e) dst[e] = dm_bf2f(src[e]) * scale;
   }
+}
+
+// x = table[id] / rms * (w_offset + w), fp32: a workgroup a row
+__global__ __launch_bounds__(NT) void embed_norm_rows_kernel(const bf16_t* table, const uint32_t* ids, int V, int n,
+                                                             const bf16_t* w, float w_offset, float eps, float* out) {
+  __shared__ float red[4];
+  const bf16_t* src = table + (size_t)min(ids[blockIdx.x], (uint32_t)(V - 1)) * n;
+  float* dst = out + (size_t)blockIdx.x * n;
+  const int tid = threadIdx.x;
+  constexpr int PC = 4;
+  const bool vec = n % 8 == 0;
+  float x[PC][8];
+  float a = 0.f;
+  if (vec) {
+#pragma unroll
+    for (int c = 0; c < PC; ++c) {
+      const int i = 8 * (tid + NT * c);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[c][e] = 0.f;
+      if (i < n) act_load<8>(src + i, x[c]);
+    }
+#pragma unroll
+    for (int c = 0; c < PC; ++c)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) a = dm_fma(x[c][e], x[c][e], a);
+  }
+  for (int i = vec ? 8 * NT * PC + tid : tid; i < n; i += NT) {
+    const float v = dm_bf2f(src[i]);
+    a = dm_fma(v, v, a);
+  }
+  a = dm_wave_sum<64>(a);
+  if ((tid & 63) == 0) red[tid >> 6] = a;
+  __syncthreads();
+  const float inv = dm_rsqrt((((red[0] + red[1]) + red[2]) + red[3]) / (float)n + eps);
+  if (vec) {
+#pragma unroll
+    for (int c = 0; c < PC; ++c) {
+      const int i = 8 * (tid + NT * c);
+      if (i >= n) continue;
+      float wv[8];
+      act_load<8>(w + i, wv);
+#pragma unroll
+      for (int h = 0; h < 2; ++h) {
+        float v[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = (x[c][4 * h + e] * inv) * (w_offset + wv[4 * h + e]);
+        act_store4(dst + i + 4 * h, v);
+      }
+    }
+  }
+  for (int i = vec ? 8 * NT * PC + tid : tid; i < n; i += NT) dst[i] = (dm_bf2f(src[i]) * inv) * (w_offset + dm_bf2f(w[i]));
 }
 
 __global__ __launch_bounds__(NT) void round_bf16_kernel(const float* x, size_t n, bf16_t* out) {
@@ -606,11 +675,11 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(RowsArgs p, int tiles_n
         if constexpr (PAIR) {
           f = n0 + wn * 32 + 8 * q + 4 * lh;
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v[e] = dm_gelu_tanh(acc[0][b][4 * q + e]) * acc[NTL - 1][b][4 * q + e];
+          for (int e = 0; e < 4; ++e) v[e] = pair_of(p.pair_act, acc[0][b][4 * q + e], acc[NTL - 1][b][4 * q + e]);
         } else {
           f = n0 + wn * (BN / 2) + a * 32 + 8 * q + 4 * lh;
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v[e] = acc[a][b][4 * q + e];
+          for (int e = 0; e < 4; ++e) v[e] = kind == ORNITH_OUT_ADD ? p.add_scale * acc[a][b][4 * q + e] : stored(p, acc[a][b][4 * q + e]);
         }
         const size_t at = (size_t)m * O + f;
         if (f + 3 < O && (O & 3) == 0) {
@@ -678,17 +747,17 @@ int ornith_norm_rows(ornith_ctx* ctx, const float* d_x, const void* d_w, float w
   return ORNITH_OK;
 }
 
-int ornith_head_norm_gate(ornith_ctx* ctx, const float* d_x, const void* d_w, const void* d_gate, int rows, int heads, int head,
-                          float eps, int act, void* d_out) {
-  ORN_REQUIRE(ctx && d_x && d_w && d_gate && d_out, "head_norm_gate: null argument");
+int ornith_head_norm_gate(ornith_ctx* ctx, const float* d_x, const void* d_w, const void* d_gate, int gate_act, int rows,
+                          int heads, int head, float eps, int act, void* d_out) {
+  ORN_REQUIRE(ctx && d_x && d_gate && d_out, "head_norm_gate: null argument");
   ORN_REQUIRE(rows >= 1 && heads >= 1 && head >= 1, "head_norm_gate: rows=%d heads=%d of %d", rows, heads, head);
   const int total = rows * heads, wgs = (total + NT / 64 - 1) / (NT / 64);
   if (act == ORNITH_F32)
     hipLaunchKernelGGL(head_norm_gate_kernel<float>, dim3(wgs), dim3(NT), 0, ctx->stream, d_x, (const bf16_t*)d_w,
-                       (const float*)d_gate, eps, heads, head, total, (float*)d_out);
+                       (const float*)d_gate, gate_act, eps, heads, head, total, (float*)d_out);
   else
     hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, dim3(wgs), dim3(NT), 0, ctx->stream, d_x, (const bf16_t*)d_w,
-                       (const bf16_t*)d_gate, eps, heads, head, total, (bf16_t*)d_out);
+                       (const bf16_t*)d_gate, gate_act, eps, heads, head, total, (bf16_t*)d_out);
   ORN_LAUNCH_CHECK("head_norm_gate_kernel");
   return ORNITH_OK;
 }
@@ -699,6 +768,16 @@ int ornith_embed_rows(ornith_ctx* ctx, const ornith_linear* table, const uint32_
   hipLaunchKernelGGL(embed_rows_kernel, dim3((table->K + 4 * NT - 1) / (4 * NT), n), dim3(NT), 0, ctx->stream, (const bf16_t*)table->d_w, d_ids, scale, table->O,
                      table->K, d_out);
   ORN_LAUNCH_CHECK("embed_rows_kernel");
+  return ORNITH_OK;
+}
+
+int ornith_embed_norm_rows(ornith_ctx* ctx, const ornith_linear* table, const uint32_t* d_ids, int n, const void* d_w,
+                           float w_offset, float eps, float* d_out) {
+  ORN_REQUIRE(ctx && table && d_ids && d_w && d_out, "embed_norm_rows: null argument");
+  ORN_REQUIRE(table->mode == ORNITH_LIN_DENSE && table->d_w && n >= 1, "embed_norm_rows: table mode %d, n=%d", table->mode, n);
+  hipLaunchKernelGGL(embed_norm_rows_kernel, dim3(n), dim3(NT), 0, ctx->stream, (const bf16_t*)table->d_w, d_ids, table->O, table->K,
+                     (const bf16_t*)d_w, w_offset, eps, d_out);
+  ORN_LAUNCH_CHECK("embed_norm_rows_kernel");
   return ORNITH_OK;
 }
 
@@ -715,8 +794,8 @@ int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* c) {
   ORN_REQUIRE(c->act == ORNITH_BF16 || c->act == ORNITH_F32, "dense_rows: activation type %d", c->act);
   ORN_REQUIRE(c->M >= 1 && c->K >= 1 && c->n >= 1 && c->n <= kSegs, "dense_rows: M=%d K=%d n=%d", c->M, c->K, c->n);
   ORN_REQUIRE(c->pre >= ORNITH_PRE_NONE && c->pre <= ORNITH_PRE_HEADS, "dense_rows: prologue %d", c->pre);
-  ORN_REQUIRE(c->pre == ORNITH_PRE_NONE || c->d_norm_w, "dense_rows: norm weight missing");
-  ORN_REQUIRE(c->pre != ORNITH_PRE_HEADS || (c->d_gate && c->head_dim >= 1 && c->K % c->head_dim == 0 && !c->gelu_pair),
+  ORN_REQUIRE(c->pre != ORNITH_PRE_NORM || c->d_norm_w, "dense_rows: norm weight missing");
+  ORN_REQUIRE(c->pre != ORNITH_PRE_HEADS || (c->d_gate && c->head_dim >= 1 && c->K % c->head_dim == 0 && !c->pair_act),
               "dense_rows: heads of %d in rows of %d", c->head_dim, c->K);
   RowsArgs p{};
   p.x = c->d_x;
@@ -724,6 +803,10 @@ int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* c) {
   p.gate = c->d_gate;
   p.w_offset = c->w_offset;
   p.eps = c->eps;
+  p.add_scale = c->add_scale;
+  p.soft_cap = c->soft_cap;
+  p.gate_act = c->gate_act;
+  p.pair_act = c->pair_act;
   p.head = c->head_dim;
   p.M = c->M;
   p.K = c->K;
@@ -738,24 +821,24 @@ int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* c) {
     p.O[i] = w->O;
     p.y[i] = c->d_y[i];
     p.out[i] = c->out[i];
-    ORN_REQUIRE(c->d_y[i] || (c->gelu_pair && i == 1), "dense_rows: output %d missing", i);
+    ORN_REQUIRE(c->d_y[i] || (c->pair_act && i == 1), "dense_rows: output %d missing", i);
   }
-  ORN_REQUIRE(!c->gelu_pair || (c->n == 2 && p.O[0] == p.O[1]), "dense_rows: a gated pair is two matrices of one size");
+  ORN_REQUIRE(!c->pair_act || (c->n == 2 && p.O[0] == p.O[1]), "dense_rows: a gated pair is two matrices of one size");
   ORN_REQUIRE(c->K % 8 != 0 || (((uintptr_t)c->d_x | (uintptr_t)c->d_gate) & 15) == 0, "dense_rows: operands must be 16-byte aligned");
   const bool gemm = c->act == ORNITH_BF16 && c->M >= kPrefillRows && c->K % 8 == 0;
   if (!gemm)
-    return c->act == ORNITH_F32 ? launch_rows<float>(ctx, p, c->pre, c->gelu_pair != 0)
-                                : launch_rows<bf16_t>(ctx, p, c->pre, c->gelu_pair != 0);
+    return c->act == ORNITH_F32 ? launch_rows<float>(ctx, p, c->pre, c->pair_act != ORNITH_PAIR_NONE)
+                                : launch_rows<bf16_t>(ctx, p, c->pre, c->pair_act != ORNITH_PAIR_NONE);
   if (c->pre != ORNITH_PRE_NONE) {
     ORN_REQUIRE(c->d_rows, "dense_rows: %d rows need the buffer for the rows the matrices read", c->M);
     const int rc = c->pre == ORNITH_PRE_NORM
                        ? ornith_norm_rows(ctx, (const float*)c->d_x, c->d_norm_w, c->w_offset, c->M, c->K, c->eps, c->act, c->d_rows)
-                       : ornith_head_norm_gate(ctx, (const float*)c->d_x, c->d_norm_w, c->d_gate, c->M, c->K / c->head_dim,
-                                               c->head_dim, c->eps, c->act, c->d_rows);
+                       : ornith_head_norm_gate(ctx, (const float*)c->d_x, c->d_norm_w, c->d_gate, c->gate_act, c->M,
+                                               c->K / c->head_dim, c->head_dim, c->eps, c->act, c->d_rows);
     if (rc) return rc;
     p.x = c->d_rows;
   }
-  return launch_gemm(ctx, p, c->gelu_pair != 0);
+  return launch_gemm(ctx, p, c->pair_act != ORNITH_PAIR_NONE);
 }
 
 }  // extern "C"

@@ -11,6 +11,7 @@
 // Prefill widths (bf16): a launch that rotates queries and appends keys and values, then flash attention
 // on the matrix cores with both maps in one pass: a value fragment read from LDS serves both.
 #include "act_device.h"
+#include "mfma_device.h"
 #include "rt.h"
 
 namespace {
@@ -398,14 +399,6 @@ typedef float d_f32x4 __attribute__((ext_vector_type(4)));
 typedef uint32_t d_u32x4 __attribute__((ext_vector_type(4)));
 
 constexpr int BQ = 64, BKV = 64, LV = BKV + 8;
-
-// position of key j (0..31) of a 32-key group in a row of Vt (the lanes' order of the score tiles)
-__device__ __forceinline__ int vt_pos(int j) { return 8 * ((j & 15) >> 2) + 4 * (j >> 4) + (j & 3); }
-
-__device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
-  hi = dm_f2bf2(a, b);
-  lo = dm_f2bf2(a - dm_bf2f_lo(hi), b - dm_bf2f_hi(hi));
-}
 
 // One workgroup: 64 query rows of one head, sixteen a wavefront. Both products run transposed
 // (S^T = K Q^T, O^T += V^T P^T): a lane owns a query from the scores to the output and the weights never

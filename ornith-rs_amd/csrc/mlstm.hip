@@ -18,6 +18,7 @@
 // n_0; mlstm_out_kernel makes the outputs, all chunks at once. q, k, v are bf16 numbers; S_0, P and the
 // weighted keys go to the matrix cores as two bf16 parts each, so nothing of the recurrence is rounded to bf16.
 #include "act_device.h"
+#include "mfma_device.h"
 #include "rt.h"
 
 namespace {
@@ -238,19 +239,7 @@ __global__ __launch_bounds__(1024) void mlstm_gates_kernel(const float* gi, cons
   }
 }
 
-// bf16 high part and the rest
-__device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
-  hi = dm_f2bf2(a, b);
-  lo = dm_f2bf2(a - dm_bf2f_lo(hi), b - dm_bf2f_hi(hi));
-}
-
-// Where S_0 of a chunk lies: bf16 high parts, then low parts, each in 16 x 32 (value x key) pieces of
-// 1 KB laid out as the matrix cores read them: value row r, key channel d -> 16-byte piece
-// (r % 16) + 16 (d / 8), element d % 8.
-__device__ __forceinline__ size_t s0_at(int DP, int j, int d) {
-  return ((size_t)(j >> 4) * (DP >> 5) + (d >> 5)) * 512 + (size_t)((j & 15) + 16 * ((d & 31) >> 3)) * 8 + (d & 7);
-}
-
+// S_0 of a chunk lies in the matrix cores' order (s0_at), bf16 high parts, then low parts.
 struct ScanArgs {
   const bf16_t *k, *v;
   const float *w, *decay;
@@ -394,10 +383,6 @@ struct OutArgs {
   const float* n0;
   float* o;
 };
-
-// position of token j (0..31) of a 32-token group in a row of Vt: the order in which the lanes of the
-// transposed weight tiles hold the tokens
-__device__ __forceinline__ int vt_pos(int j) { return 8 * ((j & 15) >> 2) + 4 * (j >> 4) + (j & 3); }
 
 // One workgroup: one chunk of one head, 32 * NV value channels. Wavefront (wq, wv) makes the outputs of
 // 32 queries (two groups of sixteen) for half the channels. All products run transposed, so that a lane

@@ -3,7 +3,7 @@
 //
 // The caches mirror /root/reference/src/model/cache.rs and the rewind
 // /root/reference/src/model/qwen3_5.rs:301-349 (TrunkCapture::rewind). A design (qwen35.cpp,
-// pigodra.cpp) brings its loader, the size of its step buffers, what each of its layers keeps
+// pigodra.cpp, ranavik.cpp) brings its loader, the size of its step buffers, what each of its layers keeps
 // from token to token, and its forward.
 //
 // Cache design (differs from the reference on purpose): every cache has a fixed
@@ -62,13 +62,13 @@ DesignEntry::DesignEntry(ModelDesign* d) {
   g_designs = d;
 }
 
-int ornith_model::rope_index(int dims, double base, double factor) {
+int ornith_model::rope_index(int dims, double base, const RopeScaling& scaling) {
   for (size_t i = 0; i < ropes.size(); ++i)
-    if (ropes[i].dims == dims && ropes[i].base == base && ropes[i].factor == factor) return (int)i;
+    if (ropes[i].dims == dims && ropes[i].base == base && ropes[i].scaling == scaling) return (int)i;
   RopeTable r;
   r.dims = dims;
   r.base = base;
-  r.factor = factor;
+  r.scaling = scaling;
   ropes.push_back(r);
   return (int)ropes.size() - 1;
 }
@@ -84,7 +84,9 @@ int model_ensure_rope(ornith_model* m, int npos) {
     const size_t bytes = (size_t)npos * (r.dims / 2) * 4;
     TRY(ornith_alloc(ctx, bytes, (void**)&r.d_cos));
     TRY(ornith_alloc(ctx, bytes, (void**)&r.d_sin));
-    TRY(ornith_rope_table_scaled(ctx, npos, r.dims, r.base, r.factor, r.d_cos, r.d_sin));
+    const RopeScaling& z = r.scaling;
+    if (z.yarn) TRY(ornith_rope_table_yarn(ctx, npos, r.dims, r.base, z.factor, z.original, z.fast, z.slow, r.d_cos, r.d_sin));
+    else TRY(ornith_rope_table_scaled(ctx, npos, r.dims, r.base, z.factor, r.d_cos, r.d_sin));
   }
   m->rope_npos = npos;
   return ORNITH_OK;
@@ -145,6 +147,7 @@ int ornith_model_destroy(ornith_model* m) {
     ornith_free(m->ctx, r.d_cos);
     ornith_free(m->ctx, r.d_sin);
   }
+  for (void* p : m->owned) ornith_free(m->ctx, p);
   delete m;
   return ORNITH_OK;
 }

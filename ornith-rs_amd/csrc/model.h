@@ -114,7 +114,7 @@ static const int kMaxRows = 16;  // activation rows a forward may carry unless t
 
 // ---- layers ------------------------------------------------------------------------
 // A layer is a mixer (what looks across tokens) and a feed-forward, either of several kinds.
-enum MixerKind { MIX_GATED_DELTA, MIX_GATED_ATTN, MIX_MLSTM, MIX_DIFF_ATTN };
+enum MixerKind { MIX_GATED_DELTA, MIX_GATED_ATTN, MIX_MLSTM, MIX_DIFF_ATTN, MIX_RETENTION, MIX_LATENT_ATTN };
 enum FfKind { FF_MOE, FF_DENSE, FF_NONE };
 
 struct GdnLayer {
@@ -141,6 +141,24 @@ struct DiffAttnLayer {
   float scale, diff, lambda;
   ornith_linear q, k, v, g, o;
 };
+// retention.hip: a matrix state a head that fades by a fixed factor, rotary positions
+struct RetentionLayer {
+  int heads, dim, vdim;
+  int rope;
+  const float* d_decay;  // f32 [heads][ORNITH_DECAY_POWERS]
+  ornith_linear q, k, v, g, o;
+};
+// latent_attn.hip: keys and values made from one low-rank row a token, a sliding window, a sink in the
+// softmax, one output gate a head
+struct LatentLayer {
+  int heads, dim, rot_dim, vdim, rank;
+  int window;  // 0: none
+  int rope;
+  int kv_layer;  // the layer whose cache it reads: its own index, or an earlier one's
+  float scale;
+  ornith_linear q, down, uk, uv, g, o;
+  const void *down_norm, *sink;
+};
 struct DenseFf {
   int ff;
   ornith_linear gate, up, down;
@@ -155,8 +173,10 @@ struct CacheSpec {
   size_t state = 0;                  // recurrent state: bytes a slot
 };
 
+struct StackMixer;  // stack.h
 struct Layer {
   MixerKind mixer = MIX_GATED_ATTN;
+  const StackMixer* ops = nullptr;  // how a layer-list model runs it
   FfKind ffn = FF_MOE;
   const void *input_ln = nullptr, *post_ln = nullptr;
   CacheSpec keeps;
@@ -164,14 +184,27 @@ struct Layer {
   AttnLayer attn{};
   MlstmLayer mlstm{};
   DiffAttnLayer dattn{};
+  RetentionLayer ret{};
+  LatentLayer latent{};
   ornith_moe_weights moe{};
   DenseFf dense{};
 };
 
-// A rotation: cos / sin of position * base^(-2i/dims) / factor
+// How a rotation's frequencies are stretched: all divided by `factor`, or with YaRN's ramp between the
+// pairs that turn `fast` and `slow` times over `original` positions (ornith_rope_table_yarn).
+struct RopeScaling {
+  double factor = 1;
+  bool yarn = false;
+  double original = 0, fast = 0, slow = 0;
+  bool operator==(const RopeScaling& o) const {
+    return factor == o.factor && yarn == o.yarn && original == o.original && fast == o.fast && slow == o.slow;
+  }
+};
+// A rotation: cos / sin of position * base^(-2i/dims), stretched
 struct RopeTable {
   int dims = 0;
-  double base = 0, factor = 1;
+  double base = 0;
+  RopeScaling scaling;
   float *d_cos = nullptr, *d_sin = nullptr;  // f32 [rope_npos, dims/2]
 };
 
@@ -195,6 +228,16 @@ struct DesignEntry {
   explicit DesignEntry(ModelDesign* d);
 };
 
+// What differs between the layer-list designs around their mixers (stack.cpp).
+struct StackStyle {
+  float norm_offset = 0.f;           // norm weights are stored as their distance from this
+  const void* embed_norm = nullptr;  // a norm on the embedded rows
+  bool side_by_side = false;         // mixer and feed-forward read the same stream, each through its norm
+  float residual_mult = 1.f;         // what a layer adds is multiplied by this
+  int ff_act = ORNITH_PAIR_GELU;
+  float logit_cap = 0.f;             // logits become cap tanh(logits / cap); 0: as they are
+};
+
 struct ornith_model {
   ornith_ctx* ctx = nullptr;
   const ModelDesign* design = nullptr;
@@ -204,7 +247,9 @@ struct ornith_model {
   ornith_linear embed_tokens{};
   ornith_linear lm_head{};
   const void* final_norm = nullptr;
+  StackStyle style;
   std::vector<Layer> layers;
+  std::vector<void*> owned;  // device memory made at load
   // step buffers, sized for `max_rows` activation rows
   int max_rows = 0;
   void* ws_buf = nullptr;
@@ -216,7 +261,7 @@ struct ornith_model {
   int value_dim() const { return cfg.linear_num_value_heads * cfg.linear_value_head_dim; }
   int conv_dim() const { return 2 * key_dim() + value_dim(); }
   // the table of such a rotation, made at the next model_ensure_rope
-  int rope_index(int dims, double base, double factor);
+  int rope_index(int dims, double base, const RopeScaling& scaling = {});
 };
 
 struct LayerCache {

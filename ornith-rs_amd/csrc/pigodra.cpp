@@ -8,44 +8,11 @@
 //   "mlp"        null, or {"kind": "dense", "ff"}
 // Tensors: embed, head, final.norm; layer i: l<i>.norm1, l<i>.norm2, l<i>.mix.*, l<i>.mlp.{gate,up,down}.
 #include <cmath>
-#include <climits>
 
-#include "json.h"
 #include "stack.h"
-
-#define TRY(e)         \
-  do {                 \
-    int rc__ = (e);    \
-    if (rc__) return rc__; \
-  } while (0)
+#include "stack_config.h"
 
 namespace {
-using orn_json::JVal;
-
-int need_num(const JVal* o, const std::string& where, const char* key, double* out) {
-  const JVal* j = o ? o->get(key) : nullptr;
-  ORN_REQUIRE(j && j->kind == JVal::Num, "config.json: missing %s%s", where.c_str(), key);
-  *out = j->num;
-  return ORNITH_OK;
-}
-
-int need_f32(const JVal* o, const std::string& where, const char* key, float* out) {
-  double v = 0;
-  TRY(need_num(o, where, key, &v));
-  *out = (float)v;
-  return ORNITH_OK;
-}
-
-int need_int(const JVal* o, const std::string& where, const char* key, int min, int* out) {
-  const JVal* j = o ? o->get(key) : nullptr;
-  size_t v = 0;
-  ORN_REQUIRE(j && j->as_usize(&v), "config.json: missing %s%s", where.c_str(), key);
-  ORN_REQUIRE(v >= (size_t)min && v <= INT_MAX / 2, "config.json: %s%s is %zu", where.c_str(), key, v);
-  *out = (int)v;
-  return ORNITH_OK;
-}
-
-bool absent(const JVal* j) { return !j || j->kind == JVal::Null; }
 
 int load_mlstm(const ornith_weights* ws, const JVal* mx, const std::string& where, const std::string& p, int W, MlstmLayer* a) {
   TRY(need_int(mx, where, "heads", 1, &a->heads));
@@ -111,7 +78,7 @@ int load_attention(ornith_model* m, const ornith_weights* ws, const JVal* mx, co
     if (!absent(scaling)) TRY(need_num(scaling, where + "rot.scaling.", "factor", &factor));
     ORN_REQUIRE(dims % 2 == 0 && dims <= a->dim && base > 0 && factor > 0, "config.json: %srot turns %d of %d dimensions, base %g, factor %g",
                 where.c_str(), dims, a->dim, base, factor);
-    if (dims > 0) a->rope = m->rope_index(dims, base, factor);
+    if (dims > 0) a->rope = m->rope_index(dims, base, RopeScaling{factor});
   }
   TRY(ws_dense(ws, p + "q", a->heads * 2 * a->dim, W, &a->q));
   TRY(ws_dense(ws, p + "k", a->kv_heads * 2 * a->dim, W, &a->k));
@@ -148,25 +115,18 @@ int load_into(ornith_model* m, const ornith_weights* ws, const JVal& cfg) {
     TRY(ws_tensor(ws, p + "norm1", ORNITH_DT_BF16, W, &L.input_ln));
     if (type->str == "mlstm") {
       L.mixer = MIX_MLSTM;
+      L.ops = &kMlstmMixer;
       TRY(load_mlstm(ws, mx, where, p + "mix.", W, &L.mlstm));
     } else if (type->str == "attention") {
       L.mixer = MIX_DIFF_ATTN;
+      L.ops = &kDiffAttnMixer;
       TRY(load_attention(m, ws, mx, where, p + "mix.", W, &L.dattn));
     } else {
       return ornith_fail(ORNITH_ERR_UNSUPPORTED, "config.json: layers[%zu] is of type \"%s\"", i, type->str.c_str());
     }
-    L.ffn = FF_NONE;
-    if (absent(mlp)) continue;
-    const JVal* kind = mlp->get("kind");
-    if (!(kind && kind->kind == JVal::Str && kind->str == "dense"))
-      return ornith_fail(ORNITH_ERR_UNSUPPORTED, "config.json: layers[%zu].mlp is of a kind this design does not have", i);
-    L.ffn = FF_DENSE;
-    TRY(need_int(mlp, "layers[" + std::to_string(i) + "].mlp.", "ff", 1, &L.dense.ff));
-    TRY(ws_tensor(ws, p + "norm2", ORNITH_DT_BF16, W, &L.post_ln));
-    TRY(ws_dense(ws, p + "mlp.gate", L.dense.ff, W, &L.dense.gate));
-    TRY(ws_dense(ws, p + "mlp.up", L.dense.ff, W, &L.dense.up));
-    TRY(ws_dense(ws, p + "mlp.down", W, L.dense.ff, &L.dense.down));
+    TRY(stack_load_ff(ws, mlp, i, W, &L));
   }
+  m->style.norm_offset = 1.f;
   return stack_finish_load(m);
 }
 

@@ -260,7 +260,7 @@ int ornith_model_load(ornith_ctx* ctx, const ornith_weights* ws, const ornith_te
   m->ctx = ctx;
   m->design = &kQwen35;
   m->cfg = c;
-  m->rope_index(c.rope_dims, c.rope_theta, 1.0);
+  m->rope_index(c.rope_dims, c.rope_theta);
   const char* P = "language_model.model.";
   int rc = ORNITH_OK;
   auto fail = [&](int code) {

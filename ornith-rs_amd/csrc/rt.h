@@ -121,6 +121,7 @@ int ornith_option_moe_down_iters();  // column groups per workgroup of the exper
 int ornith_option_gdn_chunked();  // 1: the gated-delta recurrence of calls of 128 rows or more runs chunked on the matrix cores
 int ornith_option_fuse_moe_one();  // 1: the MoE block's router, up and down phases in one launch
 int ornith_option_mlstm_chunked();  // 1: the mLSTM recurrence of wide calls runs chunked on the matrix cores
+int ornith_option_retention_chunked();  // the same for the retention recurrence
 int ornith_option_ho_spins();      // polling rounds a hand-off wait inside a launch may take
 
 // weights.cpp: a k-quant matrix descriptor with usable kind, sizes and pointers

@@ -52,7 +52,8 @@ Option g_options[] = {{"fuse_moe", "ORNITH_FUSE_MOE", 1, -1},
                       {"gemm_reg", "ORNITH_GEMM_REG", 1, -1},
                       {"gdn_block_chunks", "ORNITH_GDN_BLOCK_CHUNKS", 64, -1},
                       {"fuse_attn_prep", "ORNITH_FUSE_ATTN_PREP", 1, -1},
-                      {"mlstm_chunked", "ORNITH_MLSTM_CHUNKED", 1, -1}};
+                      {"mlstm_chunked", "ORNITH_MLSTM_CHUNKED", 1, -1},
+                      {"retention_chunked", "ORNITH_RETENTION_CHUNKED", 1, -1}};
 int option_value(int i) {
   Option& o = g_options[i];
   if (o.value < 0) {
@@ -77,6 +78,7 @@ int ornith_option_gemm_reg() { return option_value(12); }
 int ornith_option_gdn_block_chunks() { return option_value(13); }
 int ornith_option_fuse_attn_prep() { return option_value(14); }
 int ornith_option_mlstm_chunked() { return option_value(15); }
+int ornith_option_retention_chunked() { return option_value(16); }
 int ornith_option_ho_spins() { return option_value(9) < 1 ? 1 : option_value(9); }
 
 int ornith_check_handoffs(ornith_ctx* ctx) {

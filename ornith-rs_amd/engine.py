@@ -674,6 +674,9 @@ def add_rms_moe_block(ctx, w, res, y, wnorm, eps, T, h_out, normed_out, out):
 # ---- dense projections around a 32-bit residual stream, mLSTM, differential attention ---------
 PRE_NONE, PRE_NORM, PRE_HEADS = range(3)
 OUT_ACT, OUT_F32, OUT_ADD = range(3)
+GATE_SIGMOID, GATE_SILU = range(2)
+PAIR_NONE, PAIR_GELU, PAIR_SILU = range(3)
+DECAY_POWERS = 65
 
 
 class DenseCall(C.Structure):
@@ -681,7 +684,8 @@ class DenseCall(C.Structure):
     _fields_ = [("act", C.c_int), ("pre", C.c_int), ("d_x", C.c_void_p), ("d_norm_w", C.c_void_p), ("d_gate", C.c_void_p),
                 ("w_offset", C.c_float), ("eps", C.c_float), ("head_dim", C.c_int), ("M", C.c_int), ("K", C.c_int),
                 ("n", C.c_int), ("w", C.POINTER(LinearStruct) * 6), ("d_y", C.c_void_p * 6), ("out", C.c_int * 6),
-                ("gelu_pair", C.c_int), ("d_rows", C.c_void_p)]
+                ("pair_act", C.c_int), ("d_rows", C.c_void_p), ("gate_act", C.c_int), ("add_scale", C.c_float),
+                ("soft_cap", C.c_float)]
 
 
 class MlstmCall(C.Structure):
@@ -700,11 +704,28 @@ class DiffAttnCall(C.Structure):
         (n, C.c_void_p) for n in ("d_k_cache", "d_v_cache", "d_q_rot", "d_out")]
 
 
+class RetentionCall(C.Structure):
+    """ornith_retention_call"""
+    _fields_ = [("act", C.c_int)] + [(n, C.c_void_p) for n in ("d_q", "d_k", "d_v", "d_cos", "d_sin")] + [
+        ("rope_dims", C.c_int), ("table_npos", C.c_int), ("offset", C.c_int), ("d_decay", C.c_void_p), ("T", C.c_int),
+        ("H", C.c_int), ("dim", C.c_int), ("vdim", C.c_int), ("d_state_in", C.c_void_p), ("d_slots", C.c_void_p),
+        ("n_slots", C.c_int), ("first_slot", C.c_int), ("snapshots", C.c_int), ("d_o", C.c_void_p)]
+
+
+class LatentAttnCall(C.Structure):
+    """ornith_latent_attn_call"""
+    _fields_ = [("act", C.c_int)] + [(n, C.c_void_p) for n in ("d_q", "d_down", "d_down_norm")] + [
+        ("uk", C.POINTER(LinearStruct)), ("uv", C.POINTER(LinearStruct))] + [
+        (n, C.c_void_p) for n in ("d_gate", "d_sink", "d_cos", "d_sin")] + [
+        (n, C.c_int) for n in ("table_npos", "T", "H", "dim", "rot_dim", "vdim", "rank", "offset", "cap", "window")] + [
+        ("scale", C.c_float), ("eps", C.c_float)] + [(n, C.c_void_p) for n in ("d_c_cache", "d_r_cache", "d_out")]
+
+
 def dense_call(act, x, M, K, lins, ys, outs, pre=PRE_NONE, norm_w=None, gate=None, w_offset=0.0, eps=1e-6, head_dim=0,
-               gelu_pair=False, rows=None):
+               pair_act=PAIR_NONE, rows=None, gate_act=GATE_SIGMOID, add_scale=1.0, soft_cap=0.0):
     c = DenseCall(act=act, pre=pre, d_x=x.ptr, d_norm_w=norm_w.ptr if norm_w else None, d_gate=gate.ptr if gate else None,
-                  w_offset=w_offset, eps=eps, head_dim=head_dim, M=M, K=K, n=len(lins), gelu_pair=int(gelu_pair),
-                  d_rows=rows.ptr if rows else None)
+                  w_offset=w_offset, eps=eps, head_dim=head_dim, M=M, K=K, n=len(lins), pair_act=pair_act,
+                  d_rows=rows.ptr if rows else None, gate_act=gate_act, add_scale=add_scale, soft_cap=soft_cap)
     for i, (l, y, o) in enumerate(zip(lins, ys, outs)):
         c.w[i], c.d_y[i], c.out[i] = C.pointer(l.s), (y.ptr if y else None), o
     return c
@@ -747,14 +768,59 @@ def diff_attn(ctx, call=None, **kw):
     _check(lib().ornith_diff_attn(ctx.h, C.byref(c)), "diff_attn")
 
 
+def retention_state_floats(H, dim, vdim):
+    f = lib().ornith_retention_state_floats
+    f.restype = C.c_size_t
+    return int(f(H, dim, vdim))
+
+
+def decay_powers(ctx, decay, out):
+    """ornith_decay_powers; out: f32 [len(decay), DECAY_POWERS]."""
+    d = np.ascontiguousarray(decay, np.float64)
+    _check(lib().ornith_decay_powers(ctx.h, len(d), _ptr(d), out.ptr), "decay_powers")
+
+
+def retention_call(**kw):
+    return _fields(RetentionCall, kw)
+
+
+def retention(ctx, call=None, **kw):
+    """ornith_retention; buffers by the call's field names without d_ (or a RetentionCall made earlier)."""
+    c = call or _fields(RetentionCall, kw)
+    _check(lib().ornith_retention(ctx.h, C.byref(c)), "retention")
+
+
+def latent_attn_call(uk, uv, **kw):
+    c = _fields(LatentAttnCall, kw)
+    c.uk, c.uv = C.pointer(uk.s), C.pointer(uv.s)
+    return c
+
+
+def latent_attn(ctx, call=None, **kw):
+    """ornith_latent_attn; buffers by the call's field names without d_, uk and uv as Linears (or a
+    LatentAttnCall made earlier)."""
+    c = call or latent_attn_call(**kw)
+    _check(lib().ornith_latent_attn(ctx.h, C.byref(c)), "latent_attn")
+
+
+def rope_table_yarn(ctx, npos, dims, theta, factor, original, fast, slow, cos, sin):
+    _check(lib().ornith_rope_table_yarn(ctx.h, npos, dims, *(C.c_double(v) for v in (theta, factor, original, fast, slow)),
+                                        cos.ptr, sin.ptr), "rope_table_yarn")
+
+
 def norm_rows(ctx, x, w, w_offset, rows, n, eps, act, out):
     _check(lib().ornith_norm_rows(ctx.h, x.ptr, w.ptr, C.c_float(w_offset), rows, n, C.c_float(eps), act, out.ptr), "norm_rows")
 
 
-def head_norm_gate(ctx, x, w, gate, rows, heads, head_dim, eps, act, out):
-    _check(lib().ornith_head_norm_gate(ctx.h, x.ptr, w.ptr, gate.ptr, rows, heads, head_dim, C.c_float(eps), act, out.ptr),
+def head_norm_gate(ctx, x, w, gate, rows, heads, head_dim, eps, act, out, gate_act=GATE_SIGMOID):
+    _check(lib().ornith_head_norm_gate(ctx.h, x.ptr, w.ptr if w else None, gate.ptr, gate_act, rows, heads, head_dim, C.c_float(eps), act, out.ptr),
            "head_norm_gate")
 
 
 def embed_rows(ctx, table, ids, n, scale, out):
     _check(lib().ornith_embed_rows(ctx.h, C.byref(table.s), ids.ptr, n, C.c_float(scale), out.ptr), "embed_rows")
+
+
+def embed_norm_rows(ctx, table, ids, n, w, w_offset, eps, out):
+    _check(lib().ornith_embed_norm_rows(ctx.h, C.byref(table.s), ids.ptr, n, w.ptr, C.c_float(w_offset), C.c_float(eps),
+                                        out.ptr), "embed_norm_rows")

@@ -18,8 +18,17 @@ def norm_zero_centred(x, w, eps):
     return rms(x, eps) * (1.0 + w)
 
 
+def norm_plain(x, w, eps):
+    """RMS norm with the weight as it is."""
+    return rms(x, eps) * w
+
+
 def sigmoid(x):
     return 1.0 / (1.0 + np.exp(-x))
+
+
+def silu(z):
+    return z * sigmoid(z)
 
 
 def gelu_tanh(z):
@@ -30,8 +39,8 @@ def exact(x):
     return x
 
 
-def dense_ff(h, gate, up, down, r=exact):
-    return r(gelu_tanh(h @ gate.T) * (h @ up.T)) @ down.T
+def dense_ff(h, gate, up, down, r=exact, act=gelu_tanh):
+    return r(act(h @ gate.T) * (h @ up.T)) @ down.T
 
 
 def soft_cap(x, cap):
@@ -131,7 +140,99 @@ def diff_attention_mixer(h, w, p, mx, eps, cache, r=exact):
     return r(out.reshape(T, H * dv)) @ w[p + "o"].T, (K, V)
 
 
-MIXERS = {"mlstm": mlstm_mixer, "attention": diff_attention_mixer}
+def turn_frequencies(dims, base, scaling=None):
+    """Angle per position of every pair, and what cos and sin are multiplied by. scaling: none, or YaRN's
+    {factor, original, fast, slow} (Peng et al., "YaRN: Efficient Context Window Extension of Large
+    Language Models"): pairs that turn often keep their frequency, slow ones get a `factor`-th of it."""
+    f = np.array([base ** (-2.0 * i / dims) for i in range(dims // 2)])
+    if not scaling:
+        return f, 1.0
+    pair_of = lambda turns: dims * math.log(scaling["original"] / (2 * math.pi * turns)) / (2 * math.log(base))
+    lo, hi = max(math.floor(pair_of(scaling["fast"])), 0), min(math.ceil(pair_of(scaling["slow"])), dims - 1)
+    slow = np.clip((np.arange(dims // 2) - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return f * (1 - slow) + f / scaling["factor"] * slow, 0.1 * math.log(scaling["factor"]) + 1.0
+
+
+def turn(x, pos, freqs, gain, halves):
+    """x [..., dim] at position pos; a pair is (2i, 2i+1), or with halves (i, i + n), n pairs in all."""
+    y, n = np.array(x, dtype=np.float64), len(freqs)
+    for i in range(n):
+        a, b = (i, i + n) if halves else (2 * i, 2 * i + 1)
+        c, s = gain * math.cos(pos * freqs[i]), gain * math.sin(pos * freqs[i])
+        u, v = x[..., a], x[..., b]
+        y[..., a] = u * c - v * s
+        y[..., b] = v * c + u * s
+    return y
+
+
+def retention_cell(q, k, v, decay, S):
+    """One head: S [dim, vdim] fades by `decay` a token, takes k v^T and is read along q."""
+    out = np.empty((len(q), v.shape[1]))
+    for t in range(len(q)):
+        S = decay * S + np.outer(k[t], v[t])
+        out[t] = S.T @ q[t]
+    return out, S
+
+
+def retention_mixer(h, w, p, mx, eps, cache, r=exact):
+    """cache: (tokens seen, one S a head) or None."""
+    H, d, dv = mx["heads"], mx["dim"], mx["vdim"]
+    T = len(h)
+    at, states = cache or (0, [np.zeros((d, dv)) for _ in range(H)])
+    q = r(h @ w[p + "q"].T).reshape(T, H, d)
+    k = r(h @ w[p + "k"].T).reshape(T, H, d)
+    v = r(h @ w[p + "v"].T).reshape(T, H, dv)
+    freqs, gain = turn_frequencies(mx["rot"]["dims"], mx["rot"]["base"], mx["rot"].get("scaling"))
+    q = np.array([turn(q[t], at + t, freqs, gain, True) for t in range(T)])
+    k = np.array([turn(k[t], at + t, freqs, gain, True) for t in range(T)]) * d ** -0.5
+    out, new = np.empty((T, H, dv)), []
+    for a in range(H):
+        out[:, a], S = retention_cell(q[:, a], k[:, a], v[:, a], mx["decay"][a], states[a])
+        new.append(S)
+    out = r(rms(out, eps).reshape(T, H * dv) * silu(r(h @ w[p + "g"].T)))
+    return out @ w[p + "o"].T, (at + T, new)
+
+
+def attend_sink(scores, values, sink):
+    """Softmax average of the values, exp(sink) in the denominator beside the scores' exponentials."""
+    top = max(float(np.max(scores)), sink)
+    e = np.exp(scores - top)
+    return (e @ values) / (e.sum() + math.exp(sink - top))
+
+
+def latent_attention_mixer(h, w, p, mx, eps, cache, r=exact, shared=None):
+    """cache, shared: (list of latents [rank], list of turned key parts [rot_dim]); `shared` is that of the layer
+    whose keys and values this one reads (its own stays None then)."""
+    H, d, dr, dv, rank = mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"], mx["kv_rank"]
+    T, size = len(h), (mx.get("mask") or {}).get("size", 0)
+    freqs, gain = turn_frequencies(dr, mx["rot"]["base"], mx["rot"].get("scaling"))
+    q = r(h @ w[p + "q"].T).reshape(T, H, d + dr)
+    if shared is None:
+        C, K = ([], []) if cache is None else (list(cache[0]), list(cache[1]))
+        at, down = len(C), h @ w[p + "dkv"].T
+        for t in range(T):
+            C.append(r(norm_plain(down[t, :rank], w[p + "dkv.norm"], eps)))
+            K.append(r(turn(down[t, rank:], at + t, freqs, gain, False)))
+        cache = (C, K)
+    else:
+        (C, K), at = shared, len(shared[0]) - T
+    gate = sigmoid(h @ w[p + "g"].T)
+    out = np.empty((T, H, dv))
+    for t in range(T):
+        i = at + t
+        js = [j for j in range(len(C)) if visible(i, j, size, 0)]
+        c, kr = np.array([C[j] for j in js]), np.array([K[j] for j in js])
+        qr = r(turn(q[t, :, d:], i, freqs, gain, False))
+        for a in range(H):
+            keys = c @ w[p + "uk"][a * d:(a + 1) * d].T
+            vals = c @ w[p + "uv"][a * dv:(a + 1) * dv].T
+            s = (keys @ q[t, a, :d] + kr @ qr[a]) * mx["scale"]
+            out[t, a] = attend_sink(s, vals, float(w[p + "sink"][a])) * gate[t, a]
+    return r(out.reshape(T, H * dv)) @ w[p + "o"].T, cache if shared is None else None
+
+
+MIXERS = {"mlstm": mlstm_mixer, "attention": diff_attention_mixer, "retention": retention_mixer,
+          "latent_attention": latent_attention_mixer}
 
 
 class Run:
@@ -144,19 +245,47 @@ class Run:
         self.cfg, self.w = cfg, {n: np.asarray(a, np.float64) for n, a in w.items()}
         self.state = [None] * len(cfg["layers"])
 
+    def mix(self, i, h):
+        layer, kw = self.cfg["layers"][i], {}
+        if layer["mixer"].get("kv_from") is not None:
+            kw["shared"] = self.state[layer["mixer"]["kv_from"]]
+        y, self.state[i] = MIXERS[layer["type"]](h, self.w, f"l{i}.mix.", layer["mixer"], self.cfg["norm"]["eps"],
+                                                 self.state[i], self.r, **kw)
+        return y
+
+    def ff(self, i, h, act):
+        p = f"l{i}.mlp."
+        return dense_ff(h, self.w[p + "gate"], self.w[p + "up"], self.w[p + "down"], self.r, act)
+
     def feed(self, tokens, trail=None):
         """trail: a list that receives the residual stream after every layer."""
+        run = {"Pigodra": self._one_after_the_other, "Ranavik": self._side_by_side}[self.cfg["architecture"]]
+        return run(self.w["embed"][np.asarray(tokens)], trail)
+
+    def _one_after_the_other(self, x, trail):
         cfg, w, eps = self.cfg, self.w, self.cfg["norm"]["eps"]
-        x = w["embed"][np.asarray(tokens)] * cfg["embedding"]["scale"]
+        x = x * cfg["embedding"]["scale"]
         for i, layer in enumerate(cfg["layers"]):
             p = f"l{i}."
-            y, self.state[i] = MIXERS[layer["type"]](self.r(norm_zero_centred(x, w[p + "norm1"], eps)), w, p + "mix.",
-                                                     layer["mixer"], eps, self.state[i], self.r)
-            x = x + y
+            x = x + self.mix(i, self.r(norm_zero_centred(x, w[p + "norm1"], eps)))
             if layer["mlp"] is not None:
-                x = x + dense_ff(self.r(norm_zero_centred(x, w[p + "norm2"], eps)), w[p + "mlp.gate"], w[p + "mlp.up"],
-                                 w[p + "mlp.down"], self.r)
+                x = x + self.ff(i, self.r(norm_zero_centred(x, w[p + "norm2"], eps)), gelu_tanh)
             if trail is not None:
                 trail.append(x)
         self.hidden = self.r(norm_zero_centred(x, w["final.norm"], eps))
         return self.hidden @ w["head"].T
+
+    def _side_by_side(self, x, trail):
+        """Mixer and feed-forward read the same stream; their sum goes back times residual_mult."""
+        cfg, w, eps = self.cfg, self.w, self.cfg["norm"]["eps"]
+        x = norm_plain(x, w["embed.norm"], eps)
+        for i, layer in enumerate(cfg["layers"]):
+            p = f"l{i}."
+            y = self.mix(i, self.r(norm_plain(x, w[p + "norm1"], eps)))
+            if layer["mlp"] is not None:
+                y = y + self.ff(i, self.r(norm_plain(x, w[p + "norm2"], eps)), silu)
+            x = x + cfg["residual_mult"] * y
+            if trail is not None:
+                trail.append(x)
+        self.hidden = self.r(norm_plain(x, w["final.norm"], eps))
+        return soft_cap(self.hidden @ w["head"].T, cfg["logit_softcap"])

@@ -79,7 +79,7 @@ def test_dense_rows(orn, ctx, act, M, K):
             y = ctx.alloc(M * 70 * 4)
             orn.dense_rows(ctx, adt, d_xa if pre == orn.PRE_NONE else d_x, M, K, [g, u], [y, None], [0, 0], pre=pre,
                     norm_w=d_wn,
-                           w_offset=1.0, eps=1e-5, gelu_pair=True, rows=d_rows)
+                           w_offset=1.0, eps=1e-5, pair_act=orn.PAIR_GELU, rows=d_rows)
             _close(_get(y, (M, 70), act), R.gelu_tanh(h @ gw.T) * (h @ uw.T), act, ("gelu pair", pre),
                     slack=6.0 if act == 0 else 1.5)
             for b in (y, g, u):
