@@ -92,10 +92,11 @@ def test_prompt_portions_and_decoding(orn, ctx, name, act):
 
 
 @pytest.mark.parametrize("act", [0, 1])
-def test_every_prefix_length_around_the_edges(orn, ctx, act):
+@pytest.mark.parametrize("name", ["even", "rv_even"])
+def test_every_prefix_length_around_the_edges(orn, ctx, name, act):
     """Last-token logits of prompts whose length passes the windows', blocks' and chunks' edges one by one,
     the shortest included; one cache for all of them."""
-    cfg = M.CONFIGS["even"]
+    cfg = M.CONFIGS[name]
     w = M.weights(cfg, 21)
     toks = np.random.default_rng(22).integers(0, cfg["vocab"], 131)
     want = Want(cfg, w, toks, act)
@@ -107,10 +108,11 @@ def test_every_prefix_length_around_the_edges(orn, ctx, act):
 
 
 @pytest.mark.parametrize("act", [0, 1])
-def test_sequences_take_turns(orn, ctx, act):
+@pytest.mark.parametrize("name", ["odd", "rv_odd", "rv_latent"])
+def test_sequences_take_turns(orn, ctx, name, act):
     """Two sequences with caches of their own, step by step in turn, then a third in a cache given back:
     each as if alone."""
-    cfg = M.CONFIGS["odd"]
+    cfg = M.CONFIGS[name]
     w = M.weights(cfg, 31)
     rng = np.random.default_rng(32)
     d = Dut(orn, ctx, cfg, w, act)
@@ -130,9 +132,10 @@ def test_sequences_take_turns(orn, ctx, act):
 
 
 @pytest.mark.parametrize("act", [0, 1])
-def test_long_decoding(orn, ctx, act):
+@pytest.mark.parametrize("name", ["even", "rv_even"])
+def test_long_decoding(orn, ctx, name, act):
     """Three hundred tokens one by one: windows slide over decoded tokens, the cache grows twice."""
-    cfg = M.CONFIGS["even"]
+    cfg = M.CONFIGS[name]
     w = M.weights(cfg, 41, gate_bias=4.0)
     toks = np.random.default_rng(42).integers(0, cfg["vocab"], 310)
     want = Want(cfg, w, toks, act)
@@ -163,7 +166,7 @@ def test_rewind(orn, ctx, name):
     d.close()
 
 
-@pytest.mark.parametrize("name", ["even", "odd", "memory"])
+@pytest.mark.parametrize("name", ["even", "odd", "memory", "rv_even", "rv_odd"])
 def test_greedy_generation(orn, ctx, name):
     """The library's generation loop in 32-bit: the reference's argmax at every step, as far as bf16 logits
     (what the samplers read) can tell it from the runner-up; and the same from short prefill chunks. In
@@ -211,11 +214,12 @@ def _write_model(tmp_path, cfg, w, orn):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_trace_replay(orn, ctx, tmp_path, monkeypatch, capsys, dtype):
+@pytest.mark.parametrize("name", ["odd", "rv_even"])
+def test_trace_replay(orn, ctx, tmp_path, monkeypatch, capsys, name, dtype):
     """bin/trace_run's program on a model read from files: portions, wanted places in any order, a request
     that ends and another that takes its cache, steps in which nothing is wanted."""
     trace = importlib.import_module("ornith-rs_amd.trace")
-    cfg = M.CONFIGS["odd"]
+    cfg = M.CONFIGS[name]
     w = M.weights(cfg, 71)
     d = _write_model(tmp_path, cfg, w, orn)
     rng = np.random.default_rng(72)
@@ -235,9 +239,9 @@ def test_trace_replay(orn, ctx, tmp_path, monkeypatch, capsys, dtype):
     assert not (out / "1.f32").exists()
 
 
-def test_config_is_checked(orn, ctx):
-    """What a config.json or a tensor must not be is an error that names it."""
-    cfg = M.CONFIGS["even"]
+def _refuses(orn, ctx, name):
+    """What a config.json or a tensor must not be is an error that names it: fails(edit of the configuration, ..)."""
+    cfg = M.CONFIGS[name]
     w = M.weights(cfg, 81)
 
     def fails(edit, drop=None, match=None, shape=None):
@@ -253,13 +257,31 @@ def test_config_is_checked(orn, ctx):
 
     fails(lambda c: c.update(architecture="Nobody"), match="Nobody")
     fails(lambda c: c["layers"][0].update(type="conv"), match="conv")
-    fails(lambda c: c["layers"][0]["mixer"].pop("diff"), match="diff")
     fails(lambda c: c["layers"][0]["mixer"]["rot"].update(dims=7), match="rot")
-    fails(lambda c: c["layers"][1]["mixer"].update(heads=5), match="mix.q")
+    fails(lambda c: c["layers"][1]["mixer"].update(heads=5), match="decay" if name == "rv_even" else "mix.q")
     fails(lambda c: c["layers"][1]["mlp"].update(kind="moe"), match="mlp")
     fails(lambda c: c.pop("norm"), match="eps")
+    return fails
+
+
+def test_config_is_checked(orn, ctx):
+    fails = _refuses(orn, ctx, "even")
+    fails(lambda c: c["layers"][0]["mixer"].pop("diff"), match="diff")
     fails(lambda c: None, drop="l2.mix.f.b", match="l2.mix.f.b")
     fails(lambda c: None, shape="l0.mix.k", match="l0.mix.k")
+
+
+def test_config_is_checked_side_by_side(orn, ctx):
+    fails = _refuses(orn, ctx, "rv_even")
+    fails(lambda c: c.pop("residual_mult"), match="residual_mult")
+    fails(lambda c: c["layers"][0]["mixer"].pop("kv_rank"), match="kv_rank")
+    fails(lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].pop("slow"), match="slow")
+    fails(lambda c: c["layers"][2]["mixer"].update(kv_from=1), match="kv_from")
+    fails(lambda c: c["layers"][2]["mixer"].update(kv_from=2), match="kv_from")
+    fails(lambda c: c["layers"][2]["mixer"]["rot"].update(base=999.0), match="rot")
+    fails(lambda c: None, drop="l0.mix.sink", match="l0.mix.sink")
+    fails(lambda c: None, drop="embed.norm", match="embed.norm")
+    fails(lambda c: None, shape="l0.mix.uk", match="l0.mix.uk")
 
 
 def test_a_draft_head_is_refused(orn, ctx):

@@ -71,3 +71,43 @@ def test_portions_do_not_matter(name):
             got.append(run.feed(toks[at:at + n]))
             at += n
         np.testing.assert_allclose(np.concatenate(got), whole, rtol=1e-9, atol=1e-9)
+
+
+def test_retention_against_the_sum_over_tokens():
+    """o_t = sum_s decay^(t-s) (q_t . k_s) v_s."""
+    rng = np.random.default_rng(5)
+    T, d, dv = 30, 6, 5
+    q, k, v = rng.standard_normal((T, d)), rng.standard_normal((T, d)), rng.standard_normal((T, dv))
+    for g in (0.0, 0.9, 1.0):
+        out, S = R.retention_cell(q, k, v, g, np.zeros((d, dv)))
+        for t in range(T):
+            w = np.array([g ** (t - s) for s in range(t + 1)]) * (k[:t + 1] @ q[t])
+            np.testing.assert_allclose(out[t], w @ v[:t + 1], rtol=1e-9, atol=1e-12)
+    np.testing.assert_allclose(S, k.T @ v, rtol=1e-9, atol=1e-12)
+
+
+def test_turned_halves_are_turned_pairs_in_another_order():
+    rng = np.random.default_rng(6)
+    x, f = rng.standard_normal(11), R.turn_frequencies(8, 300.0)[0]
+    order = [0, 4, 1, 5, 2, 6, 3, 7, 8, 9, 10]
+    np.testing.assert_allclose(R.turn(x, 9, f, 1.0, True)[order], R.turn(x[order], 9, f, 1.0, False), rtol=1e-12)
+    np.testing.assert_allclose(R.turn(x, 9, f, 1.0, False), R.rope_interleaved(x, 9, 8, 300.0, 1.0), rtol=1e-12)
+
+
+def test_yarn_keeps_fast_pairs_and_stretches_slow_ones():
+    sc = dict(factor=8.0, original=4096, fast=32.0, slow=1.0)
+    f, gain = R.turn_frequencies(64, 1e4, sc)
+    plain, one = R.turn_frequencies(64, 1e4)
+    turns = 4096 * plain / (2 * math.pi)  # over the original positions
+    assert one == 1.0 and abs(gain - (1 + 0.1 * math.log(8))) < 1e-12
+    np.testing.assert_allclose(f[turns > 45], plain[turns > 45], rtol=1e-12)
+    np.testing.assert_allclose(f[turns < 0.7], plain[turns < 0.7] / 8, rtol=1e-12)
+    assert np.all(np.diff(f / plain) <= 1e-12)
+    np.testing.assert_allclose(R.turn_frequencies(64, 1e4, dict(sc, factor=1.0))[0], plain, rtol=1e-12)
+
+
+def test_a_sink_is_a_key_without_a_value():
+    rng = np.random.default_rng(7)
+    s, v = rng.standard_normal(5), rng.standard_normal((5, 3))
+    e = np.exp(np.append(s, 0.7))
+    np.testing.assert_allclose(R.attend_sink(s, v, 0.7), (e / e.sum()) @ np.vstack([v, np.zeros(3)]), rtol=1e-12)
