@@ -649,32 +649,41 @@ def config5(args, orn, ctx, synth, np, model, ws, cfg, dev_name):
     return line
 
 
-# ---- a layer-list design beside the closest existing model (`--design Pigodra`) -------------------
+# ---- a layer-list design beside the closest existing model (`--design NAME`) -------------------
 MFMA_PEAK_TFLOPS = 2500.0
 DESIGN_SIZES = {
     # width, mLSTM (heads, dim, vdim), attention (heads, kv_heads, dim, vdim, window, kept), ff
-    2048: dict(mlstm=(8, 128, 256), attn=(16, 4, 64, 128, 2048, 64), ff=5632),
-    4096: dict(mlstm=(8, 256, 512), attn=(32, 8, 64, 128, 4096, 128), ff=11008)}
+    # latent attention (dim, rot_dim, vdim, rank) has the attention's heads and window, retention the mLSTM's sizes
+    2048: dict(mlstm=(8, 128, 256), attn=(16, 4, 64, 128, 2048, 64), latent=(128, 64, 128, 512), ff=5632),
+    4096: dict(mlstm=(8, 256, 512), attn=(32, 8, 64, 128, 4096, 128), latent=(128, 64, 128, 512), ff=11008)}
 
 
-def design_config(width, layers, vocab):
-    """`layers` layers of a Pigodra model of that width, every fourth one attention, every second one
+def design_config(name, width, layers, vocab):
+    """`layers` layers of such a model of that width, every fourth one attention, every second one
     with a feed-forward."""
     z = DESIGN_SIZES[width]
     H, d, dv = z["mlstm"]
     h, g, ad, av, win, keep = z["attn"]
-    out = []
+    ld, lr, lv, rank = z["latent"]
+    rv, out = name == "Ranavik", []
     for i in range(layers):
-        if i % 4 == 3:
+        if i % 4 == 3 and rv:
+            mx = {"heads": h, "dim": ld, "rot_dim": lr, "vdim": lv, "kv_rank": rank, "scale": (ld + lr) ** -0.5, "mask": {"size": win},
+                  "rot": {"base": 1e4, "dims": lr, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+            lay = {"type": "latent_attention", "mixer": mx}
+        elif i % 4 == 3:
             lay = {"type": "attention", "mixer": {"heads": h, "kv_heads": g, "dim": ad, "vdim": av, "diff": 0.55,
                                                   "scale": ad ** -0.5, "mask": {"size": win, "keep_first": keep},
                                                   "rot": {"base": 250000.0, "dims": ad // 2, "scaling": {"factor": 2.0}}}}
+        elif rv:
+            lay = {"type": "retention", "mixer": {"heads": H, "dim": d, "vdim": dv, "rot": {"base": 1e4, "dims": d},
+                                                  "decay": [1 - 2.0 ** (-5 - a) for a in range(H)]}}
         else:
             lay = {"type": "mlstm", "mixer": {"heads": H, "dim": d, "vdim": dv, "gate_cap": 15.0}}
         lay["mlp"] = {"kind": "dense", "ff": z["ff"]} if i % 2 else None
         out.append(lay)
-    return {"architecture": "Pigodra", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
-            "layers": out}
+    cfg = {"architecture": name, "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": out}
+    return dict(cfg, residual_mult=0.7, logit_softcap=30.0) if rv else dict(cfg, embedding={"scale": 1.0})
 
 
 def design_tensors(cfg, rng, np):
@@ -683,38 +692,49 @@ def design_tensors(cfg, rng, np):
     block = util.f32_to_bf16(rng.standard_normal(1 << 22).astype(np.float32))
     f32 = util.bf16_to_f32(block)
 
-    def mat(*shape, std=1.0):
+    def mat(*shape, std=1.0, mean=0.0):
         n = int(np.prod(shape))
         at = int(rng.integers(0, 1 << 20))
-        src = np.resize(f32[at:], n) * np.float32(std)
+        src = np.resize(f32[at:], n) * np.float32(std) + np.float32(mean)
         return util.f32_to_bf16(src).reshape(shape)
 
     W, V = cfg["width"], cfg["vocab"]
+    plain = 1.0 if cfg["architecture"] == "Ranavik" else 0.0
     yield "embed", mat(V, W)
     yield "head", mat(V, W, std=W ** -0.5)
-    yield "final.norm", mat(W, std=0.1)
+    yield "final.norm", mat(W, std=0.1, mean=plain)
+    if plain:
+        yield "embed.norm", mat(W, std=0.1, mean=plain)
     for i, lay in enumerate(cfg["layers"]):
-        p, m = f"l{i}.", lay["mixer"]
-        yield p + "norm1", mat(W, std=0.1)
-        if lay["type"] == "mlstm":
-            nk, nv = m["heads"] * m["dim"], m["heads"] * m["vdim"]
-            for n, o in (("q", nk), ("k", nk), ("v", nv), ("g", nv), ("i", m["heads"]), ("f", m["heads"])):
+        p, m, kind = f"l{i}.", lay["mixer"], lay["type"]
+        yield p + "norm1", mat(W, std=0.1, mean=plain)
+        nv = m["heads"] * m["vdim"]
+        if kind in ("mlstm", "retention"):
+            nk = m["heads"] * m["dim"]
+            for n, o in (("q", nk), ("k", nk), ("v", nv), ("g", nv)) + ((("i", m["heads"]), ("f", m["heads"])) if kind == "mlstm" else ()):
                 yield p + "mix." + n, mat(o, W, std=W ** -0.5)
-            yield p + "mix.i.b", mat(m["heads"], std=0.5)
-            yield p + "mix.f.b", util.f32_to_bf16(np.full(m["heads"], 3.0, np.float32))
-            yield p + "mix.norm", util.f32_to_bf16(np.ones(nv, np.float32))
-            yield p + "mix.o", mat(W, nv, std=0.5 * nv ** -0.5)
-        else:
-            nv = m["heads"] * m["vdim"]
+            if kind == "mlstm":
+                yield p + "mix.i.b", mat(m["heads"], std=0.5)
+                yield p + "mix.f.b", util.f32_to_bf16(np.full(m["heads"], 3.0, np.float32))
+                yield p + "mix.norm", util.f32_to_bf16(np.ones(nv, np.float32))
+        elif kind == "attention":
             for n, o in (("q", m["heads"] * 2 * m["dim"]), ("k", m["kv_heads"] * 2 * m["dim"]),
                          ("v", m["kv_heads"] * m["vdim"]), ("g", m["heads"])):
                 yield p + "mix." + n, mat(o, W, std=W ** -0.5)
             for n in ("lq1", "lk1", "lq2", "lk2"):
                 yield p + "mix." + n, mat(m["dim"], std=0.1)
-            yield p + "mix.o", mat(W, nv, std=0.5 * nv ** -0.5)
+        else:
+            r = m["kv_rank"]
+            for n, o in (("q", m["heads"] * (m["dim"] + m["rot_dim"])), ("dkv", r + m["rot_dim"]), ("g", m["heads"])):
+                yield p + "mix." + n, mat(o, W, std=W ** -0.5)
+            yield p + "mix.dkv.norm", mat(r, std=0.1, mean=1.0)
+            yield p + "mix.uk", mat(m["heads"] * m["dim"], r, std=r ** -0.5)
+            yield p + "mix.uv", mat(nv, r, std=r ** -0.5)
+            yield p + "mix.sink", mat(m["heads"], std=1.0)
+        yield p + "mix.o", mat(W, nv, std=0.5 * nv ** -0.5)
         if lay["mlp"]:
             ff = lay["mlp"]["ff"]
-            yield p + "norm2", mat(W, std=0.1)
+            yield p + "norm2", mat(W, std=0.1, mean=plain)
             yield p + "mlp.gate", mat(ff, W, std=W ** -0.5)
             yield p + "mlp.up", mat(ff, W, std=W ** -0.5)
             yield p + "mlp.down", mat(W, ff, std=0.5 * ff ** -0.5)
@@ -744,41 +764,41 @@ def design_model_rates(orn, ctx, np, model, vocab, ctx_len, n_gen, rows):
     return out
 
 
-def design_kernels(orn, ctx, np, width, only=None):
-    """Every kernel of the design at `width` beside the like kernel of the closest existing model (the
-    gated-delta / gated-attention hybrid) at the same width, both in turn on this device: microseconds
-    a launch and the fraction of its roofline (HBM bytes, or matrix-core flops where those are the longer
-    time). Weights are cycled through copies of > 512 MB in all, so no launch finds them cached."""
-    import util
-    z = DESIGN_SIZES[width]
-    rng = np.random.default_rng(7)
-    block = rng.standard_normal(1 << 20).astype(np.float32)
-    W, res, garbage = width, [], []
+class KernelTable:
+    """Kernels of a design beside the like kernels of another model, timed in turn on this device:
+    microseconds a launch and the fraction of the roofline (HBM bytes, or matrix-core flops where those are
+    the longer time). Weights are cycled through copies of > 512 MB in all, so no launch finds them cached."""
 
-    def dev(shape, dtype="bf16", std=1.0):
-        a = np.resize(block, int(np.prod(shape))) * np.float32(std)
-        b = ctx.to_device(util.f32_to_bf16(a) if dtype == "bf16" else a)
-        garbage.append(b)
+    def __init__(self, orn, ctx, np, only):
+        self.orn, self.ctx, self.np, self.only = orn, ctx, np, only
+        self.rng = np.random.default_rng(7)
+        self.block = self.rng.standard_normal(1 << 20).astype(np.float32)
+        self.res, self.garbage = [], []
+
+    def dev(self, shape, dtype="bf16", std=1.0):
+        import util
+        a = self.np.resize(self.block, int(self.np.prod(shape))) * self.np.float32(std)
+        b = self.ctx.to_device(util.f32_to_bf16(a) if dtype == "bf16" else a)
+        self.garbage.append(b)
         return b
 
-    def dense(O, K, copies):
-        out = []
-        for _ in range(copies):
-            w = orn.Linear(orn.LinearStruct(orn.LIN_DENSE, O, K, orn.KMatrixStruct(), dev((O, K), std=K ** -0.5).ptr,
-                    None, None), [])
-            out.append(w)
+    def dense(self, O, K, copies):
+        orn = self.orn
+        return [orn.Linear(orn.LinearStruct(orn.LIN_DENSE, O, K, orn.KMatrixStruct(), self.dev((O, K), std=K ** -0.5).ptr, None,
+                                            None), []) for _ in range(copies)]
+
+    def kq(self, kind, O, K, copies):
+        import util
+        km = util.HostLinear.kq(self.rng, kind, O, K)
+        out = [km.dev(self.orn, self.ctx) for _ in range(copies)]
+        self.garbage.extend(out)
         return out
 
-    def kq(kind, O, K, copies):
-        km = util.HostLinear.kq(rng, kind, O, K)
-        out = [km.dev(orn, ctx) for _ in range(copies)]
-        garbage.extend(out)
-        return out
-
+    @staticmethod
     def copies_for(nbytes):
         return max(2, min(24, int(-(-(600 << 20) // nbytes))))
 
-    def row(name, us, nbytes, flops=0.0, peer=False, note=""):
+    def row(self, name, us, nbytes, flops=0.0, peer=False, note=""):
         t_hbm, t_mm = nbytes / (HBM_PEAK_GBS * 1e3), flops / (MFMA_PEAK_TFLOPS * 1e6)
         r = {"kernel": name, "us": round(us, 2), "GB_s": round(nbytes / us / 1e3, 1), "roofline_frac": round(max(t_hbm,
                 t_mm) / us, 4)}
@@ -790,18 +810,35 @@ def design_kernels(orn, ctx, np, width, only=None):
         log(("    like: " if peer else "  ") + json.dumps(r))
         return r
 
-    def pair(name, mine, peer, peer_name):
-        res.append({"what": name, "design": mine, "closest": dict(peer, kernel=peer_name) if peer else None,
-                    "times_as_far": round(peer["roofline_frac"] / mine["roofline_frac"], 2) if peer else None})
+    def pair(self, name, mine, peer, peer_name):
+        self.res.append({"what": name, "design": mine, "closest": dict(peer, kernel=peer_name) if peer else None,
+                         "times_as_far": round(peer["roofline_frac"] / mine["roofline_frac"], 2) if peer else None})
 
-    def want(name):
-        return only is None or any(o in name for o in only)
+    def want(self, name):
+        return self.only is None or any(o in name for o in self.only)
 
-    def calls(fn, made):
+    def calls(self, fn, made):
         """fn(ctx, call) over call structures made beforehand (the host must not be what is timed)"""
-        return lambda i: fn(ctx, made[i % len(made)])
+        return lambda i: fn(self.ctx, made[i % len(made)])
 
-    t_of = lambda fn, n=200, warm=20: _time_loop(ctx, fn, n, warm)
+    def t_of(self, fn, n=200, warm=20):
+        return _time_loop(self.ctx, fn, n, warm)
+
+    def done(self):
+        for b in self.garbage:
+            b.free()
+        return self.res
+
+
+def design_kernels(orn, ctx, np, width, only=None):
+    """Every kernel of Pigodra at `width` beside the like kernel of the closest model that was there before
+    it (the gated-delta / gated-attention hybrid) at the same width."""
+    import util
+    z, W = DESIGN_SIZES[width], width
+    kt = KernelTable(orn, ctx, np, only)
+    rng, block = kt.rng, kt.block
+    dev, dense, kq, copies_for, row, pair, want, calls, t_of = (kt.dev, kt.dense, kt.kq, kt.copies_for, kt.row, kt.pair, kt.want,
+                                                                kt.calls, kt.t_of)
     H, d, dv = z["mlstm"]
     nk, nv = H * d, H * dv
     h, g, ad, av, win, keep = z["attn"]
@@ -998,33 +1035,196 @@ def design_kernels(orn, ctx, np, width, only=None):
             pair(f"prefill attention, T = {T}", mine, row("x", us, T * (Hq * 512 + 2 * Hkv * 256 + Hq * 256) * 2,
                     2.0 * full * Hq * 512, peer=True),
                  "attn_decode at prefill width (prep + attention)")
-    for b in garbage:
-        b.free()
-    return res
+    return kt.done()
+
+
+def ranavik_kernels(orn, ctx, np, width, only=None):
+    """Every kernel of Ranavik at `width` beside the like kernel of Pigodra at the same width: retention beside
+    the mLSTM at equal heads, latent attention beside differential attention at equal heads, value width and
+    window."""
+    z, W = DESIGN_SIZES[width], width
+    kt = KernelTable(orn, ctx, np, only)
+    dev, dense, copies_for, row, pair, want, calls, t_of = (kt.dev, kt.dense, kt.copies_for, kt.row, kt.pair, kt.want, kt.calls,
+                                                            kt.t_of)
+    H, d, dv = z["mlstm"]
+    nk, nv = H * d, H * dv
+    h, g, ad, av, win, keep = z["attn"]
+    ld, lr, lv, rank = z["latent"]
+    ff = z["ff"]
+    B, ACT, F32, ADD = orn.BF16, orn.OUT_ACT, orn.OUT_F32, orn.OUT_ADD
+
+    def projections(what, T, mine_shapes, peer_shapes, mine_outs, peer_outs, pre):
+        """A mixer's input projections of both designs, with the norm in front at decode widths."""
+        made, reps = [], {} if T < 32 else dict(n=20, warm=3)
+        for shapes, outs in ((mine_shapes, mine_outs), (peer_shapes, peer_outs)):
+            nb = sum(shapes) * W * 2
+            n = copies_for(nb) if T < 32 else 1
+            ws = [dense(o, W, n) for o in shapes]
+            x, wn = dev((T, W), "f32" if pre else "bf16"), dev((W,), std=0.1)
+            ys = [ctx.alloc(T * o * 4) for o in shapes]
+            us = t_of(calls(orn.dense_rows, [orn.dense_call(B, x, T, W, [w[i % n] for w in ws], ys, outs,
+                                                           pre=orn.PRE_NORM if pre else orn.PRE_NONE, norm_w=wn) for i in range(n)]), **reps)
+            made.append(row("x", us, nb + T * W * 4 + T * sum(shapes) * 2, 2.0 * T * W * sum(shapes) if T >= 32 else 0.0,
+                            peer=bool(made)))
+            for b in ys:
+                b.free()
+        pair(f"{what}, T = {T}", made[0], made[1], "the same into its like")
+
+    ret_in, mem_in = [nk, nk, nv, nv], [nk, nk, nv, nv, H, H]
+    lat_in, dif_in = [h * (ld + lr), h, rank + lr], [h * 2 * ad, g * 2 * ad, g * av, h]
+    for T in (1, 4, 512, 4096):
+        if want("decode projections" if T < 32 else "prefill GEMM"):
+            kind = "decode projections" if T < 32 else "prefill GEMM"
+            projections(f"{kind} into retention", T, ret_in, mem_in, [ACT] * 4, [ACT] * 4 + [F32] * 2, T < 32)
+            projections(f"{kind} into latent attention", T, lat_in, dif_in, [ACT, F32, F32], [ACT] * 3 + [F32], T < 32)
+    for T in (1, 4):
+        if want("decode projections"):
+            n = copies_for(W * nv * 2)
+            wo = dense(W, nv, n)
+            o, gate, wn2, xs = dev((T, nv), "f32"), dev((T, nv)), dev((nv,)), dev((T, W), "f32")
+            us = [t_of(calls(orn.dense_rows, [orn.dense_call(B, o, T, nv, [wo[i % n]], [xs], [ADD], pre=orn.PRE_HEADS, norm_w=w,
+                                                            gate=gate, head_dim=dv, gate_act=act, add_scale=m) for i in range(n)]))
+                  for w, act, m in ((None, orn.GATE_SILU, 0.7), (wn2, orn.GATE_SIGMOID, 1.0))]
+            nb = W * nv * 2 + T * nv * 6
+            pair(f"decode projection out, T = {T}", row("head norm, silu gate + output projection + sum", us[0], nb),
+                 row("x", us[1], nb, peer=True), "head norm, gate + output projection + sum")
+            n = copies_for(2 * ff * W * 2)
+            wg, wu, wd = dense(ff, W, n), dense(ff, W, n), dense(W, ff, n)
+            x, wn, act = dev((T, W), "f32"), dev((W,), std=0.1), ctx.alloc(T * ff * 2)
+            us = [t_of(calls(orn.dense_rows, [orn.dense_call(B, x, T, W, [wg[i % n], wu[i % n]], [act, None], [0, 0], pre=orn.PRE_NORM,
+                                                            norm_w=wn, pair_act=a) for i in range(n)]))
+                  for a in (orn.PAIR_SILU, orn.PAIR_GELU)]
+            pair(f"decode gate, up, T = {T}", row("norm + gate, up + silu", us[0], 2 * ff * W * 2),
+                 row("x", us[1], 2 * ff * W * 2, peer=True), "norm + gate, up + gelu")
+            us = [t_of(calls(orn.dense_rows, [orn.dense_call(B, act, T, ff, [wd[i % n]], [xs], [ADD], add_scale=m) for i in range(n)]))
+                  for m in (0.7, 1.0)]
+            pair(f"decode down, T = {T}", row("down + sum", us[0], ff * W * 2), row("x", us[1], ff * W * 2, peer=True), "down + sum")
+        if want("decode recurrence"):
+            layers = 24
+            co, si = ctx.rope_table(64, d, 1e4)
+            pw = ctx.alloc(H * orn.DECAY_POWERS * 4)
+            orn.decay_powers(ctx, [1 - 2.0 ** (-5 - i % 8) for i in range(H)], pw)
+            q, k, v, gi, gf, b1 = dev((T, nk)), dev((T, nk)), dev((T, nv)), dev((T, H), "f32"), dev((T, H), "f32"), dev((H,))
+            o = ctx.alloc(T * nv * 4)
+            sf = orn.retention_state_floats(H, d, dv)
+            slots = [dev((T + 2, sf), "f32", 0.01) for _ in range(layers)]
+            at = lambda i, sf: dict(state_in=slots[i % layers].ptr.value + ((i // layers) % 2) * sf * 4, slots=slots[i % layers],
+                                    n_slots=T + 2, first_slot=1 - (i // layers) % 2, snapshots=0, o=o)
+            us = t_of(calls(orn.retention, [orn.retention_call(act=B, q=q, k=k, v=v, cos=co, sin=si, rope_dims=d, table_npos=64, offset=9,
+                                                              decay=pw, T=T, H=H, dim=d, vdim=dv, **at(i, sf)) for i in range(2 * layers)]))
+            mine = row("retention step", us, 2 * sf * 4 + T * (2 * nk + nv) * 2 + T * nv * 4)
+            sm = orn.mlstm_state_floats(H, d, dv)
+            slots = [dev((T + 2, sm), "f32", 0.01) for _ in range(layers)]
+            us = t_of(calls(orn.mlstm, [orn.mlstm_call(act=B, q=q, k=k, v=v, gi=gi, gf=gf, bi=b1, bf=b1, gate_cap=15.0, T=T, H=H, dim=d,
+                                                      vdim=dv, **at(i, sm)) for i in range(2 * layers)]))
+            pair(f"decode recurrence, T = {T}", mine, row("x", us, 2 * sm * 4 + T * (2 * nk + nv) * 2 + T * nv * 4, peer=True), "mLSTM step")
+
+    def attention(T, ctx_len, off, caps, reps):
+        """Latent attention (append, maps, sink and gate included) beside differential attention."""
+        co, si = ctx.rope_table(ctx_len, lr, 1e4)
+        cc, rc = [dev((ctx_len, rank)) for _ in range(caps)], [dev((ctx_len, lr)) for _ in range(caps)]
+        uk, uv = dense(h * ld, rank, caps), dense(h * lv, rank, caps)
+        q, down, nw, gt, sink = dev((T, h * (ld + lr))), dev((T, rank + lr), "f32"), dev((rank,)), dev((T, h), "f32"), dev((h,))
+        out = ctx.alloc(T * h * max(lv, av) * 2)
+        us = t_of(calls(orn.latent_attn, [orn.latent_attn_call(
+            uk[i], uv[i], act=B, q=q, down=down, down_norm=nw, gate=gt, sink=sink, cos=co, sin=si, table_npos=ctx_len, T=T, H=h, dim=ld,
+            rot_dim=lr, vdim=lv, rank=rank, offset=off, cap=ctx_len, window=win, scale=(ld + lr) ** -0.5, eps=1e-6, c_cache=cc[i],
+            r_cache=rc[i], out=out) for i in range(caps)]), **reps)
+        i_ = np.arange(off, off + T)
+        seen = float(np.sum(np.minimum(i_ + 1, win)))
+        maps = h * (ld + lv) * rank
+        wide = T >= 32
+        mine = row("latent attention", us, maps * 2 + min(ctx_len, win + T) * (rank + lr) * 2 + T * (h * (ld + lr + lv) * 2 + (rank + lr) * 4),
+                   2.0 * T * maps + 2.0 * seen * h * (ld + lr + lv) if wide else 0.0)
+        kc, vc = [dev((g, ctx_len, 2 * ad)) for _ in range(caps)], [dev((g, ctx_len, av)) for _ in range(caps)]
+        q, k, v = dev((T, h * 2 * ad)), dev((T, g * 2 * ad)), dev((T, g * av))
+        co, si = ctx.rope_table(ctx_len, ad // 2, 250000.0)
+        qr = ctx.alloc(T * h * 2 * ad * 2)
+        us = t_of(calls(orn.diff_attn, [orn.diff_attn_call(
+            act=B, q=q, k=k, v=v, gate=gt, cos=co, sin=si, rope_dims=ad // 2, table_npos=ctx_len, T=T, H=h, G=g, dim=ad, vdim=av,
+            offset=off, cap=ctx_len, window=win, keep_first=0, scale=ad ** -0.5, lam=0.5, diff=0.55, eps=1e-6, k_cache=kc[i],
+            v_cache=vc[i], q_rot=qr, out=out) for i in range(caps)]), **reps)
+        peer = row("x", us, g * min(ctx_len, win + T) * (2 * ad + av) * 2 + T * (h * 2 * ad + h * av) * 2,
+                   2.0 * seen * h * 2 * (ad + av) if wide else 0.0, peer=True)
+        pair(f"{'prefill' if wide else 'decode'} attention, {min(ctx_len, win)} keys, T = {T}", mine, peer, "differential attention")
+
+    for T in (1, 4):
+        if want("decode attention"):
+            for n in (256, win + T):
+                attention(T, n, n - T, 24, {})
+    # ---- prefill
+    for T in (512, 4096):
+        reps = dict(n=20, warm=3)
+        if want("prefill GEMM"):
+            wg, wu = dense(ff, W, 1)[0], dense(ff, W, 1)[0]
+            x, act = dev((T, W)), ctx.alloc(T * ff * 2)
+            us = [t_of(calls(orn.dense_rows, [orn.dense_call(B, x, T, W, [wg, wu], [act, None], [0, 0], pair_act=a)]), **reps)
+                  for a in (orn.PAIR_SILU, orn.PAIR_GELU)]
+            size = (2 * ff * W * 2 + T * (W + ff) * 2, 4.0 * T * W * ff)
+            pair(f"prefill GEMM gate, up, T = {T}", row("gate, up + silu", us[0], *size), row("x", us[1], *size, peer=True), "gate, up + gelu")
+        if want("prefill rows"):
+            o, gate, wn2, out = dev((T, nv), "f32"), dev((T, nv)), dev((nv,)), ctx.alloc(T * max(W, nv) * 4)
+            us = [t_of(lambda i: orn.head_norm_gate(ctx, o, w, gate, T, H, dv, 1e-6, B, out, gate_act=a), **reps)
+                  for w, a in ((None, orn.GATE_SILU), (wn2, orn.GATE_SIGMOID))]
+            pair(f"prefill rows: head norm, T = {T}", row("head norm, silu gate", us[0], T * nv * 8),
+                 row("x", us[1], T * nv * 8, peer=True), "head norm, gate")
+            table, wn = dense(32768, W, 1)[0], dev((W,))
+            ids = ctx.to_device(kt.rng.integers(0, 32768, T).astype(np.uint32))
+            us = [t_of(lambda i: orn.embed_norm_rows(ctx, table, ids, T, wn, 0.0, 1e-6, out), **reps),
+                  t_of(lambda i: orn.embed_rows(ctx, table, ids, T, 1.0, out), **reps)]
+            pair(f"prefill rows: embedding, T = {T}", row("embedding + norm", us[0], T * W * 6), row("x", us[1], T * W * 6, peer=True),
+                 "embedding")
+        if want("prefill recurrence"):
+            co, si = ctx.rope_table(T, d, 1e4)
+            pw = ctx.alloc(H * orn.DECAY_POWERS * 4)
+            orn.decay_powers(ctx, [1 - 2.0 ** (-5 - i % 8) for i in range(H)], pw)
+            q, k, v, gi, gf, b1 = dev((T, nk)), dev((T, nk)), dev((T, nv)), dev((T, H), "f32"), dev((T, H), "f32"), dev((H,))
+            o = ctx.alloc(T * nv * 4)
+            sf, sm = orn.retention_state_floats(H, d, dv), orn.mlstm_state_floats(H, d, dv)
+            slots = dev((2, sm), "f32", 0.01)
+            at = lambda i, n: dict(state_in=slots.ptr.value + (i % 2) * n * 4, slots=slots, n_slots=2, first_slot=1 - i % 2, snapshots=0, o=o)
+            size = (T * (2 * nk + nv) * 2 + T * nv * 4 + 2 * sf * 4, 2.0 * T * H * (2 * d * dv + 32 * (d + dv)))
+            us = t_of(calls(orn.retention, [orn.retention_call(act=B, q=q, k=k, v=v, cos=co, sin=si, rope_dims=d, table_npos=T, offset=0,
+                                                              decay=pw, T=T, H=H, dim=d, vdim=dv, **at(i, sf)) for i in range(2)]), **reps)
+            mine = row("retention in chunks (rotation included)", us, *size)
+            us = t_of(calls(orn.mlstm, [orn.mlstm_call(act=B, q=q, k=k, v=v, gi=gi, gf=gf, bi=b1, bf=b1, gate_cap=15.0, T=T, H=H, dim=d,
+                                                      vdim=dv, **at(i, sm)) for i in range(2)]), **reps)
+            pair(f"prefill recurrence, T = {T}", mine, row("x", us, *size, peer=True), "mLSTM in chunks")
+        if want("prefill attention"):
+            attention(T, T, 0, 1, reps)
+    return kt.done()
 
 
 def design_bench(args, orn, ctx, synth, np, dev_name):
-    """`--design Pigodra`: prefill and decode rates of the design at layer sizes of real models (random
-    weights) beside the closest existing model at equal width and depth, and kernel by kernel."""
+    """`--design NAME`: prefill and decode rates of the design at layer sizes of real models (random
+    weights) beside the closest other model at equal width and depth, and kernel by kernel."""
     out = {"design": args.design, "device": dev_name, "data": "synthetic", "models": [], "kernels": []}
     layers, vocab = 8, 32768
     only = args.design_kernels.split(",") if args.design_kernels else None
-    for width in (int(w) for w in args.design_widths.split(",")):
-        log(f"width {width}: kernels")
-        out["kernels"].append({"width": width, "rows": design_kernels(orn, ctx, np, width, only)})
-        if args.design_no_models:
-            continue
-        cfg = design_config(width, layers, vocab)
+    kernels = {"Pigodra": design_kernels, "Ranavik": ranavik_kernels}[args.design]
+
+    def rates(name, width):
+        cfg = design_config(name, width, layers, vocab)
         ws = orn.WeightStore(ctx)
         for n, a in design_tensors(cfg, np.random.default_rng(3), np):
             ws.put(n, a, orn.DT_BF16)
         model = orn.TextModel.from_json(ctx, ws, cfg)
-        e = {"width": width, "layers": layers, "weight_bytes": ws.stats()[1],
-             "design": [design_model_rates(orn, ctx, np, model, vocab, n, 128, 4096) for n in (128, 4096)]}
+        r = [design_model_rates(orn, ctx, np, model, vocab, n, 128, 4096) for n in (128, 4096)], ws.stats()[1]
         model.close()
         ws.close()
+        return r
+
+    for width in (int(w) for w in args.design_widths.split(",")):
+        log(f"width {width}: kernels")
+        out["kernels"].append({"width": width, "rows": kernels(orn, ctx, np, width, only)})
+        if args.design_no_models:
+            continue
+        e = {"width": width, "layers": layers}
+        e["design"], e["weight_bytes"] = rates(args.design, width)
+        if args.design == "Ranavik":
+            e["closest"], e["closest_weight_bytes"] = rates("Pigodra", width)
         # the hybrid's stepwise kernels are made for hidden size 2048: its width there
-        if width == 2048:
+        elif width == 2048:
             qc = dict(synth.FULL, num_hidden_layers=layers, vocab_size=vocab, num_experts=64)
             sm = synth.SynthModel(qc, seed=9, with_mtp=False, with_oracle=False)
             ws = sm.upload(orn, ctx, drop_host=True)
@@ -1078,7 +1278,7 @@ def main():
                     help="only the phase time stamps of the expert pair (needs the library built with -DORN_TIMING)")
     ap.add_argument("--warm-cold", action="store_true",
                     help="only the mat-vec timings on re-used, unread and just-read weights")
-    ap.add_argument("--design", choices=("Pigodra",), default=None,
+    ap.add_argument("--design", choices=("Pigodra", "Ranavik"), default=None,
                     help="instead of the metric's workload: prefill and decode rates of that design at layer sizes of real "
                          "models (random weights) beside the closest existing model, and every kernel of both")
     ap.add_argument("--design-widths", default="2048,4096", help="with --design: model widths, commas between them")
