@@ -4,9 +4,12 @@
 //
 // Decode widths (and 32-bit models): the key map goes into the query and the value map onto the result, so a
 // cached row is read once for all heads and never expanded. Three launches: latent_query_kernel makes the
-// queries uk^T q beside their turned part, and appends the call's rows to the cache; latent_decode_kernel takes
-// one block of a query's visible rows for a group of heads; latent_out_kernel joins a head's blocks, maps the
-// result through uv and gates it. Everything between the bf16 operands is fp32.
+// queries uk^T q beside their turned part, and appends the call's rows to the cache; a decode kernel takes one
+// block of a query's visible rows for a group of heads; latent_out_kernel joins a head's blocks, maps the
+// result through uv and gates it. Everything between the bf16 operands is fp32. For bf16 rows of up to 576
+// values the blocks run on the matrix cores (latent_mfma_kernel: heads are one side of both products; queries
+// and softmax weights go in as two bf16 parts), others on the vector units (latent_decode_kernel). Blocks are
+// counted along a query's own visible rows, so a row does not depend on what else is in the call.
 //
 // Prefill widths (bf16): the rows are appended, one GEMM makes keys and values of the rows in sight, and flash
 // attention runs on the matrix cores, its keys the expanded part and the shared turned part side by side.
@@ -30,6 +33,15 @@ struct LaArgs {
 };
 
 __device__ __forceinline__ int first_visible(const LaArgs& p, int pos) { return p.window > 0 ? max(0, pos - p.window + 1) : 0; }
+// rows of a query's blocks: `unit`, or, where a workgroup can go on (a negative unit), twice as many until
+// there are at most kMaxBlocks of them
+constexpr int kMaxBlocks = 64;
+__device__ __forceinline__ int block_rows(int nvis, int unit) {
+  if (unit > 0) return unit;
+  int kb = -unit;
+  while (nvis > kMaxBlocks * kb) kb *= 2;
+  return kb;
+}
 __device__ __forceinline__ float gate_at(const LaArgs& p, int t, int h) {
   return p.gate ? dm_sigmoid_f32(p.gate[(size_t)t * p.H + h]) : 1.0f;
 }
@@ -83,9 +95,24 @@ __device__ __forceinline__ void append_row(const LaArgs& p, int t, float* red) {
 // ---- decode widths ---------------------------------------------------------------------
 constexpr int QC = 128, DG = NT / 16;  // latent columns of a query workgroup; its groups of head dimensions
 
-// grid (column tiles, H + 1, row groups). qs: f32 [T][H][rank + rot], scaled. The last grid row appends.
+// Queries over the cached rows, [T][H][rank + rot], scaled: fp32 or as two bf16 parts.
+struct MappedQ {
+  float* f;
+  bf16_t *hi, *lo;
+  __device__ __forceinline__ void put(size_t at, float v) const {
+    if (f) {
+      f[at] = v;
+    } else {
+      const bf16_t h = dm_f2bf(v);
+      hi[at] = h;
+      lo[at] = dm_f2bf(v - dm_bf2f(h));
+    }
+  }
+};
+
+// grid (column tiles, H + 1, row groups). The last grid row appends.
 template <typename A, int MR, bool VEC>
-__global__ __launch_bounds__(NT) void latent_query_kernel(LaArgs p, float* qs) {
+__global__ __launch_bounds__(NT) void latent_query_kernel(LaArgs p, MappedQ qs) {
   extern __shared__ __attribute__((aligned(16))) char lds_raw[];
   float* red = reinterpret_cast<float*>(lds_raw);  // [DG][MR][QC]
   float* xq = red + DG * MR * QC;                  // [MR][dim]
@@ -123,9 +150,9 @@ __global__ __launch_bounds__(NT) void latent_query_kernel(LaArgs p, float* qs) {
       const A* s = q + ((size_t)(m0 + m) * p.H + h) * qd + p.dim + 2 * e;
       float u = act_f(s[0]), v = act_f(s[1]);
       turn_pair(p, p.offset + m0 + m, e, u, v);
-      float* d = qs + ((size_t)(m0 + m) * p.H + h) * QS + p.rank + 2 * e;
-      d[0] = u * p.scale;
-      d[1] = v * p.scale;
+      const size_t at = ((size_t)(m0 + m) * p.H + h) * QS + p.rank + 2 * e;
+      qs.put(at, u * p.scale);
+      qs.put(at + 1, v * p.scale);
     }
   __syncthreads();
   float acc[MR][8];
@@ -161,7 +188,7 @@ __global__ __launch_bounds__(NT) void latent_query_kernel(LaArgs p, float* qs) {
     float a = 0.f;
 #pragma unroll
     for (int g = 0; g < DG; ++g) a += red[(g * MR + m) * QC + c];
-    qs[((size_t)(m0 + m) * p.H + h) * QS + r] = a * p.scale;
+    qs.put(((size_t)(m0 + m) * p.H + h) * QS + r, a * p.scale);
   }
 }
 
@@ -278,17 +305,19 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(LaArgs p, const float
   }
 }
 
-// grid (value tiles, H, rows): the blocks of a query joined, in ascending order with weights e^(m_b - M), then
-// VB values of the head, a wavefront VB / 4 of them.
+// grid (value tiles, H, rows): the blocks of a query joined with weights e^(m_b - M), groups of threads taking
+// every G-th block, then VB values of the head, a wavefront VB / 4 of them.
 constexpr int VB = 32;
 template <typename A, bool VEC>
-__global__ __launch_bounds__(NT) void latent_out_kernel(LaArgs p, int KB, int t_base, int stride, const float* part, const float* ml) {
+__global__ __launch_bounds__(NT) void latent_out_kernel(LaArgs p, int unit, int t_base, int stride, const float* part, const float* ml) {
   extern __shared__ __attribute__((aligned(16))) char lds_raw[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int h = blockIdx.y, t = t_base + blockIdx.z, pos = p.offset + t;
-  const int nb = (pos - first_visible(p, pos) + 1 + KB - 1) / KB;
+  const int nvis = pos - first_visible(p, pos) + 1, KB = block_rows(nvis, unit), nb = (nvis + KB - 1) / KB;
+  const int rp = (p.rank + 7) & ~7;
   float* ol = reinterpret_cast<float*>(lds_raw);  // [rank rounded up to 8]
-  float* wb = ol + ((p.rank + 7) & ~7);           // [stride]
+  float* wb = ol + rp;                            // [stride rounded up to 4]
+  float* red = wb + ((stride + 3) & ~3);          // [G][rank]
   const size_t base = ((size_t)blockIdx.z * p.H + h) * stride;
   // this wavefront's weights, asked for ahead
   constexpr int VR = VB / 4;
@@ -300,9 +329,23 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(LaArgs p, int KB, int t_
     for (int r = 0; r < VR; ++r)
       if (v0 + r < p.vdim && 8 * lane < p.rank) first[r] = *reinterpret_cast<const uint4*>(w + (size_t)r * p.rank + 8 * lane);
   }
+  // four columns a thread, and the first blocks of its group, asked for before the weights are made
+  constexpr int W = VEC ? 4 : 1, U = 8;
+  const int cols = p.rank / W, G = max(1, NT / cols), g = tid / cols, c0 = tid % cols;
+  const float* src = part + base * p.rank;
+  float x[U][W];
+  auto fetch = [&](int b0, int c) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int b = min(b0 + G * u, nb - 1);
+      if constexpr (VEC) act_load<4>(src + (size_t)b * p.rank + 4 * c, x[u]);
+      else x[u][0] = src[(size_t)b * p.rank + c];
+    }
+  };
+  if (g < G) fetch(g, c0);
   if (wave == 0) {
-    const float* mr = ml + base * 2;
     const float sink = p.sink ? dm_bf2f(p.sink[h]) : -DM_INF;
+    const float* mr = ml + base * 2;
     float M = sink;
     for (int b = lane; b < nb; b += 64) M = __builtin_fmaxf(M, mr[2 * b]);
     M = dm_wave_max<64>(M);
@@ -317,49 +360,234 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(LaArgs p, int KB, int t_
     for (int b = lane; b < nb; b += 64) wb[b] = wb[b] / L;
   }
   __syncthreads();
-  const float* src = part + base * p.rank;
-  for (int c = tid; c < ((p.rank + 7) & ~7); c += NT) {
-    float o = 0.f;
-    if (c < p.rank) {
-      int b = 0;
-      for (; b + 16 <= nb; b += 16) {
-        float x[16];
+  for (int c = c0; c < cols; c += NT) {  // (one round unless a row is longer than the workgroup)
+    if (g < G) {
+      float o[W];
 #pragma unroll
-        for (int e = 0; e < 16; ++e) x[e] = src[(size_t)(b + e) * p.rank + c];
+      for (int e = 0; e < W; ++e) o[e] = 0.f;
+      if (c != c0) fetch(g, c);
+      for (int b0 = g; b0 < nb; b0 += G * U) {
 #pragma unroll
-        for (int e = 0; e < 16; ++e) o = dm_fma(wb[b + e], x[e], o);
+        for (int u = 0; u < U; ++u) {
+          const float wt = b0 + G * u < nb ? wb[b0 + G * u] : 0.f;
+#pragma unroll
+          for (int e = 0; e < W; ++e) o[e] = b0 + G * u < nb ? dm_fma(wt, x[u][e], o[e]) : o[e];
+        }
+        if (b0 + G * U < nb) fetch(b0 + G * U, c);
       }
-      for (; b < nb; ++b) o = dm_fma(wb[b], src[(size_t)b * p.rank + c], o);
+#pragma unroll
+      for (int e = 0; e < W; ++e) red[g * p.rank + W * c + e] = o[e];
     }
+  }
+  __syncthreads();
+  for (int c = tid; c < rp; c += NT) {
+    float o = 0.f;
+    if (c < p.rank)
+      for (int i = 0; i < G; ++i) o += red[i * p.rank + c];
     ol[c] = o;
   }
   __syncthreads();
   const float gt = gate_at(p, t, h);
   A* dst = reinterpret_cast<A*>(p.out) + ((size_t)t * p.H + h) * p.vdim;
+  float a[VR];
 #pragma unroll
-  for (int r = 0; r < VR; ++r) {
-    if (v0 + r >= p.vdim) break;
-    float a = 0.f;
-    if constexpr (VEC) {
-      for (int c = 8 * lane; c < p.rank; c += 512) {
-        const uint4 x = c == 8 * lane ? first[r] : *reinterpret_cast<const uint4*>(w + (size_t)r * p.rank + c);
-        const float wv[8] = {dm_bf2f_lo(x.x), dm_bf2f_hi(x.x), dm_bf2f_lo(x.y), dm_bf2f_hi(x.y),
-                             dm_bf2f_lo(x.z), dm_bf2f_hi(x.z), dm_bf2f_lo(x.w), dm_bf2f_hi(x.w)};
-        float ov[8];
-        act_load<8>(ol + c, ov);
+  for (int r = 0; r < VR; ++r) a[r] = 0.f;
+  if constexpr (VEC) {
+    for (int c = 8 * lane; c < p.rank; c += 512) {
+      float ov[8];
+      act_load<8>(ol + c, ov);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) a = dm_fma(wv[e], ov[e], a);
+      for (int r = 0; r < VR; ++r) {
+        if (v0 + r >= p.vdim) continue;
+        const uint4 y = c == 8 * lane ? first[r] : *reinterpret_cast<const uint4*>(w + (size_t)r * p.rank + c);
+        const float wv[8] = {dm_bf2f_lo(y.x), dm_bf2f_hi(y.x), dm_bf2f_lo(y.y), dm_bf2f_hi(y.y),
+                             dm_bf2f_lo(y.z), dm_bf2f_hi(y.z), dm_bf2f_lo(y.w), dm_bf2f_hi(y.w)};
+#pragma unroll
+        for (int e = 0; e < 8; ++e) a[r] = dm_fma(wv[e], ov[e], a[r]);
       }
-    } else {
-      for (int c = lane; c < p.rank; c += 64) a = dm_fma(dm_bf2f(w[(size_t)r * p.rank + c]), ol[c], a);
     }
-    a = dm_wave_sum<64>(a);
-    if (lane == 0) dst[v0 + r] = act_of<A>(a * gt);
+  } else {
+#pragma unroll
+    for (int r = 0; r < VR; ++r)
+      if (v0 + r < p.vdim)
+        for (int c = lane; c < p.rank; c += 64) a[r] = dm_fma(dm_bf2f(w[(size_t)r * p.rank + c]), ol[c], a[r]);
+  }
+#pragma unroll
+  for (int r = 0; r < VR; ++r) a[r] = dm_wave_sum<64>(a[r]);
+#pragma unroll
+  for (int r = 0; r < VR; ++r)
+    if (lane == r && v0 + r < p.vdim) dst[v0 + r] = act_of<A>(a[r] * gt);
+}
+
+typedef __bf16 l_bf16x8 __attribute__((ext_vector_type(8)));
+typedef float l_f32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t l_u32x4 __attribute__((ext_vector_type(4)));
+
+// The same blocks on the matrix cores, 32 rows a step: grid (blocks, groups of 16 HT heads, rows). Scores run
+// as S^T = C Q^T: wavefront (key half, channel half) takes sixteen rows of the step over half of their
+// channels for all heads of the group, straight from memory; softmax by eight threads a head; O^T += C^T P^T with
+// the rows turned in LDS, a wavefront every fourth tile of sixteen columns. NS: 32-channel steps of a
+// wavefront; rows of at most 64 NS values, latents of at most 512.
+constexpr int MK = 32, MV = MK + 8, MCT = 8;
+template <int NS, int HT>
+__global__ __launch_bounds__(NT, 1) void latent_mfma_kernel(LaArgs p, const bf16_t* q_hi, const bf16_t* q_lo, int t_base, float* part,
+                                                            float* ml) {
+  constexpr int HP = 16 * HT, TPH = NT / HP, KPT = MK / TPH;  // heads, threads a head, keys of such a thread
+  __shared__ __attribute__((aligned(16))) bf16_t Vt[MCT * 64][MV];
+  __shared__ __attribute__((aligned(16))) float sp[2][HP][MK + 4];
+  __shared__ __attribute__((aligned(16))) bf16_t Ph[HP][MV], Pl[HP][MV];
+  __shared__ float al[HP];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, lg = lane >> 4;
+  const int t = t_base + blockIdx.z, pos = p.offset + t, lo = first_visible(p, pos), nvis = pos - lo + 1;
+  const int KB = block_rows(nvis, -MK), u0 = blockIdx.x * KB;
+  if (u0 >= nvis) return;  // (every thread of the workgroup)
+  const int u1 = min(nvis, u0 + KB), h0 = blockIdx.y * HP, QS = p.rank + p.rot;
+  const int kt = wave & 1, s0 = (wave >> 1) * NS;
+  const bf16_t* cc = reinterpret_cast<const bf16_t*>(p.c_cache);
+  const bf16_t* rc = reinterpret_cast<const bf16_t*>(p.r_cache);
+  const l_u32x4 zero = {0, 0, 0, 0};
+  // rows as score operands, and pairs of rows to be turned
+  l_bf16x8 kf[NS];
+  l_u32x4 vr[4][2];
+  auto fetch = [&](int u) {
+    const size_t row = lo + min(u + 16 * kt + l16, nvis - 1);
+#pragma unroll
+    for (int i = 0; i < NS; ++i) {
+      const int d = 32 * (s0 + i) + 8 * lg;
+      const bf16_t* src = d < p.rank ? cc + row * p.rank + d : rc + row * p.rot + (d - p.rank);
+      kf[i] = __builtin_bit_cast(l_bf16x8, d < QS ? *reinterpret_cast<const l_u32x4*>(src) : zero);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int e = tid + NT * i, oct = (e & 3) + 4 * (e >> 6), pair = (e >> 2) & 15;
+#pragma unroll
+      for (int b = 0; b < 2; ++b) {
+        const size_t r = lo + min(u + 2 * pair + b, nvis - 1);
+        vr[i][b] = 8 * oct < p.rank ? *reinterpret_cast<const l_u32x4*>(cc + r * p.rank + 8 * oct) : zero;
+      }
+    }
+  };
+  fetch(u0);
+  l_bf16x8 qh[HT][NS], ql[HT][NS];
+#pragma unroll
+  for (int a = 0; a < HT; ++a) {
+    const size_t row = ((size_t)t * p.H + min(h0 + 16 * a + l16, p.H - 1)) * QS;
+#pragma unroll
+    for (int i = 0; i < NS; ++i) {
+      const int d = 32 * (s0 + i) + 8 * lg;
+      qh[a][i] = __builtin_bit_cast(l_bf16x8, d < QS ? *reinterpret_cast<const l_u32x4*>(q_hi + row + d) : zero);
+      ql[a][i] = __builtin_bit_cast(l_bf16x8, d < QS ? *reinterpret_cast<const l_u32x4*>(q_lo + row + d) : zero);
+    }
+  }
+  l_f32x4 acc[HT][MCT];
+#pragma unroll
+  for (int a = 0; a < HT; ++a)
+#pragma unroll
+    for (int c = 0; c < MCT; ++c) acc[a][c] = l_f32x4{0.f, 0.f, 0.f, 0.f};
+  const int hh = tid / TPH, sub = tid % TPH;  // a head's softmax
+  float m = -DM_INF, l = 0.f;
+  for (int u = u0; u < u1; u += MK) {
+    l_f32x4 sc[HT];
+#pragma unroll
+    for (int a = 0; a < HT; ++a) sc[a] = l_f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NS; ++i)
+#pragma unroll
+      for (int a = 0; a < HT; ++a) {
+        sc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], qh[a][i], sc[a], 0, 0, 0);
+        sc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], ql[a][i], sc[a], 0, 0, 0);
+      }
+    if (u != u0) __syncthreads();  // the step before is done with LDS
+#pragma unroll
+    for (int a = 0; a < HT; ++a) *reinterpret_cast<l_f32x4*>(&sp[wave >> 1][16 * a + l16][16 * kt + 4 * lg]) = sc[a];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int e = tid + NT * i, oct = (e & 3) + 4 * (e >> 6), pair = (e >> 2) & 15;
+      if (8 * oct < p.rank) {
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+          *reinterpret_cast<uint32_t*>(&Vt[8 * oct + 2 * w][2 * pair]) = __builtin_amdgcn_perm(vr[i][1][w], vr[i][0][w], 0x05040100u);
+          *reinterpret_cast<uint32_t*>(&Vt[8 * oct + 2 * w + 1][2 * pair]) = __builtin_amdgcn_perm(vr[i][1][w], vr[i][0][w], 0x07060302u);
+        }
+      }
+    }
+    if (u + MK < u1) fetch(u + MK);
+    __syncthreads();
+    {
+      float s[KPT], top = -DM_INF;
+#pragma unroll
+      for (int e = 0; e < KPT; ++e) {
+        const int key = KPT * sub + e;
+        s[e] = u + key < u1 ? sp[0][hh][key] + sp[1][hh][key] : -DM_INF;
+        top = __builtin_fmaxf(top, s[e]);
+      }
+#pragma unroll
+      for (int o = 1; o < TPH; o <<= 1) top = __builtin_fmaxf(top, __shfl_xor(top, o));
+      const float mn = __builtin_fmaxf(m, top), alpha = dm_exp(m - mn);
+      float sum = 0.f;
+#pragma unroll
+      for (int e = 0; e < KPT; ++e) {
+        s[e] = dm_exp(s[e] - mn);
+        sum += s[e];
+      }
+#pragma unroll
+      for (int o = 1; o < TPH; o <<= 1) sum += __shfl_xor(sum, o);
+      l = dm_fma(l, alpha, sum);
+      m = mn;
+#pragma unroll
+      for (int e = 0; e < KPT; e += 2) {
+        uint32_t hi, lo2;
+        split2(s[e], s[e + 1], hi, lo2);
+        *reinterpret_cast<uint32_t*>(&Ph[hh][KPT * sub + e]) = hi;
+        *reinterpret_cast<uint32_t*>(&Pl[hh][KPT * sub + e]) = lo2;
+      }
+      if (sub == 0) al[hh] = alpha;
+    }
+    __syncthreads();
+    l_bf16x8 ph[HT], pl[HT];
+#pragma unroll
+    for (int a = 0; a < HT; ++a) {
+      ph[a] = *reinterpret_cast<const l_bf16x8*>(&Ph[16 * a + l16][8 * lg]);
+      pl[a] = *reinterpret_cast<const l_bf16x8*>(&Pl[16 * a + l16][8 * lg]);
+      if (u != u0) {
+        const float x = al[16 * a + l16];
+#pragma unroll
+        for (int c = 0; c < MCT; ++c) acc[a][c] *= x;
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < MCT; ++c) {
+      const int tile = wave + 4 * c;
+      if (16 * tile >= p.rank) break;
+      const l_bf16x8 vf = *reinterpret_cast<const l_bf16x8*>(&Vt[16 * tile + l16][8 * lg]);
+#pragma unroll
+      for (int a = 0; a < HT; ++a) {
+        acc[a][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[a], acc[a][c], 0, 0, 0);
+        acc[a][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[a], acc[a][c], 0, 0, 0);
+      }
+    }
+  }
+  const int blocks = gridDim.x;
+#pragma unroll
+  for (int a = 0; a < HT; ++a) {
+    const int h = h0 + 16 * a + l16;
+    if (h >= p.H) continue;
+    float* dst = part + (((size_t)blockIdx.z * p.H + h) * blocks + blockIdx.x) * p.rank;
+#pragma unroll
+    for (int c = 0; c < MCT; ++c) {
+      const int col = 16 * (wave + 4 * c) + 4 * lg;
+      if (col < p.rank) *reinterpret_cast<l_f32x4*>(dst + col) = acc[a][c];
+    }
+  }
+  if (sub == 0 && h0 + hh < p.H) {
+    float* d = ml + (((size_t)blockIdx.z * p.H + h0 + hh) * blocks + blockIdx.x) * 2;
+    d[0] = m;
+    d[1] = l;
   }
 }
 
 template <typename A, int MR>
-int launch_query(ornith_ctx* ctx, const LaArgs& p, bool vec, float* qs) {
+int launch_query(ornith_ctx* ctx, const LaArgs& p, bool vec, const MappedQ& qs) {
   const size_t lds = (size_t)(DG * MR * QC + MR * p.dim) * 4;
   const dim3 grid((p.rank + QC - 1) / QC, p.H + (p.down ? 1 : 0), (p.T + MR - 1) / MR);
   ORN_REQUIRE(lds <= 65536, "latent_attn: heads of %d dimensions", p.dim);
@@ -369,10 +597,19 @@ int launch_query(ornith_ctx* ctx, const LaArgs& p, bool vec, float* qs) {
   return ORNITH_OK;
 }
 
+template <int NS>
+void launch_mfma(ornith_ctx* ctx, const LaArgs& p, const MappedQ& q, int blocks, int t, int n, float* part, float* ml) {
+  if (p.H <= 16)
+    hipLaunchKernelGGL((latent_mfma_kernel<NS, 1>), dim3(blocks, 1, n), dim3(NT), 0, ctx->stream, p, q.hi, q.lo, t, part, ml);
+  else
+    hipLaunchKernelGGL((latent_mfma_kernel<NS, 2>), dim3(blocks, (p.H + 31) / 32, n), dim3(NT), 0, ctx->stream, p, q.hi, q.lo, t, part, ml);
+}
+
 template <typename A>
 int run_decode(ornith_ctx* ctx, const LaArgs& p) {
   const bool vec = p.rank % 8 == 0 && p.rot % 8 == 0;
-  const int QS = p.rank + p.rot;
+  const int QS = p.rank + p.rot, NS = (QS + 63) / 64;
+  const bool mfma = sizeof(A) == 2 && vec && p.rank <= 64 * MCT && NS <= 9;
   const size_t q4 = (QS + 3) & ~3, cst = ((QS + 7) & ~7) + 16 / sizeof(A);
   int HG = 1;
   while (HG < 4 && HG < p.H) HG *= 2;
@@ -381,41 +618,55 @@ int run_decode(ornith_ctx* ctx, const LaArgs& p) {
   while (lds_of() > 65536 && KB > 8) KB /= 2;
   while (lds_of() > 65536 && HG > 1) HG /= 2;
   const size_t lds = lds_of();
-  ORN_REQUIRE(lds <= 160 * 1024, "latent_attn: rows of %d values do not fit a compute unit's local memory", QS);
-  if (lds > 65536) {
-    ORN_HIP(hipFuncSetAttribute((const void*)latent_decode_kernel<A, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-    ORN_HIP(hipFuncSetAttribute((const void*)latent_decode_kernel<A, false>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+  if (!mfma) {
+    ORN_REQUIRE(lds <= 160 * 1024, "latent_attn: rows of %d values do not fit a compute unit's local memory", QS);
+    if (lds > 65536) {
+      ORN_HIP(hipFuncSetAttribute((const void*)latent_decode_kernel<A, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+      ORN_HIP(hipFuncSetAttribute((const void*)latent_decode_kernel<A, false>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    }
   }
   const int last = p.offset + p.T - 1;
-  const int most = p.window > 0 && p.window < last + 1 ? p.window : last + 1, blocks = (most + KB - 1) / KB;
+  const int most = p.window > 0 && p.window < last + 1 ? p.window : last + 1;
+  const int unit = mfma ? -MK : KB, cut = (most + (mfma ? MK : KB) - 1) / (mfma ? MK : KB);
+  const int blocks = mfma && cut > kMaxBlocks ? kMaxBlocks : cut;  // of the query that has the most
   // rows in groups whose partial results stay below 256 MB
   const size_t per = (size_t)p.H * blocks * (p.rank + 2) * 4, fit = (size_t(256) << 20) / per;
   int group = p.T < 32768 ? p.T : 32768;
   if ((size_t)group > fit) group = fit < 1 ? 1 : (int)fit;
   const size_t nq = (size_t)p.T * p.H * QS;
   void* base = nullptr;
-  int rc = ornith_scratch(ctx, nq * 4 + per * group + 4 * 256, &base);
+  int rc = ornith_scratch(ctx, nq * 4 + per * group + 8 * 256, &base);
   if (rc) return rc;
   ScratchCursor sc(base);
-  float* qs = sc.take<float>(nq);
+  MappedQ qs{};
+  if (mfma) {
+    qs.hi = sc.take<bf16_t>(nq);
+    qs.lo = sc.take<bf16_t>(nq);
+  } else {
+    qs.f = sc.take<float>(nq);
+  }
   float* part = sc.take<float>((size_t)group * p.H * blocks * p.rank);
   float* ml = sc.take<float>((size_t)group * p.H * blocks * 2);
   rc = p.T == 1 ? launch_query<A, 1>(ctx, p, vec, qs) : p.T == 2 ? launch_query<A, 2>(ctx, p, vec, qs) : launch_query<A, 4>(ctx, p, vec, qs);
   if (rc) return rc;
-  const size_t olds = (size_t)(((p.rank + 7) & ~7) + blocks) * 4;
-  ORN_REQUIRE(olds <= 65536, "latent_attn: %d blocks of %d rows in sight", blocks, KB);
+  const int cols = vec ? p.rank / 4 : p.rank, G = cols < NT ? NT / cols : 1;
+  const size_t olds = (size_t)(((p.rank + 7) & ~7) + ((blocks + 3) & ~3) + G * p.rank) * 4;
+  ORN_REQUIRE(olds <= 65536, "latent_attn: %d blocks of rows in sight, rank %d", blocks, p.rank);
   for (int t = 0; t < p.T; t += group) {
     const int n = p.T - t < group ? p.T - t : group;
     const dim3 grid(blocks, (p.H + HG - 1) / HG, n), ogrid((p.vdim + VB - 1) / VB, p.H, n);
-    if (vec) {
-      hipLaunchKernelGGL((latent_decode_kernel<A, true>), grid, dim3(NT), lds, ctx->stream, p, qs, KB, HG, t, part, ml);
-      ORN_LAUNCH_CHECK("latent_decode_kernel");
-      hipLaunchKernelGGL((latent_out_kernel<A, true>), ogrid, dim3(NT), olds, ctx->stream, p, KB, t, blocks, part, ml);
+    if (mfma) {
+      if (NS <= 3) launch_mfma<3>(ctx, p, qs, blocks, t, n, part, ml);
+      else if (NS <= 6) launch_mfma<6>(ctx, p, qs, blocks, t, n, part, ml);
+      else launch_mfma<9>(ctx, p, qs, blocks, t, n, part, ml);
+    } else if (vec) {
+      hipLaunchKernelGGL((latent_decode_kernel<A, true>), grid, dim3(NT), lds, ctx->stream, p, qs.f, KB, HG, t, part, ml);
     } else {
-      hipLaunchKernelGGL((latent_decode_kernel<A, false>), grid, dim3(NT), lds, ctx->stream, p, qs, KB, HG, t, part, ml);
-      ORN_LAUNCH_CHECK("latent_decode_kernel");
-      hipLaunchKernelGGL((latent_out_kernel<A, false>), ogrid, dim3(NT), olds, ctx->stream, p, KB, t, blocks, part, ml);
+      hipLaunchKernelGGL((latent_decode_kernel<A, false>), grid, dim3(NT), lds, ctx->stream, p, qs.f, KB, HG, t, part, ml);
     }
+    ORN_LAUNCH_CHECK("latent attention over a block");
+    if (vec) hipLaunchKernelGGL((latent_out_kernel<A, true>), ogrid, dim3(NT), olds, ctx->stream, p, unit, t, blocks, part, ml);
+    else hipLaunchKernelGGL((latent_out_kernel<A, false>), ogrid, dim3(NT), olds, ctx->stream, p, unit, t, blocks, part, ml);
     ORN_LAUNCH_CHECK("latent_out_kernel");
   }
   return ORNITH_OK;
@@ -426,10 +677,6 @@ __global__ __launch_bounds__(NT) void latent_append_kernel(LaArgs p) {
   __shared__ float red[4];
   append_row<bf16_t>(p, blockIdx.x, red);
 }
-
-typedef __bf16 l_bf16x8 __attribute__((ext_vector_type(8)));
-typedef float l_f32x4 __attribute__((ext_vector_type(4)));
-typedef uint32_t l_u32x4 __attribute__((ext_vector_type(4)));
 
 constexpr int BKV = 64, LV = BKV + 8;
 

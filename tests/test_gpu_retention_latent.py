@@ -253,7 +253,8 @@ class Latent:
             b.free()
         return got
 
-    def want(self, x, size=None, sink=True, commit=True):
+    def want(self, x, size=None, sink=True, commit=True, rows=None):
+        """rows: only the call's last ones are worked out (the others come back as zeros)."""
         p, rnd = self.p, _bf if self.act else (lambda a: a)
         H, d, dv, rank = p["H"], p["dim"], p["vdim"], p["rank"]
         src, size = self.of or self, self.size if size is None else size
@@ -264,6 +265,9 @@ class Latent:
             if self.of is None:
                 C.append(rnd(R.norm_plain(dn[:rank], self.norm, 1e-5)).astype(np.float64))
                 K.append(rnd(R.turn(dn[rank:], i, self.freqs, self.gain, False)).astype(np.float64))
+            if rows is not None and t < T - rows:
+                out.append(np.zeros((H, dv)))
+                continue
             js = [j for j in range(i + 1) if R.visible(i, j, size, 0)]
             c, kr, row = np.array([C[j] for j in js]), np.array([K[j] for j in js]), []
             for h in range(H):
@@ -282,7 +286,7 @@ class Latent:
 
 
 SHAPES = [  # H, dim, rot, vdim, rank, window
-    (2, 16, 8, 16, 24, 5), (4, 32, 32, 64, 64, 64), (6, 24, 8, 40, 40, 65), (3, 72, 24, 136, 104, 100), (2, 128, 64, 256, 192, 33),
+    (20, 16, 8, 16, 24, 5), (35, 8, 8, 8, 256, 90), (17, 24, 64, 40, 512, 50), (2, 16, 8, 16, 24, 5), (4, 32, 32, 64, 64, 64), (6, 24, 8, 40, 40, 65), (3, 72, 24, 136, 104, 100), (2, 128, 64, 256, 192, 33),
     (3, 14, 6, 9, 23, 20), (1, 7, 2, 3, 5, 1), (5, 40, 16, 48, 520, 0), (2, 192, 64, 128, 136, 1000), (7, 8, 8, 8, 8, 130)]
 
 
@@ -297,6 +301,25 @@ def test_latent_portions(orn, ctx, act, shape):
     for T in (1, 2, 40, 1, 64, 33, 3, 100, 1, 7):
         x = la.inputs(rng, T)
         _close(la.step(x), la.want(x), act, (shape, T), slack=6.0 if act == 0 else 3.0)
+    la.close()
+
+
+@pytest.mark.parametrize("shape", [(18, 16, 8, 24, 320, 0), (3, 24, 8, 16, 40, 2300), (2, 16, 16, 24, 544, 2050)])
+def test_latent_far_rows(orn, ctx, shape):
+    """Thousands of rows in sight, where a decoded row's blocks grow longer; one early row stands out."""
+    H, dim, rot, vdim, rank, size = shape
+    la, rng, n = Latent(orn, ctx, 1, *shape, cap=3000), np.random.default_rng(rank), 2600
+    x = la.inputs(rng, n)
+    spot = n - 2000
+    c = R.norm_plain(x["down"][spot, :rank].astype(np.float64), la.norm, 1e-5)
+    tail = la.inputs(rng, 4)
+    for q in (x["q"][-1], tail["q"][0], tail["q"][3]):
+        for h in range(H):
+            key = la.uk[dim * h:dim * h + dim] @ c
+            q[h, :dim] = _bf(key * 12.0 / (key @ key) / la.scale)
+    _close(la.step(x)[-3:], la.want(x, rows=3)[-3:], 1, "prompt", slack=3.0)
+    for part in ({k: a[:1] for k, a in tail.items()}, {k: a[1:] for k, a in tail.items()}):
+        _close(la.step(part), la.want(part), 1, "decoded", slack=3.0)
     la.close()
 
 
