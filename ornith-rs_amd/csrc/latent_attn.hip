@@ -95,10 +95,12 @@ __device__ __forceinline__ void append_row(const LaArgs& p, int t, float* red) {
 // ---- decode widths ---------------------------------------------------------------------
 constexpr int QC = 128, DG = NT / 16;  // latent columns of a query workgroup; its groups of head dimensions
 
-// Queries over the cached rows, [T][H][rank + rot], scaled: fp32 or as two bf16 parts.
+// Queries over the cached rows, [T][H][rank + rot, padded with zeros to `stride`], scaled: fp32 or as two
+// bf16 parts.
 struct MappedQ {
   float* f;
   bf16_t *hi, *lo;
+  int stride;
   __device__ __forceinline__ void put(size_t at, float v) const {
     if (f) {
       f[at] = v;
@@ -122,7 +124,7 @@ __global__ __launch_bounds__(NT) void latent_query_kernel(LaArgs p, MappedQ qs) 
       for (int m = 0; m < n; ++m) append_row<A>(p, m0 + m, red);
     return;  // (the whole workgroup)
   }
-  const int qd = p.dim + p.rot, QS = p.rank + p.rot;
+  const int qd = p.dim + p.rot, QS = qs.stride;
   const int cg = tid & 15, dg = tid >> 4, r0 = blockIdx.x * QC + 8 * cg;
   const bf16_t* w = p.uk + (size_t)h * p.dim * p.rank + r0;
   const int in = min(8, p.rank - r0);  // columns of this thread that exist
@@ -154,6 +156,9 @@ __global__ __launch_bounds__(NT) void latent_query_kernel(LaArgs p, MappedQ qs) 
       qs.put(at, u * p.scale);
       qs.put(at + 1, v * p.scale);
     }
+  const int pad = QS - p.rank - p.rot;
+  if (blockIdx.x == 0)
+    for (int i = tid; i < n * pad; i += NT) qs.put(((size_t)(m0 + i / pad) * p.H + h) * QS + p.rank + p.rot + i % pad, 0.f);
   __syncthreads();
   float acc[MR][8];
 #pragma unroll
@@ -306,10 +311,10 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(LaArgs p, const float
 }
 
 // grid (value tiles, H, rows): the blocks of a query joined with weights e^(m_b - M), groups of threads taking
-// every G-th block, then VB values of the head, a wavefront VB / 4 of them.
-constexpr int VB = 32;
+// every G-th block, then VB values of the head, a wavefront VB / 8 of them.
+constexpr int VB = 32, ONT = 512;
 template <typename A, bool VEC>
-__global__ __launch_bounds__(NT) void latent_out_kernel(LaArgs p, int unit, int t_base, int stride, const float* part, const float* ml) {
+__global__ __launch_bounds__(ONT) void latent_out_kernel(LaArgs p, int unit, int t_base, int stride, const float* part, const float* ml) {
   extern __shared__ __attribute__((aligned(16))) char lds_raw[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int h = blockIdx.y, t = t_base + blockIdx.z, pos = p.offset + t;
@@ -320,7 +325,7 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(LaArgs p, int unit, int 
   float* red = wb + ((stride + 3) & ~3);          // [G][rank]
   const size_t base = ((size_t)blockIdx.z * p.H + h) * stride;
   // this wavefront's weights, asked for ahead
-  constexpr int VR = VB / 4;
+  constexpr int VR = VB / (ONT / 64);
   const int v0 = blockIdx.x * VB + wave * VR;
   const bf16_t* w = p.uv + ((size_t)h * p.vdim + v0) * p.rank;
   uint4 first[VR];
@@ -331,7 +336,7 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(LaArgs p, int unit, int 
   }
   // four columns a thread, and the first blocks of its group, asked for before the weights are made
   constexpr int W = VEC ? 4 : 1, U = 8;
-  const int cols = p.rank / W, G = max(1, NT / cols), g = tid / cols, c0 = tid % cols;
+  const int cols = p.rank / W, G = max(1, ONT / cols), g = tid / cols, c0 = tid % cols;
   const float* src = part + base * p.rank;
   float x[U][W];
   auto fetch = [&](int b0, int c) {
@@ -360,7 +365,7 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(LaArgs p, int unit, int 
     for (int b = lane; b < nb; b += 64) wb[b] = wb[b] / L;
   }
   __syncthreads();
-  for (int c = c0; c < cols; c += NT) {  // (one round unless a row is longer than the workgroup)
+  for (int c = c0; c < cols; c += ONT) {  // (one round unless a row is longer than the workgroup)
     if (g < G) {
       float o[W];
 #pragma unroll
@@ -380,7 +385,7 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(LaArgs p, int unit, int 
     }
   }
   __syncthreads();
-  for (int c = tid; c < rp; c += NT) {
+  for (int c = tid; c < rp; c += ONT) {
     float o = 0.f;
     if (c < p.rank)
       for (int i = 0; i < G; ++i) o += red[i * p.rank + c];
@@ -423,160 +428,115 @@ typedef __bf16 l_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float l_f32x4 __attribute__((ext_vector_type(4)));
 typedef uint32_t l_u32x4 __attribute__((ext_vector_type(4)));
 
-// The same blocks on the matrix cores, 32 rows a step: grid (blocks, groups of 16 HT heads, rows). Scores run
-// as S^T = C Q^T: wavefront (key half, channel half) takes sixteen rows of the step over half of their
-// channels for all heads of the group, straight from memory; softmax by eight threads a head; O^T += C^T P^T with
-// the rows turned in LDS, a wavefront every fourth tile of sixteen columns. NS: 32-channel steps of a
-// wavefront; rows of at most 64 NS values, latents of at most 512.
-constexpr int MK = 32, MV = MK + 8, MCT = 8;
-template <int NS, int HT>
+// The same blocks on the matrix cores, 32 rows a step: grid (blocks, groups of 16 heads, rows). Scores run as
+// S^T = C Q^T: wavefront (key half, channel half) takes sixteen rows of the step over half of their channels,
+// straight from memory; softmax by sixteen threads a head; O^T += C^T P^T with the rows turned in LDS, a
+// wavefront every fourth tile of sixteen columns. NS: 32-channel steps of a wavefront, CT: its column tiles;
+// rows of at most 64 NS values (queries padded to that with zeros), latents of at most 64 CT. Loads past a
+// row's end fetch its last piece again: they meet zeros, or columns nobody stores. The loop's body is the same
+// from the first step on (weights start at e^-inf) and not unrolled: at these widths a launch waits for its
+// instructions as much as for its data.
+constexpr int MK = 32, MV = MK + 8, MH = 16;
+template <int NS, int CT>
 __global__ __launch_bounds__(NT, 1) void latent_mfma_kernel(LaArgs p, const bf16_t* q_hi, const bf16_t* q_lo, int t_base, float* part,
                                                             float* ml) {
-  constexpr int HP = 16 * HT, TPH = NT / HP, KPT = MK / TPH;  // heads, threads a head, keys of such a thread
-  __shared__ __attribute__((aligned(16))) bf16_t Vt[MCT * 64][MV];
-  __shared__ __attribute__((aligned(16))) float sp[2][HP][MK + 4];
-  __shared__ __attribute__((aligned(16))) bf16_t Ph[HP][MV], Pl[HP][MV];
-  __shared__ float al[HP];
+  constexpr int TPH = NT / MH, KPT = MK / TPH, VI = (CT + 1) / 2;  // threads a head, keys of such a thread
+  static_assert(KPT == 2, "a thread's weights are a pair");
+  __shared__ __attribute__((aligned(16))) bf16_t Vt[VI * 128][MV];
+  __shared__ __attribute__((aligned(16))) float sp[2][MH][MK + 4];
+  __shared__ __attribute__((aligned(16))) bf16_t Ph[MH][MV], Pl[MH][MV];
+  __shared__ float al[MH];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, lg = lane >> 4;
   const int t = t_base + blockIdx.z, pos = p.offset + t, lo = first_visible(p, pos), nvis = pos - lo + 1;
   const int KB = block_rows(nvis, -MK), u0 = blockIdx.x * KB;
   if (u0 >= nvis) return;  // (every thread of the workgroup)
-  const int u1 = min(nvis, u0 + KB), h0 = blockIdx.y * HP, QS = p.rank + p.rot;
+  const int u1 = min(nvis, u0 + KB), h0 = blockIdx.y * MH, QS = p.rank + p.rot;
   const int kt = wave & 1, s0 = (wave >> 1) * NS;
   const bf16_t* cc = reinterpret_cast<const bf16_t*>(p.c_cache);
   const bf16_t* rc = reinterpret_cast<const bf16_t*>(p.r_cache);
-  const l_u32x4 zero = {0, 0, 0, 0};
   // rows as score operands, and pairs of rows to be turned
   l_bf16x8 kf[NS];
-  l_u32x4 vr[4][2];
+  l_u32x4 vr[VI][2];
+  const int pair = (tid >> 2) & 15, oct0 = (tid & 3) + 4 * (tid >> 6);
   auto fetch = [&](int u) {
     const size_t row = lo + min(u + 16 * kt + l16, nvis - 1);
+    const bf16_t *ck = cc + row * p.rank, *rk = rc + row * p.rot - p.rank;
 #pragma unroll
     for (int i = 0; i < NS; ++i) {
-      const int d = 32 * (s0 + i) + 8 * lg;
-      const bf16_t* src = d < p.rank ? cc + row * p.rank + d : rc + row * p.rot + (d - p.rank);
-      kf[i] = __builtin_bit_cast(l_bf16x8, d < QS ? *reinterpret_cast<const l_u32x4*>(src) : zero);
+      const int d = min(32 * (s0 + i) + 8 * lg, QS - 8);
+      kf[i] = __builtin_bit_cast(l_bf16x8, *reinterpret_cast<const l_u32x4*>((d < p.rank ? ck : rk) + d));
     }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int e = tid + NT * i, oct = (e & 3) + 4 * (e >> 6), pair = (e >> 2) & 15;
+    for (int b = 0; b < 2; ++b) {
+      const bf16_t* cv = cc + (size_t)(lo + min(u + 2 * pair + b, nvis - 1)) * p.rank;
 #pragma unroll
-      for (int b = 0; b < 2; ++b) {
-        const size_t r = lo + min(u + 2 * pair + b, nvis - 1);
-        vr[i][b] = 8 * oct < p.rank ? *reinterpret_cast<const l_u32x4*>(cc + r * p.rank + 8 * oct) : zero;
-      }
+      for (int i = 0; i < VI; ++i) vr[i][b] = *reinterpret_cast<const l_u32x4*>(cv + min(8 * (oct0 + 16 * i), p.rank - 8));
     }
   };
   fetch(u0);
-  l_bf16x8 qh[HT][NS], ql[HT][NS];
+  l_bf16x8 qh[NS], ql[NS];
+  const size_t q_at = ((size_t)t * p.H + min(h0 + l16, p.H - 1)) * (64 * NS) + 32 * s0 + 8 * lg;
 #pragma unroll
-  for (int a = 0; a < HT; ++a) {
-    const size_t row = ((size_t)t * p.H + min(h0 + 16 * a + l16, p.H - 1)) * QS;
-#pragma unroll
-    for (int i = 0; i < NS; ++i) {
-      const int d = 32 * (s0 + i) + 8 * lg;
-      qh[a][i] = __builtin_bit_cast(l_bf16x8, d < QS ? *reinterpret_cast<const l_u32x4*>(q_hi + row + d) : zero);
-      ql[a][i] = __builtin_bit_cast(l_bf16x8, d < QS ? *reinterpret_cast<const l_u32x4*>(q_lo + row + d) : zero);
-    }
+  for (int i = 0; i < NS; ++i) {
+    qh[i] = *reinterpret_cast<const l_bf16x8*>(q_hi + q_at + 32 * i);
+    ql[i] = *reinterpret_cast<const l_bf16x8*>(q_lo + q_at + 32 * i);
   }
-  l_f32x4 acc[HT][MCT];
+  l_f32x4 acc[CT];
 #pragma unroll
-  for (int a = 0; a < HT; ++a)
-#pragma unroll
-    for (int c = 0; c < MCT; ++c) acc[a][c] = l_f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int c = 0; c < CT; ++c) acc[c] = l_f32x4{0.f, 0.f, 0.f, 0.f};
   const int hh = tid / TPH, sub = tid % TPH;  // a head's softmax
   float m = -DM_INF, l = 0.f;
+#pragma clang loop unroll(disable)
   for (int u = u0; u < u1; u += MK) {
-    l_f32x4 sc[HT];
+    l_f32x4 sc[2] = {l_f32x4{0.f, 0.f, 0.f, 0.f}, l_f32x4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
-    for (int a = 0; a < HT; ++a) sc[a] = l_f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < NS; ++i) {
+      sc[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], qh[i], sc[0], 0, 0, 0);
+      sc[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], ql[i], sc[1], 0, 0, 0);
+    }
+    __syncthreads();  // the step before is done with LDS
+    *reinterpret_cast<l_f32x4*>(&sp[wave >> 1][l16][16 * kt + 4 * lg]) = sc[0] + sc[1];
 #pragma unroll
-    for (int i = 0; i < NS; ++i)
+    for (int i = 0; i < VI; ++i) {
+      bf16_t* v = &Vt[8 * (oct0 + 16 * i)][2 * pair];
 #pragma unroll
-      for (int a = 0; a < HT; ++a) {
-        sc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], qh[a][i], sc[a], 0, 0, 0);
-        sc[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], ql[a][i], sc[a], 0, 0, 0);
-      }
-    if (u != u0) __syncthreads();  // the step before is done with LDS
-#pragma unroll
-    for (int a = 0; a < HT; ++a) *reinterpret_cast<l_f32x4*>(&sp[wave >> 1][16 * a + l16][16 * kt + 4 * lg]) = sc[a];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int e = tid + NT * i, oct = (e & 3) + 4 * (e >> 6), pair = (e >> 2) & 15;
-      if (8 * oct < p.rank) {
-#pragma unroll
-        for (int w = 0; w < 4; ++w) {
-          *reinterpret_cast<uint32_t*>(&Vt[8 * oct + 2 * w][2 * pair]) = __builtin_amdgcn_perm(vr[i][1][w], vr[i][0][w], 0x05040100u);
-          *reinterpret_cast<uint32_t*>(&Vt[8 * oct + 2 * w + 1][2 * pair]) = __builtin_amdgcn_perm(vr[i][1][w], vr[i][0][w], 0x07060302u);
-        }
+      for (int w = 0; w < 4; ++w) {
+        *reinterpret_cast<uint32_t*>(v + 2 * w * MV) = __builtin_amdgcn_perm(vr[i][1][w], vr[i][0][w], 0x05040100u);
+        *reinterpret_cast<uint32_t*>(v + (2 * w + 1) * MV) = __builtin_amdgcn_perm(vr[i][1][w], vr[i][0][w], 0x07060302u);
       }
     }
     if (u + MK < u1) fetch(u + MK);
     __syncthreads();
     {
-      float s[KPT], top = -DM_INF;
-#pragma unroll
-      for (int e = 0; e < KPT; ++e) {
-        const int key = KPT * sub + e;
-        s[e] = u + key < u1 ? sp[0][hh][key] + sp[1][hh][key] : -DM_INF;
-        top = __builtin_fmaxf(top, s[e]);
-      }
-#pragma unroll
-      for (int o = 1; o < TPH; o <<= 1) top = __builtin_fmaxf(top, __shfl_xor(top, o));
-      const float mn = __builtin_fmaxf(m, top), alpha = dm_exp(m - mn);
-      float sum = 0.f;
-#pragma unroll
-      for (int e = 0; e < KPT; ++e) {
-        s[e] = dm_exp(s[e] - mn);
-        sum += s[e];
-      }
-#pragma unroll
-      for (int o = 1; o < TPH; o <<= 1) sum += __shfl_xor(sum, o);
-      l = dm_fma(l, alpha, sum);
+      const float2 a = *reinterpret_cast<const float2*>(&sp[0][hh][KPT * sub]), b = *reinterpret_cast<const float2*>(&sp[1][hh][KPT * sub]);
+      const float x = u + KPT * sub < u1 ? a.x + b.x : -DM_INF, y = u + KPT * sub + 1 < u1 ? a.y + b.y : -DM_INF;
+      const float mn = __builtin_fmaxf(m, dm_wave_max<TPH>(__builtin_fmaxf(x, y)));
+      const float alpha = dm_exp(m - mn), ex = dm_exp(x - mn), ey = dm_exp(y - mn);
+      l = dm_fma(l, alpha, dm_wave_sum<TPH>(ex + ey));
       m = mn;
-#pragma unroll
-      for (int e = 0; e < KPT; e += 2) {
-        uint32_t hi, lo2;
-        split2(s[e], s[e + 1], hi, lo2);
-        *reinterpret_cast<uint32_t*>(&Ph[hh][KPT * sub + e]) = hi;
-        *reinterpret_cast<uint32_t*>(&Pl[hh][KPT * sub + e]) = lo2;
-      }
+      uint32_t hi, lo2;
+      split2(ex, ey, hi, lo2);
+      *reinterpret_cast<uint32_t*>(&Ph[hh][KPT * sub]) = hi;
+      *reinterpret_cast<uint32_t*>(&Pl[hh][KPT * sub]) = lo2;
       if (sub == 0) al[hh] = alpha;
     }
     __syncthreads();
-    l_bf16x8 ph[HT], pl[HT];
+    const l_bf16x8 ph = *reinterpret_cast<const l_bf16x8*>(&Ph[l16][8 * lg]), pl = *reinterpret_cast<const l_bf16x8*>(&Pl[l16][8 * lg]);
+    const float x = al[l16];
 #pragma unroll
-    for (int a = 0; a < HT; ++a) {
-      ph[a] = *reinterpret_cast<const l_bf16x8*>(&Ph[16 * a + l16][8 * lg]);
-      pl[a] = *reinterpret_cast<const l_bf16x8*>(&Pl[16 * a + l16][8 * lg]);
-      if (u != u0) {
-        const float x = al[16 * a + l16];
-#pragma unroll
-        for (int c = 0; c < MCT; ++c) acc[a][c] *= x;
-      }
-    }
-#pragma unroll
-    for (int c = 0; c < MCT; ++c) {
-      const int tile = wave + 4 * c;
-      if (16 * tile >= p.rank) break;
-      const l_bf16x8 vf = *reinterpret_cast<const l_bf16x8*>(&Vt[16 * tile + l16][8 * lg]);
-#pragma unroll
-      for (int a = 0; a < HT; ++a) {
-        acc[a][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[a], acc[a][c], 0, 0, 0);
-        acc[a][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[a], acc[a][c], 0, 0, 0);
-      }
+    for (int c = 0; c < CT; ++c) {
+      const l_bf16x8 vf = *reinterpret_cast<const l_bf16x8*>(&Vt[16 * (wave + 4 * c) + l16][8 * lg]);
+      acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph, acc[c] * x, 0, 0, 0);
+      acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, acc[c], 0, 0, 0);
     }
   }
-  const int blocks = gridDim.x;
-#pragma unroll
-  for (int a = 0; a < HT; ++a) {
-    const int h = h0 + 16 * a + l16;
-    if (h >= p.H) continue;
+  const int blocks = gridDim.x, h = h0 + l16;
+  if (h < p.H) {
     float* dst = part + (((size_t)blockIdx.z * p.H + h) * blocks + blockIdx.x) * p.rank;
 #pragma unroll
-    for (int c = 0; c < MCT; ++c) {
+    for (int c = 0; c < CT; ++c) {
       const int col = 16 * (wave + 4 * c) + 4 * lg;
-      if (col < p.rank) *reinterpret_cast<l_f32x4*>(dst + col) = acc[a][c];
+      if (col < p.rank) *reinterpret_cast<l_f32x4*>(dst + col) = acc[c];
     }
   }
   if (sub == 0 && h0 + hh < p.H) {
@@ -597,19 +557,17 @@ int launch_query(ornith_ctx* ctx, const LaArgs& p, bool vec, const MappedQ& qs) 
   return ORNITH_OK;
 }
 
-template <int NS>
+template <int NS, int CT>
 void launch_mfma(ornith_ctx* ctx, const LaArgs& p, const MappedQ& q, int blocks, int t, int n, float* part, float* ml) {
-  if (p.H <= 16)
-    hipLaunchKernelGGL((latent_mfma_kernel<NS, 1>), dim3(blocks, 1, n), dim3(NT), 0, ctx->stream, p, q.hi, q.lo, t, part, ml);
-  else
-    hipLaunchKernelGGL((latent_mfma_kernel<NS, 2>), dim3(blocks, (p.H + 31) / 32, n), dim3(NT), 0, ctx->stream, p, q.hi, q.lo, t, part, ml);
+  hipLaunchKernelGGL((latent_mfma_kernel<NS, CT>), dim3(blocks, (p.H + MH - 1) / MH, n), dim3(NT), 0, ctx->stream, p, q.hi, q.lo, t,
+                     part, ml);
 }
 
 template <typename A>
 int run_decode(ornith_ctx* ctx, const LaArgs& p) {
   const bool vec = p.rank % 8 == 0 && p.rot % 8 == 0;
   const int QS = p.rank + p.rot, NS = (QS + 63) / 64;
-  const bool mfma = sizeof(A) == 2 && vec && p.rank <= 64 * MCT && NS <= 9;
+  const bool mfma = sizeof(A) == 2 && vec && p.rank <= 512 && NS <= 9;
   const size_t q4 = (QS + 3) & ~3, cst = ((QS + 7) & ~7) + 16 / sizeof(A);
   int HG = 1;
   while (HG < 4 && HG < p.H) HG *= 2;
@@ -633,12 +591,13 @@ int run_decode(ornith_ctx* ctx, const LaArgs& p) {
   const size_t per = (size_t)p.H * blocks * (p.rank + 2) * 4, fit = (size_t(256) << 20) / per;
   int group = p.T < 32768 ? p.T : 32768;
   if ((size_t)group > fit) group = fit < 1 ? 1 : (int)fit;
-  const size_t nq = (size_t)p.T * p.H * QS;
+  MappedQ qs{};
+  qs.stride = mfma ? 64 * (NS <= 3 ? 3 : NS <= 6 ? 6 : 9) : QS;
+  const size_t nq = (size_t)p.T * p.H * qs.stride;
   void* base = nullptr;
   int rc = ornith_scratch(ctx, nq * 4 + per * group + 8 * 256, &base);
   if (rc) return rc;
   ScratchCursor sc(base);
-  MappedQ qs{};
   if (mfma) {
     qs.hi = sc.take<bf16_t>(nq);
     qs.lo = sc.take<bf16_t>(nq);
@@ -649,24 +608,24 @@ int run_decode(ornith_ctx* ctx, const LaArgs& p) {
   float* ml = sc.take<float>((size_t)group * p.H * blocks * 2);
   rc = p.T == 1 ? launch_query<A, 1>(ctx, p, vec, qs) : p.T == 2 ? launch_query<A, 2>(ctx, p, vec, qs) : launch_query<A, 4>(ctx, p, vec, qs);
   if (rc) return rc;
-  const int cols = vec ? p.rank / 4 : p.rank, G = cols < NT ? NT / cols : 1;
+  const int cols = vec ? p.rank / 4 : p.rank, G = cols < ONT ? ONT / cols : 1;
   const size_t olds = (size_t)(((p.rank + 7) & ~7) + ((blocks + 3) & ~3) + G * p.rank) * 4;
   ORN_REQUIRE(olds <= 65536, "latent_attn: %d blocks of rows in sight, rank %d", blocks, p.rank);
   for (int t = 0; t < p.T; t += group) {
     const int n = p.T - t < group ? p.T - t : group;
     const dim3 grid(blocks, (p.H + HG - 1) / HG, n), ogrid((p.vdim + VB - 1) / VB, p.H, n);
     if (mfma) {
-      if (NS <= 3) launch_mfma<3>(ctx, p, qs, blocks, t, n, part, ml);
-      else if (NS <= 6) launch_mfma<6>(ctx, p, qs, blocks, t, n, part, ml);
-      else launch_mfma<9>(ctx, p, qs, blocks, t, n, part, ml);
+      if (NS <= 3) launch_mfma<3, 3>(ctx, p, qs, blocks, t, n, part, ml);
+      else if (NS <= 6) launch_mfma<6, 6>(ctx, p, qs, blocks, t, n, part, ml);
+      else launch_mfma<9, 8>(ctx, p, qs, blocks, t, n, part, ml);
     } else if (vec) {
       hipLaunchKernelGGL((latent_decode_kernel<A, true>), grid, dim3(NT), lds, ctx->stream, p, qs.f, KB, HG, t, part, ml);
     } else {
       hipLaunchKernelGGL((latent_decode_kernel<A, false>), grid, dim3(NT), lds, ctx->stream, p, qs.f, KB, HG, t, part, ml);
     }
     ORN_LAUNCH_CHECK("latent attention over a block");
-    if (vec) hipLaunchKernelGGL((latent_out_kernel<A, true>), ogrid, dim3(NT), olds, ctx->stream, p, unit, t, blocks, part, ml);
-    else hipLaunchKernelGGL((latent_out_kernel<A, false>), ogrid, dim3(NT), olds, ctx->stream, p, unit, t, blocks, part, ml);
+    if (vec) hipLaunchKernelGGL((latent_out_kernel<A, true>), ogrid, dim3(ONT), olds, ctx->stream, p, unit, t, blocks, part, ml);
+    else hipLaunchKernelGGL((latent_out_kernel<A, false>), ogrid, dim3(ONT), olds, ctx->stream, p, unit, t, blocks, part, ml);
     ORN_LAUNCH_CHECK("latent_out_kernel");
   }
   return ORNITH_OK;
