@@ -312,7 +312,7 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(LaArgs p, const float
 
 // grid (value tiles, H, rows): the blocks of a query joined with weights e^(m_b - M), groups of threads taking
 // every G-th block, then VB values of the head, a wavefront VB / 8 of them.
-constexpr int VB = 32, ONT = 512;
+constexpr int VB = 64, ONT = 512;
 template <typename A, bool VEC>
 __global__ __launch_bounds__(ONT) void latent_out_kernel(LaArgs p, int unit, int t_base, int stride, const float* part, const float* ml) {
   extern __shared__ __attribute__((aligned(16))) char lds_raw[];
