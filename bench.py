@@ -1096,6 +1096,15 @@ def ranavik_kernels(orn, ctx, np, width, only=None):
                   for a in (orn.PAIR_SILU, orn.PAIR_GELU)]
             pair(f"decode gate, up, T = {T}", row("norm + gate, up + silu", us[0], 2 * ff * W * 2),
                  row("x", us[1], 2 * ff * W * 2, peer=True), "norm + gate, up + gelu")
+            ws = [dense(o, W, n) for o in ret_in]
+            ys, wn2 = [ctx.alloc(T * o * 4) for o in ret_in], dev((W,), std=0.1)
+            duo = [(orn.dense_call(B, x, T, W, [w[i] for w in ws], ys, [ACT] * 4, pre=orn.PRE_NORM, norm_w=wn2),
+                    orn.dense_call(B, x, T, W, [wg[i], wu[i]], [act, None], [0, 0], pre=orn.PRE_NORM, norm_w=wn, pair_act=orn.PAIR_SILU))
+                   for i in range(n)]
+            us = [t_of(calls(orn.dense_rows_duo, duo)), t_of(lambda i: [orn.dense_rows(ctx, c) for c in duo[i % n]])]
+            nb = (2 * ff + sum(ret_in)) * W * 2
+            pair(f"decode projections beside gate, up, T = {T}", row("norms + q, k, v, g and gate, up + silu", us[0], nb),
+                 row("x", us[1], nb, peer=True), "the same in two launches")
             us = [t_of(calls(orn.dense_rows, [orn.dense_call(B, act, T, ff, [wd[i % n]], [xs], [ADD], add_scale=m) for i in range(n)]))
                   for m in (0.7, 1.0)]
             pair(f"decode down, T = {T}", row("down + sum", us[0], ff * W * 2), row("x", us[1], ff * W * 2, peer=True), "down + sum")

@@ -445,6 +445,9 @@ typedef struct ornith_dense_call {
   float soft_cap; /* > 0: sums stored (not added) become soft_cap tanh(sum / soft_cap) */
 } ornith_dense_call;
 ORNITH_API int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* call);
+/* Two calls over the same rows, each with a norm of its own in front (ORNITH_PRE_NORM): plain outputs and a
+ * gated pair. One launch below the gemm_rows option, with the bits of two; neither may write what the other reads. */
+ORNITH_API int ornith_dense_rows_duo(ornith_ctx* ctx, const ornith_dense_call* plain, const ornith_dense_call* pair);
 /* the prologues alone */
 ORNITH_API int ornith_norm_rows(ornith_ctx* ctx, const float* d_x, const void* d_w, float w_offset, int rows, int n,
                                 float eps, int act, void* d_out);

@@ -90,16 +90,17 @@ __device__ __forceinline__ void group_rows(const RowsArgs& p, int g, const bf16_
   }
 }
 
+// workgroup wg of `wgs` that share the call's groups of output rows
 template <typename A, int MR, int PRE, bool PAIR, bool VEC>
-__global__ __launch_bounds__(NT) void dense_rows_kernel(RowsArgs p, int groups) {
+__device__ __forceinline__ void dense_rows_body(const RowsArgs& p, int groups, int wg, int wgs) {
   extern __shared__ __attribute__((aligned(16))) char lds_raw[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int K = p.K, K8 = (K + 7) / 8, Kp = K8 * 8;
   A* xs = reinterpret_cast<A*>(lds_raw);                              // [MR][Kp]
   float* aux = reinterpret_cast<float*>(lds_raw + (size_t)MR * Kp * sizeof(A));
   const int m0 = blockIdx.y * MR;
-  const int stride = gridDim.x * (NT / 64), nb = (K8 + 64 * NU - 1) / (64 * NU);
-  int g = blockIdx.x * (NT / 64) + wave;
+  const int stride = wgs * (NT / 64), nb = (K8 + 64 * NU - 1) / (64 * NU);
+  int g = wg * (NT / 64) + wave;
 
   uint4 cur[NR][NU], nxt[NR][NU];
   const bf16_t* wr[NR];
@@ -337,6 +338,19 @@ __global__ __launch_bounds__(NT) void dense_rows_kernel(RowsArgs p, int groups) 
   }
 }
 
+template <typename A, int MR, int PRE, bool PAIR, bool VEC>
+__global__ __launch_bounds__(NT) void dense_rows_kernel(RowsArgs p, int groups) {
+  dense_rows_body<A, MR, PRE, PAIR, VEC>(p, groups, blockIdx.x, gridDim.x);
+}
+
+// Two calls that read the same rows, each through its norm: plain outputs, and a gated pair. The first
+// `split` workgroups take the first.
+template <typename A, int MR, bool VEC>
+__global__ __launch_bounds__(NT) void dense_rows_duo_kernel(RowsArgs a, RowsArgs b, int groups_a, int groups_b, int split) {
+  if ((int)blockIdx.x < split) dense_rows_body<A, MR, ORNITH_PRE_NORM, false, VEC>(a, groups_a, blockIdx.x, split);
+  else dense_rows_body<A, MR, ORNITH_PRE_NORM, true, VEC>(b, groups_b, blockIdx.x - split, gridDim.x - split);
+}
+
 size_t rows_lds(int MR, int K, size_t es, int pre, int head, bool vec) {
   const size_t Kp = (size_t)(K + 7) / 8 * 8;
   size_t aux = 16;
@@ -372,11 +386,49 @@ int launch_rows_pre(ornith_ctx* ctx, const RowsArgs& p, int groups, size_t lds, 
   }
 }
 
+int row_groups(const RowsArgs& p, bool pair) {
+  if (pair) return p.O[0];
+  int groups = 0;
+  for (int i = 0; i < p.n; ++i) groups += (p.O[i] + NR - 1) / NR;
+  return groups;
+}
+
+template <typename A, int MR, bool VEC>
+int launch_duo_kernel(ornith_ctx* ctx, const RowsArgs& a, const RowsArgs& b, size_t lds) {
+  if (lds > 65536)
+    ORN_HIP(hipFuncSetAttribute((const void*)dense_rows_duo_kernel<A, MR, VEC>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+  constexpr int PER = NT / 64;
+  const int ga = row_groups(a, false), gb = row_groups(b, true), cap = 3 * (ctx->compute_units > 0 ? ctx->compute_units : 256);
+  int wa = (ga + PER - 1) / PER, wb = (gb + PER - 1) / PER;
+  if (wa + wb > cap) {  // shares by their work; a group is two rows of either
+    wa = (int)((long)cap * ga / (ga + gb));
+    wa = wa < 1 ? 1 : wa > cap - 1 ? cap - 1 : wa;
+    wb = cap - wa;
+  }
+  hipLaunchKernelGGL((dense_rows_duo_kernel<A, MR, VEC>), dim3(wa + wb, (a.M + MR - 1) / MR), dim3(NT), lds, ctx->stream, a, b, ga, gb,
+                     wa);
+  ORN_LAUNCH_CHECK("dense_rows_duo_kernel");
+  return ORNITH_OK;
+}
+
+template <typename A>
+int launch_duo(ornith_ctx* ctx, const RowsArgs& a, const RowsArgs& b) {
+  const bool vec = a.K % 8 == 0;
+  int MR = !vec ? 1 : a.M >= 3 ? 4 : a.M;
+  while (MR > 1 && rows_lds(MR, a.K, sizeof(A), ORNITH_PRE_NORM, 0, vec) > 65536) MR /= 2;
+  const size_t lds = rows_lds(MR, a.K, sizeof(A), ORNITH_PRE_NORM, 0, vec);
+  ORN_REQUIRE(lds <= 160 * 1024, "dense_rows: rows of %d values do not fit a compute unit's local memory", a.K);
+  if (!vec) return launch_duo_kernel<A, 1, false>(ctx, a, b, lds);
+  switch (MR) {
+    case 1: return launch_duo_kernel<A, 1, true>(ctx, a, b, lds);
+    case 2: return launch_duo_kernel<A, 2, true>(ctx, a, b, lds);
+    default: return launch_duo_kernel<A, 4, true>(ctx, a, b, lds);
+  }
+}
+
 template <typename A>
 int launch_rows(ornith_ctx* ctx, const RowsArgs& p, int pre, bool pair) {
-  int groups = 0;
-  if (pair) groups = p.O[0];
-  else for (int i = 0; i < p.n; ++i) groups += (p.O[i] + NR - 1) / NR;
+  const int groups = row_groups(p, pair);
   const bool vec = p.K % 8 == 0 && (pre != ORNITH_PRE_HEADS || p.head % 4 == 0);
   int MR = !vec ? 1 : p.M >= 3 ? 4 : p.M;
   while (MR > 1 && rows_lds(MR, p.K, sizeof(A), pre, p.head, vec) > 65536) MR /= 2;
@@ -789,7 +841,7 @@ int ornith_round_bf16(ornith_ctx* ctx, const float* d_x, size_t n, void* d_out) 
   return ORNITH_OK;
 }
 
-int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* c) {
+static int rows_args(ornith_ctx* ctx, const ornith_dense_call* c, RowsArgs& p) {
   ORN_REQUIRE(ctx && c && c->d_x, "dense_rows: null argument");
   ORN_REQUIRE(c->act == ORNITH_BF16 || c->act == ORNITH_F32, "dense_rows: activation type %d", c->act);
   ORN_REQUIRE(c->M >= 1 && c->K >= 1 && c->n >= 1 && c->n <= kSegs, "dense_rows: M=%d K=%d n=%d", c->M, c->K, c->n);
@@ -797,7 +849,7 @@ int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* c) {
   ORN_REQUIRE(c->pre != ORNITH_PRE_NORM || c->d_norm_w, "dense_rows: norm weight missing");
   ORN_REQUIRE(c->pre != ORNITH_PRE_HEADS || (c->d_gate && c->head_dim >= 1 && c->K % c->head_dim == 0 && !c->pair_act),
               "dense_rows: heads of %d in rows of %d", c->head_dim, c->K);
-  RowsArgs p{};
+  p = RowsArgs{};
   p.x = c->d_x;
   p.wn = (const bf16_t*)c->d_norm_w;
   p.gate = c->d_gate;
@@ -825,13 +877,34 @@ int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* c) {
   }
   ORN_REQUIRE(!c->pair_act || (c->n == 2 && p.O[0] == p.O[1]), "dense_rows: a gated pair is two matrices of one size");
   ORN_REQUIRE(c->K % 8 != 0 || (((uintptr_t)c->d_x | (uintptr_t)c->d_gate) & 15) == 0, "dense_rows: operands must be 16-byte aligned");
-  const bool gemm = c->act == ORNITH_BF16 && c->M >= kPrefillRows && c->K % 8 == 0;
-  if (!gemm)
+  return ORNITH_OK;
+}
+
+static bool runs_as_gemm(const ornith_dense_call* c) { return c->act == ORNITH_BF16 && c->M >= kPrefillRows && c->K % 8 == 0; }
+
+int ornith_dense_rows_duo(ornith_ctx* ctx, const ornith_dense_call* a, const ornith_dense_call* b) {
+  RowsArgs p, q;
+  int rc = rows_args(ctx, a, p);
+  if (!rc) rc = rows_args(ctx, b, q);
+  if (rc) return rc;
+  ORN_REQUIRE(a->act == b->act && a->M == b->M && a->K == b->K && a->pre == ORNITH_PRE_NORM && b->pre == ORNITH_PRE_NORM &&
+                  !a->pair_act && b->pair_act,
+              "dense_rows_duo: normed rows [%d,%d] for plain outputs beside normed rows [%d,%d] for a gated pair", a->M, a->K, b->M, b->K);
+  if (!runs_as_gemm(a)) return a->act == ORNITH_F32 ? launch_duo<float>(ctx, p, q) : launch_duo<bf16_t>(ctx, p, q);
+  rc = ornith_dense_rows(ctx, a);
+  return rc ? rc : ornith_dense_rows(ctx, b);
+}
+
+int ornith_dense_rows(ornith_ctx* ctx, const ornith_dense_call* c) {
+  RowsArgs p;
+  int rc = rows_args(ctx, c, p);
+  if (rc) return rc;
+  if (!runs_as_gemm(c))
     return c->act == ORNITH_F32 ? launch_rows<float>(ctx, p, c->pre, c->pair_act != ORNITH_PAIR_NONE)
                                 : launch_rows<bf16_t>(ctx, p, c->pre, c->pair_act != ORNITH_PAIR_NONE);
   if (c->pre != ORNITH_PRE_NONE) {
     ORN_REQUIRE(c->d_rows, "dense_rows: %d rows need the buffer for the rows the matrices read", c->M);
-    const int rc = c->pre == ORNITH_PRE_NORM
+    rc = c->pre == ORNITH_PRE_NORM
                        ? ornith_norm_rows(ctx, (const float*)c->d_x, c->d_norm_w, c->w_offset, c->M, c->K, c->eps, c->act, c->d_rows)
                        : ornith_head_norm_gate(ctx, (const float*)c->d_x, c->d_norm_w, c->d_gate, c->gate_act, c->M,
                                                c->K / c->head_dim, c->head_dim, c->eps, c->act, c->d_rows);

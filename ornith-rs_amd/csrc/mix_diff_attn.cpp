@@ -21,16 +21,21 @@ void keeps(const ornith_model* m, int layer, CacheSpec& out) {
   out.v_row = (size_t)a.vdim * es;
 }
 
+StackCall input(const StackStep& st, int layer) {
+  const Layer& L = st.m->layers[layer];
+  const DiffAttnLayer& a = L.dattn;
+  const StepBufs& s = st.s;
+  StackCall in = mixer_input(st, L);
+  in.to(a.q, s.q).to(a.k, s.k).to(a.v, s.v).to(a.g, s.s0, ORNITH_OUT_F32);
+  return in;
+}
+
 int mix(const StackStep& st, int layer) {
   const ornith_model* m = st.m;
   const Layer& L = m->layers[layer];
   const LayerCache& lc = st.cc->layers[layer];
   const DiffAttnLayer& a = L.dattn;
   const StepBufs& s = st.s;
-  StackCall in = mixer_input(st, L);
-  in.to(a.q, s.q).to(a.k, s.k).to(a.v, s.v).to(a.g, s.s0, ORNITH_OUT_F32);
-  const int rc = ornith_dense_rows(m->ctx, &in);
-  if (rc) return rc;
   const RopeTable* rot = a.rope >= 0 ? &m->ropes[a.rope] : nullptr;
   ornith_diff_attn_call c{};
   c.act = m->act_dtype;
@@ -62,12 +67,12 @@ int mix(const StackStep& st, int layer) {
   return ornith_diff_attn(m->ctx, &c);
 }
 
-int close(const StackStep& st, int layer) {
+StackCall output(const StackStep& st, int layer) {
   const DiffAttnLayer& a = st.m->layers[layer].dattn;
   StackCall out = StackCall(st, a.heads * a.vdim, st.s.att).to(a.o, st.s.x, ORNITH_OUT_ADD);
-  return ornith_dense_rows(st.m->ctx, &out);
+  return out;
 }
 
 }  // namespace
 
-StackMixer kDiffAttnMixer = {needs, keeps, mix, close};
+StackMixer kDiffAttnMixer = {needs, keeps, input, mix, output};

@@ -20,6 +20,16 @@ void keeps(const ornith_model* m, int layer, CacheSpec& out) {
   out.v_row = (size_t)a.rot_dim * es;
 }
 
+StackCall input(const StackStep& st, int layer) {
+  const Layer& L = st.m->layers[layer];
+  const LatentLayer& a = L.latent;
+  const StepBufs& s = st.s;
+  StackCall in = mixer_input(st, L);
+  in.to(a.q, s.q).to(a.g, s.s0, ORNITH_OUT_F32);
+  if (a.kv_layer == layer) in.to(a.down, s.o, ORNITH_OUT_F32);
+  return in;
+}
+
 int mix(const StackStep& st, int layer) {
   const ornith_model* m = st.m;
   const Layer& L = m->layers[layer];
@@ -27,11 +37,6 @@ int mix(const StackStep& st, int layer) {
   const LayerCache& lc = st.cc->layers[a.kv_layer];
   const StepBufs& s = st.s;
   const bool own = a.kv_layer == layer;
-  StackCall in = mixer_input(st, L);
-  in.to(a.q, s.q).to(a.g, s.s0, ORNITH_OUT_F32);
-  if (own) in.to(a.down, s.o, ORNITH_OUT_F32);
-  const int rc = ornith_dense_rows(m->ctx, &in);
-  if (rc) return rc;
   const RopeTable* rot = a.rope >= 0 ? &m->ropes[a.rope] : nullptr;
   ornith_latent_attn_call c{};
   c.act = m->act_dtype;
@@ -62,12 +67,12 @@ int mix(const StackStep& st, int layer) {
   return ornith_latent_attn(m->ctx, &c);
 }
 
-int close(const StackStep& st, int layer) {
+StackCall output(const StackStep& st, int layer) {
   const LatentLayer& a = st.m->layers[layer].latent;
   StackCall out = StackCall(st, a.heads * a.vdim, st.s.att).to(a.o, st.s.x, ORNITH_OUT_ADD);
-  return ornith_dense_rows(st.m->ctx, &out);
+  return out;
 }
 
 }  // namespace
 
-StackMixer kLatentMixer = {needs, keeps, mix, close};
+StackMixer kLatentMixer = {needs, keeps, input, mix, output};

@@ -17,15 +17,20 @@ void keeps(const ornith_model* m, int layer, CacheSpec& out) {
   out.state = ornith_mlstm_state_floats(a.heads, a.dim, a.vdim) * 4;
 }
 
+StackCall input(const StackStep& st, int layer) {
+  const Layer& L = st.m->layers[layer];
+  const MlstmLayer& a = L.mlstm;
+  const StepBufs& s = st.s;
+  StackCall in = mixer_input(st, L);
+  in.to(a.q, s.q).to(a.k, s.k).to(a.v, s.v).to(a.g, s.g).to(a.i, s.s0, ORNITH_OUT_F32).to(a.f, s.s1, ORNITH_OUT_F32);
+  return in;
+}
+
 int mix(const StackStep& st, int layer) {
   const Layer& L = st.m->layers[layer];
   const LayerCache& lc = st.cc->layers[layer];
   const MlstmLayer& a = L.mlstm;
   const StepBufs& s = st.s;
-  StackCall in = mixer_input(st, L);
-  in.to(a.q, s.q).to(a.k, s.k).to(a.v, s.v).to(a.g, s.g).to(a.i, s.s0, ORNITH_OUT_F32).to(a.f, s.s1, ORNITH_OUT_F32);
-  const int rc = ornith_dense_rows(st.m->ctx, &in);
-  if (rc) return rc;
   ornith_mlstm_call c{};
   c.act = st.m->act_dtype;
   c.d_q = s.q;
@@ -49,13 +54,13 @@ int mix(const StackStep& st, int layer) {
   return ornith_mlstm(st.m->ctx, &c);
 }
 
-int close(const StackStep& st, int layer) {
+StackCall output(const StackStep& st, int layer) {
   const MlstmLayer& a = st.m->layers[layer].mlstm;
   StackCall out = StackCall(st, a.heads * a.vdim, st.s.o).heads(a.norm, st.s.g, ORNITH_GATE_SIGMOID, a.vdim);
   out.to(a.o, st.s.x, ORNITH_OUT_ADD);
-  return ornith_dense_rows(st.m->ctx, &out);
+  return out;
 }
 
 }  // namespace
 
-StackMixer kMlstmMixer = {needs, keeps, mix, close};
+StackMixer kMlstmMixer = {needs, keeps, input, mix, output};

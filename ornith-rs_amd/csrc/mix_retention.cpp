@@ -16,16 +16,21 @@ void keeps(const ornith_model* m, int layer, CacheSpec& out) {
   out.state = ornith_retention_state_floats(a.heads, a.dim, a.vdim) * 4;
 }
 
+StackCall input(const StackStep& st, int layer) {
+  const Layer& L = st.m->layers[layer];
+  const RetentionLayer& a = L.ret;
+  const StepBufs& s = st.s;
+  StackCall in = mixer_input(st, L);
+  in.to(a.q, s.q).to(a.k, s.k).to(a.v, s.v).to(a.g, s.g);
+  return in;
+}
+
 int mix(const StackStep& st, int layer) {
   const ornith_model* m = st.m;
   const Layer& L = m->layers[layer];
   const LayerCache& lc = st.cc->layers[layer];
   const RetentionLayer& a = L.ret;
   const StepBufs& s = st.s;
-  StackCall in = mixer_input(st, L);
-  in.to(a.q, s.q).to(a.k, s.k).to(a.v, s.v).to(a.g, s.g);
-  const int rc = ornith_dense_rows(m->ctx, &in);
-  if (rc) return rc;
   const RopeTable* rot = a.rope >= 0 ? &m->ropes[a.rope] : nullptr;
   ornith_retention_call c{};
   c.act = m->act_dtype;
@@ -51,13 +56,13 @@ int mix(const StackStep& st, int layer) {
   return ornith_retention(m->ctx, &c);
 }
 
-int close(const StackStep& st, int layer) {
+StackCall output(const StackStep& st, int layer) {
   const RetentionLayer& a = st.m->layers[layer].ret;
   StackCall out = StackCall(st, a.heads * a.vdim, st.s.o).heads(nullptr, st.s.g, ORNITH_GATE_SILU, a.vdim);
   out.to(a.o, st.s.x, ORNITH_OUT_ADD);
-  return ornith_dense_rows(st.m->ctx, &out);
+  return out;
 }
 
 }  // namespace
 
-StackMixer kRetentionMixer = {needs, keeps, mix, close};
+StackMixer kRetentionMixer = {needs, keeps, input, mix, output};

@@ -1,14 +1,14 @@
 // The step of a layer-list model: embedding (and its norm), the layers, the closing norm. The residual
 // stream and everything a layer adds to it are fp32; activations are bf16, or fp32 for a model opened in
 // 32-bit. A layer is norm -> mixer -> sum, norm -> feed-forward -> sum, or both halves side by side on the
-// same stream: then the second norm's projections run before the mixer's sum reaches the stream.
+// same stream: then the projections behind both norms come first, in one launch at decode widths.
 //
 // Launches of a layer at decode widths: a recurrent mixer is three (projections with the norm in their
 // head; the memory's step; the output projection with the heads' norm and gate in its head and the
 // residual sum in its tail), differential attention three (four past one block of keys), latent attention
 // five, a feed-forward two (gate and up with the norm in the head and the activation in the tail; down with
-// the residual sum). At prefill widths the rows a norm makes are a launch of their own and the projections
-// are matrix-core GEMMs with the same tails.
+// the residual sum), of which only the second is a launch of its own beside a mixer. At prefill widths the
+// rows a norm makes are a launch of their own and the projections are matrix-core GEMMs with the same tails.
 #include "stack.h"
 
 #define TRY(e)         \
@@ -45,16 +45,17 @@ StepBufs carve(const ornith_model* m, void* base, int R, size_t* total = nullptr
   return s;
 }
 
-int ff_in(const StackStep& st, const Layer& L) {
+int run(const StackStep& st, const StackCall& c) { return ornith_dense_rows(st.m->ctx, &c); }
+
+StackCall ff_in(const StackStep& st, const Layer& L) {
   StackCall c = StackCall(st, st.m->cfg.hidden_size, st.s.x).norm(L.post_ln, st.m->style.norm_offset);
   c.to(L.dense.gate, st.s.act).to(L.dense.up, nullptr);
   c.pair_act = st.m->style.ff_act;
-  return ornith_dense_rows(st.m->ctx, &c);
+  return c;
 }
 
-int ff_out(const StackStep& st, const Layer& L) {
-  StackCall c = StackCall(st, L.dense.ff, st.s.act).to(L.dense.down, st.s.x, ORNITH_OUT_ADD);
-  return ornith_dense_rows(st.m->ctx, &c);
+StackCall ff_out(const StackStep& st, const Layer& L) {
+  return StackCall(st, L.dense.ff, st.s.act).to(L.dense.down, st.s.x, ORNITH_OUT_ADD);
 }
 
 }  // namespace
@@ -75,11 +76,17 @@ int stack_forward(ornith_model* m, ornith_caches* cc, const uint32_t* d_tokens, 
   for (int i = 0; i < (int)m->layers.size(); ++i) {
     const Layer& L = m->layers[i];
     const bool ff = L.ffn == FF_DENSE;
+    const StackCall in = L.ops->input(st, i);
+    if (ff && y.side_by_side) {
+      const StackCall up = ff_in(st, L);
+      TRY(ornith_dense_rows_duo(m->ctx, &in, &up));
+    } else {
+      TRY(run(st, in));
+    }
     TRY(L.ops->mix(st, i));
-    if (ff && y.side_by_side) TRY(ff_in(st, L));
-    TRY(L.ops->close(st, i));
-    if (ff && !y.side_by_side) TRY(ff_in(st, L));
-    if (ff) TRY(ff_out(st, L));
+    TRY(run(st, L.ops->output(st, i)));
+    if (ff && !y.side_by_side) TRY(run(st, ff_in(st, L)));
+    if (ff) TRY(run(st, ff_out(st, L)));
   }
   return ornith_norm_rows(m->ctx, st.s.x, m->final_norm, y.norm_offset, T, m->cfg.hidden_size, m->cfg.rms_norm_eps,
                           m->act_dtype, d_hidden);

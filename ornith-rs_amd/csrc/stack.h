@@ -25,17 +25,6 @@ struct StackStep {
   bool capture;
 };
 
-// A kind of mixer.
-struct StackMixer {
-  void (*needs)(const Layer& L, StepNeeds& n);
-  void (*keeps)(const ornith_model* m, int layer, CacheSpec& out);
-  // everything up to the rows the output projection reads; the stream is only read
-  int (*mix)(const StackStep& st, int layer);
-  // the output projection, added to the stream
-  int (*close)(const StackStep& st, int layer);
-};
-extern StackMixer kMlstmMixer, kDiffAttnMixer, kRetentionMixer, kLatentMixer;
-
 // a projection call of the step's rows
 struct StackCall : ornith_dense_call {
   StackCall(const StackStep& st, int K_, const void* x) {
@@ -73,6 +62,19 @@ struct StackCall : ornith_dense_call {
 inline StackCall mixer_input(const StackStep& st, const Layer& L) {
   return StackCall(st, st.m->cfg.hidden_size, st.s.x).norm(L.input_ln, st.m->style.norm_offset);
 }
+
+// A kind of mixer.
+struct StackMixer {
+  void (*needs)(const Layer& L, StepNeeds& n);
+  void (*keeps)(const ornith_model* m, int layer, CacheSpec& out);
+  // the projections of the normed stream
+  StackCall (*input)(const StackStep& st, int layer);
+  // from those to the rows the output projection reads; the stream stays as it is
+  int (*mix)(const StackStep& st, int layer);
+  // the output projection, added to the stream
+  StackCall (*output)(const StackStep& st, int layer);
+};
+extern StackMixer kMlstmMixer, kDiffAttnMixer, kRetentionMixer, kLatentMixer;
 
 size_t stack_step_bytes(const ornith_model* m, int rows);
 int stack_forward(ornith_model* m, ornith_caches* cc, const uint32_t* d_tokens, int T, bool capture, void* d_hidden);

@@ -737,6 +737,11 @@ def dense_rows(ctx, *a, **kw):
     _check(lib().ornith_dense_rows(ctx.h, C.byref(c)), "dense_rows")
 
 
+def dense_rows_duo(ctx, calls):
+    """ornith_dense_rows_duo on two calls made earlier: plain outputs, a gated pair."""
+    _check(lib().ornith_dense_rows_duo(ctx.h, C.byref(calls[0]), C.byref(calls[1])), "dense_rows_duo")
+
+
 def mlstm_state_floats(H, dim, vdim):
     f = lib().ornith_mlstm_state_floats
     f.restype = C.c_size_t

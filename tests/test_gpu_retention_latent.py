@@ -45,6 +45,38 @@ def test_dense_rows_forms(orn, ctx, act, M, K, head):
         b.free()
 
 
+@pytest.mark.parametrize("act", [0, 1])
+@pytest.mark.parametrize("M,K,O,ff", [(1, 96, (33, 8), 40), (2, 2048, (1500, 700, 4), 3000), (5, 264, (64,), 9), (3, 91, (17, 5), 12),
+                                      (40, 128, (96, 24), 200)])
+def test_two_calls_in_one_launch(orn, ctx, act, M, K, O, ff):
+    """Projections behind one norm and a gated pair behind another over the same rows: the bits of two calls,
+    whether the workgroups suffice for every group of rows or have to be shared out."""
+    rng = np.random.default_rng(M + K)
+    lin = lambda o: orn.Linear.dense(ctx, util.f32_to_bf16(rng.standard_normal((o, K)).astype(np.float32) * K ** -0.5))
+    plain, pair = [lin(o) for o in O], [lin(ff) for _ in range(2)]
+    x, wn = ctx.to_device(rng.standard_normal((M, K)).astype(np.float32)), [ctx.to_device(util.f32_to_bf16(
+        1 + 0.3 * rng.standard_normal(K).astype(np.float32))) for _ in range(2)]
+    rows, adt = ctx.alloc(M * K * 4), orn.F32 if act == 0 else orn.BF16
+    got = []
+    for one in (False, True):
+        ys, up = [ctx.alloc(M * o * 4).zero() for o in O], ctx.alloc(M * ff * 4).zero()
+        calls = [orn.dense_call(adt, x, M, K, plain, ys, [orn.OUT_F32] * len(O), pre=orn.PRE_NORM, norm_w=wn[0], rows=rows),
+                 orn.dense_call(adt, x, M, K, pair, [up, None], [0, 0], pre=orn.PRE_NORM, norm_w=wn[1], pair_act=orn.PAIR_SILU,
+                                rows=rows)]
+        if one:
+            orn.dense_rows_duo(ctx, calls)
+        else:
+            for c in calls:
+                orn.dense_rows(ctx, c)
+        got.append([y.download(np.float32, (M, o)) for y, o in zip(ys, O)] + [_get(up, (M, ff), act)])
+        assert all(np.any(a) for a in got[-1])
+        for b in ys + [up]:
+            b.free()
+    assert all(np.array_equal(a, b) for a, b in zip(*got))
+    for b in plain + pair + wn + [x, rows]:
+        b.free()
+
+
 @pytest.mark.parametrize("n", [64, 91, 1000, 8200])
 def test_embedded_rows_are_normed(orn, ctx, n):
     rng = np.random.default_rng(n)
